@@ -3,6 +3,9 @@
 //     S_t = diag(w_t) S_(t-1) - (a_t * n_t) (n_t^T S_(t-1)) + k_t v_t^T,     o_t = S_t^T r_t,     n = k / sqrt(|k|^2 + tiny)
 // with both terms reading the old state.  S float [d, vd] per (slot, head).  Everything but the projections themselves
 // (decay, removal rate, unit key, state, outputs) is float whatever the activation type T is.
+// The gated delta rule is its relative with one decay g and one write strength beta per head,
+//     S' = g S,   u = beta (v - S'^T k),   S <- S' + k u^T,   o = S^T q,     k, q unit vectors behind short convolutions:
+// the same scan with two arrays and two scalars per token instead of five arrays.
 #include "ragged_common.h"
 
 using namespace ragged;
@@ -52,6 +55,91 @@ extern "C" int ragged_delta_gates(const void* P, int64_t ldp, int r0, int k0, in
 }
 
 // ---------------------------------------------------------------------------------------------------------------
+// The gated delta rule's inputs from this step's projections (columns 0 .. of P: q [G d] | k [G d] | v [H vd], all of them
+// behind a short causal convolution and silu): qf = unit(q) * d^(-1/2), kf = unit(k), float [rows, G d] each, with unit(u) =
+// u / sqrt(|u|^2 + tiny); vo of type T [rows, H vd]; gb float [rows, H, 2] = (exp(-arate softplus(a + dt bias)), sigmoid(b)).
+// The inputs before this step come from `state` [slots, taps - 1, C]; `write_state` (every sequence brings exactly one row)
+// also shifts it.  One wavefront per (row, item): 2 G unit vectors, blocks of 256 value channels, the gates.
+struct GatedDeltaArgs {
+  const void* P;
+  int64_t ldp;
+  const float* cw;       // [C, taps], C = 2 G d + H vd
+  int taps;
+  void* state;
+  int b0, a0;            // columns of P: write strengths and step logits, H each
+  const float* arate;    // [H]
+  const float* dt_bias;  // [H]
+  float tiny;
+  float* qf;
+  float* kf;
+  void* vo;
+  float* gb;
+  int H, G, d, vd, write_state;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a, int items, Batch bt) {
+  extern __shared__ float smem[];
+  const int lane = threadIdx.x & 63;
+  float* buf = smem + (threadIdx.x >> 6) * a.d;
+  const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (id >= (int64_t)bt.T * items) return;
+  const int t = (int)(id / items), it = (int)(id % items);
+  const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
+  const T* P = (const T*)a.P;
+  const int C = 2 * a.G * a.d + a.H * a.vd, keep = a.taps - 1;
+  T* hist = (T*)a.state + (int64_t)slot * keep * C;
+  auto conv = [&](int ch) {                                  // silu of the convolved channel; with write_state shifts its history
+    float u = 0.f;
+    for (int j = 0; j < a.taps; ++j) {
+      const int back = keep - j, pp = pos - back;
+      T raw = from_f<T>(0.f);
+      if (pp >= past) raw = P[(int64_t)(t - back) * a.ldp + ch];
+      else if (pp >= 0) raw = hist[(int64_t)(pp - past + keep) * C + ch];
+      u += a.cw[(int64_t)ch * a.taps + j] * to_f(raw);
+      if (a.write_state && j > 0) hist[(int64_t)(j - 1) * C + ch] = raw;      // (row j - 1 has been read)
+    }
+    return u / (1.0f + expf(-u));
+  };
+  if (it < 2 * a.G) {
+    const bool isq = it < a.G;
+    float ss = 0.f;
+    for (int c = lane; c < a.d; c += 64) { const float v = conv(it * a.d + c); buf[c] = v; ss += v * v; }
+    float f = 1.0f / sqrtf(wave_sum(ss) + a.tiny);
+    if (isq) f *= 1.0f / sqrtf((float)a.d);
+    float* o = (isq ? a.qf : a.kf) + ((int64_t)t * a.G + (isq ? it : it - a.G)) * a.d;
+    for (int c = lane; c < a.d; c += 64) o[c] = buf[c] * f;          // (what this lane itself has stored)
+  } else if (it < items - 1) {
+    const int c0 = (it - 2 * a.G) * 256;
+    for (int c = c0 + lane; c < c0 + 256 && c < a.H * a.vd; c += 64)
+      ((T*)a.vo)[(int64_t)t * a.H * a.vd + c] = from_f<T>(conv(2 * a.G * a.d + c));
+  } else {
+    const T* row = P + (int64_t)t * a.ldp;
+    for (int h = lane; h < a.H; h += 64) {
+      const float z = to_f(row[a.a0 + h]) + a.dt_bias[h];
+      const float sp = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+      float* o = a.gb + ((int64_t)t * a.H + h) * 2;
+      o[0] = expf(-a.arate[h] * sp);
+      o[1] = 1.0f / (1.0f + expf(-to_f(row[a.b0 + h])));
+    }
+  }
+}
+
+extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hipStream_t st) {
+  if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.d <= 0 || a.d > 1024 || a.vd <= 0 || a.taps < 1 || a.taps > 16) return -1;
+  if (!a.P || !a.cw || (a.taps > 1 && !a.state) || !a.arate || !a.dt_bias || !a.qf || !a.kf || !a.vo || !a.gb) return -1;
+  const int C = 2 * a.G * a.d + a.H * a.vd;
+  if (a.b0 < C || a.a0 < C || a.ldp < a.b0 + a.H || a.ldp < a.a0 + a.H || (a.write_state && bt.B != bt.T)) return -1;
+  if (a.taps == 1) a.write_state = 0;
+  const int items = 2 * a.G + (a.H * a.vd + 255) / 256 + 1;
+  const int64_t blocks = ((int64_t)bt.T * items + 3) / 4;
+  if (blocks > 0x7fffffff) return -1;
+  RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((gated_delta_prep_kernel<T>), dim3((unsigned)blocks), dim3(256), 4 * a.d * sizeof(float), st,
+                                            a, items, bt))
+  return RAGGED_LAUNCH_OK();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
 // The scan.  Columns of S are independent: column j follows s <- w * s - b (n . s) + k v_j, and its output is r . s.
 // A wavefront owns 64 / R columns; R neighbouring lanes share a column, lane r of them holds rows 32 r .. 32 r + 31 in
 // registers (R = d / 32 rounded up to a power of two; rows past d carry w = 1 and zeros and stay zero), so a token costs
@@ -61,19 +149,22 @@ extern "C" int ragged_delta_gates(const void* P, int64_t ldp, int r0, int k0, in
 // while the previous block is scanned (register look-ahead, two LDS buffers) and read back as 16-byte broadcasts.
 // Grid: (column blocks, heads, sequences).  `values` = 0: v is taken as 0 (the state only decays and forgets: from an
 // identity state this yields a chunk's transition matrix).
+// NA = 5: the generalised rule.  NA = 2: the gated rule; the arrays are q and k of G heads (head h reads head h / (H / G)),
+// `gb` holds every token's decay and write strength per head, and the four arrays of the general form shrink to k and scalars:
+// w = g, n = k, b = beta g k, and k v takes the factor beta.
 constexpr int DL_DR = 32;
 constexpr int DL_SEG = DL_DR + 4;   // LDS floats per lane group and token (padding shifts the banks between groups)
 constexpr int DL_TBR = 32;          // TB * R <= this
-constexpr int DL_NA = 5;
 
-template <typename T, int NW>
+template <typename T, int NW, int NA>
 __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ rf, const float* __restrict__ wf,
                                                          const float* __restrict__ nf, const float* __restrict__ bf,
-                                                         const float* __restrict__ kf, const T* __restrict__ P, int64_t ldp, int v0,
+                                                         const float* __restrict__ kf, const float* __restrict__ gb, int G,
+                                                         const T* __restrict__ P, int64_t ldp, int v0,
                                                          float* __restrict__ state, float* __restrict__ out, int H, int d, int vd,
                                                          int R, int TB, int values, Batch bt) {
-  constexpr int NT = 64 * NW, DL_PRE = DL_NA * DL_TBR * DL_DR / NT;
-  extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k: [TB][R][SEG] each, v[TB][wcols] }
+  constexpr int NT = 64 * NW, DL_PRE = NA * DL_TBR * DL_DR / NT;
+  extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k (r, k): [TB][R][SEG] each, v[TB][wcols], (g, beta)[TB] }
   const int b = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63;
   const int cols = 64 / R, wcols = NW * cols;
@@ -82,9 +173,9 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
   const int start = bt.seq_start[b], n = bt.seq_start[b + 1] - start, past = bt.seq_past[b], slot = bt.seq_slot[b];
   const bool colok = col < vd;
   const int row0 = r * DL_DR;
-  const int HD = H * d;
+  const int HD = NA == 2 ? G * d : H * d, hd0 = NA == 2 ? h / (H / G) * d : h * d;      // floats of an array's row, this head's first
   const int qsz = TB * R * DL_SEG;                         // floats of one array in a buffer
-  const int bufsz = DL_NA * qsz + TB * wcols;
+  const int bufsz = NA * qsz + TB * wcols + (NA == 2 ? (2 * TB + 3) & ~3 : 0);
   float S[DL_DR];
   float* sp = state + (((int64_t)slot * H + h) * d) * vd;
   {
@@ -96,25 +187,26 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
       S[k] = (past > 0 && colok && row < d) ? v : 0.f;
     }
   }
-  float pre[DL_PRE], prev[4];
+  float pre[DL_PRE], prev[4], preg = 0.f;
   // element e of a block = (token tk, array, row): tokens are the slowest index, so a block of few tokens (a single
-  // decoded one) ends the loops early; R * 32 is a power of two (lr = its logarithm) and 5 a constant, so no step divides
+  // decoded one) ends the loops early; R * 32 is a power of two (lr = its logarithm) and NA a constant, so no step divides
   const int lr = 31 - __clz(R * DL_DR), rows = R * DL_DR;
   auto fetch = [&](int i0) {                               // block of tokens i0 .. i0 + TB - 1 into registers
-    const int live = (n - i0 < TB ? n - i0 : TB) * DL_NA * rows;
+    const int live = (n - i0 < TB ? n - i0 : TB) * NA * rows;
 #pragma unroll
     for (int u = 0; u < DL_PRE; ++u) {
       if (NT * u >= live) break;
       const int e = tid + NT * u;
       const int ta = e >> lr, row = e & (rows - 1);
-      const int tk = ta / DL_NA, which = ta - tk * DL_NA;
-      float v = which == 1 ? 1.f : 0.f;                    // padding: w = 1, everything else 0
+      const int tk = ta / NA, which = ta - tk * NA;
+      float v = NA == 5 && which == 1 ? 1.f : 0.f;         // padding: w = 1, everything else 0
       if (e < live && row < d) {
-        const float* src = which == 0 ? rf : which == 1 ? wf : which == 2 ? nf : which == 3 ? bf : kf;
-        v = src[(int64_t)(start + i0 + tk) * HD + h * d + row];
+        const float* src = which == 0 ? rf : NA == 2 ? kf : which == 1 ? wf : which == 2 ? nf : which == 3 ? bf : kf;
+        v = src[(int64_t)(start + i0 + tk) * HD + hd0 + row];
       }
       pre[u] = v;
     }
+    if (NA == 2 && tid < 2 * TB && i0 + (tid >> 1) < n) preg = gb[((int64_t)(start + i0 + (tid >> 1)) * H + h) * 2 + (tid & 1)];
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int e = tid + NT * u;
@@ -127,22 +219,23 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
     }
   };
   auto stash = [&](float* buf, int i0) {
-    const int live = (n - i0 < TB ? n - i0 : TB) * DL_NA * rows;
+    const int live = (n - i0 < TB ? n - i0 : TB) * NA * rows;
 #pragma unroll
     for (int u = 0; u < DL_PRE; ++u) {
       if (NT * u >= live) break;
       const int e = tid + NT * u;
       if (e < live) {
         const int ta = e >> lr, row = e & (rows - 1);
-        const int tk = ta / DL_NA, which = ta - tk * DL_NA;
+        const int tk = ta / NA, which = ta - tk * NA;
         buf[which * qsz + (tk * R + (row >> 5)) * DL_SEG + (row & 31)] = pre[u];
       }
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int e = tid + NT * u;
-      if (e < TB * wcols) buf[DL_NA * qsz + e] = prev[u];
+      if (e < TB * wcols) buf[NA * qsz + e] = prev[u];
     }
+    if (NA == 2 && tid < 2 * TB) buf[NA * qsz + TB * wcols + tid] = preg;
   };
   if (n > 0) { fetch(0); stash(smem, 0); }
   __syncthreads();
@@ -155,11 +248,11 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
     for (int tk = 0; tk < nt; ++tk) {
       const int seg = (tk * R + r) * DL_SEG;
       const float4* r4 = reinterpret_cast<const float4*>(buf + seg);
-      const float4* w4 = reinterpret_cast<const float4*>(buf + qsz + seg);
-      const float4* n4 = reinterpret_cast<const float4*>(buf + 2 * qsz + seg);
-      const float4* b4 = reinterpret_cast<const float4*>(buf + 3 * qsz + seg);
-      const float4* k4 = reinterpret_cast<const float4*>(buf + 4 * qsz + seg);
-      const float v = buf[DL_NA * qsz + tk * wcols + lc];
+      const float4* k4 = reinterpret_cast<const float4*>(buf + (NA - 1) * qsz + seg);
+      const float4* w4 = reinterpret_cast<const float4*>(buf + qsz + seg);               // (NA == 5)
+      const float4* n4 = NA == 5 ? reinterpret_cast<const float4*>(buf + 2 * qsz + seg) : k4;
+      const float4* b4 = reinterpret_cast<const float4*>(buf + (NA == 5 ? 3 * qsz : 0) + seg);   // (NA == 5)
+      const float v = buf[NA * qsz + tk * wcols + lc];
       // n . s over the old state
       float acc[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -169,14 +262,28 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
       }
       const float dot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
       acc[0] = acc[1] = acc[2] = acc[3] = 0.f;
+      if (NA == 2) {
+        const float2 gs = *reinterpret_cast<const float2*>(buf + NA * qsz + TB * wcols + 2 * tk);
+        const float w = gs.x, c = gs.y * (v - w * dot);
 #pragma unroll
-      for (int k = 0; k < DL_DR / 4; ++k) {
-        const float4 w = w4[k], bb = b4[k], kk = k4[k], q = r4[k];
-        S[4 * k] = w.x * S[4 * k] - bb.x * dot + kk.x * v;
-        S[4 * k + 1] = w.y * S[4 * k + 1] - bb.y * dot + kk.y * v;
-        S[4 * k + 2] = w.z * S[4 * k + 2] - bb.z * dot + kk.z * v;
-        S[4 * k + 3] = w.w * S[4 * k + 3] - bb.w * dot + kk.w * v;
-        acc[0] += S[4 * k] * q.x; acc[1] += S[4 * k + 1] * q.y; acc[2] += S[4 * k + 2] * q.z; acc[3] += S[4 * k + 3] * q.w;
+        for (int k = 0; k < DL_DR / 4; ++k) {
+          const float4 kk = k4[k], q = r4[k];
+          S[4 * k] = w * S[4 * k] + kk.x * c;
+          S[4 * k + 1] = w * S[4 * k + 1] + kk.y * c;
+          S[4 * k + 2] = w * S[4 * k + 2] + kk.z * c;
+          S[4 * k + 3] = w * S[4 * k + 3] + kk.w * c;
+          acc[0] += S[4 * k] * q.x; acc[1] += S[4 * k + 1] * q.y; acc[2] += S[4 * k + 2] * q.z; acc[3] += S[4 * k + 3] * q.w;
+        }
+      } else {
+#pragma unroll
+        for (int k = 0; k < DL_DR / 4; ++k) {
+          const float4 w = w4[k], bb = b4[k], kk = k4[k], q = r4[k];
+          S[4 * k] = w.x * S[4 * k] - bb.x * dot + kk.x * v;
+          S[4 * k + 1] = w.y * S[4 * k + 1] - bb.y * dot + kk.y * v;
+          S[4 * k + 2] = w.z * S[4 * k + 2] - bb.z * dot + kk.z * v;
+          S[4 * k + 3] = w.w * S[4 * k + 3] - bb.w * dot + kk.w * v;
+          acc[0] += S[4 * k] * q.x; acc[1] += S[4 * k + 1] * q.y; acc[2] += S[4 * k + 2] * q.z; acc[3] += S[4 * k + 3] * q.w;
+        }
       }
       const float tot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
       if (out && r == 0 && colok) out[(int64_t)(start + i0 + tk) * (H * vd) + h * vd + col] = tot;
@@ -192,10 +299,10 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
   }
 }
 
-// out may be null (only the end states are wanted); values = 0: the value columns of P are not read and count as 0
-extern "C" int ragged_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const void* P,
-                                 int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
-                                 int dtype, hipStream_t st) {
+template <int NA>
+static int launch_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const float* gb, int G,
+                             const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
+                             int dtype, hipStream_t st) {
   if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 32 || (values && !P)) return -1;
   int R = 1;
   while (R * DL_DR < d) R <<= 1;
@@ -204,14 +311,29 @@ extern "C" int ragged_delta_scan(const float* rf, const float* wf, const float* 
   int TB = DL_TBR / R < 16 ? DL_TBR / R : 16;
   if (TB * wcols > 4 * 64 * nw) TB = 4 * 64 * nw / wcols;   // the value look-ahead holds 4 floats per thread
   if (TB < 1) return -1;
-  const size_t sm = 2 * (size_t)(DL_NA * TB * R * DL_SEG + TB * wcols) * sizeof(float);
+  // (2 TB <= 32 threads bring the gated rule's scalars; TB wcols and a buffer's parts are multiples of 16 bytes)
+  const size_t sm = 2 * (size_t)(NA * TB * R * DL_SEG + TB * wcols + (NA == 2 ? (2 * TB + 3) & ~3 : 0)) * sizeof(float);
   const dim3 grid((vd + wcols - 1) / wcols, H, bt.B);
   RAGGED_DISPATCH(dtype,
-    if (nw == 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2>), grid, dim3(128), sm, st, rf, wf, nf, bf, kf, (const T*)P, ldp, v0, state,
-                                    out, H, d, vd, R, TB, values, bt);
-    else hipLaunchKernelGGL((delta_scan_kernel<T, 4>), grid, dim3(256), sm, st, rf, wf, nf, bf, kf, (const T*)P, ldp, v0, state, out,
-                            H, d, vd, R, TB, values, bt))
+    if (nw == 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, NA>), grid, dim3(128), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp,
+                                    v0, state, out, H, d, vd, R, TB, values, bt);
+    else hipLaunchKernelGGL((delta_scan_kernel<T, 4, NA>), grid, dim3(256), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp, v0,
+                            state, out, H, d, vd, R, TB, values, bt))
   return RAGGED_LAUNCH_OK();
+}
+
+// out may be null (only the end states are wanted); values = 0: the value columns of P are not read and count as 0
+extern "C" int ragged_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const void* P,
+                                 int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
+                                 int dtype, hipStream_t st) {
+  return launch_delta_scan<5>(rf, wf, nf, bf, kf, nullptr, H, P, ldp, v0, state, out, H, d, vd, values, bt, dtype, st);
+}
+
+// the gated rule: qf, kf [rows, G d], gb [rows, H, 2]
+extern "C" int ragged_gated_delta_scan(const float* qf, const float* kf, const float* gb, int G, const void* P, int64_t ldp, int v0,
+                                       float* state, float* out, int H, int d, int vd, int values, Batch bt, int dtype, hipStream_t st) {
+  if (G <= 0 || H % G || !gb) return -1;
+  return launch_delta_scan<2>(qf, nullptr, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, bt, dtype, st);
 }
 
 // ---------------------------------------------------------------------------------------------------------------

@@ -1,6 +1,7 @@
 // Row-wise kernels of the ragged engine: residual sum + grouped RMS norm, short causal convolution with per-sequence
 // state + per-head norm + rotary + paged append, clamped gated activation, HGRN2 gates / scan / output norm, the stream
-// updates of the sandwich, parallel and sequential pre-norm blocks (the last over several copies of the stream),
+// updates of the sandwich, parallel and sequential pre-norm blocks (the last over several copies of the stream) and of the
+// output-norm block (LayerNorm on a sublayer's result, causal convolution of the stream in front of the next mixer),
 // embedding rows, activations of dense feed-forwards, gates per channel.
 // gfx950, wave64.  Everything that the engine keeps in 32 bits (residual, norms, angles, gates, recurrent state) is
 // float here whatever the activation type T is.
@@ -816,5 +817,277 @@ extern "C" int ragged_gate_cols(const float* o, const void* P, int64_t ldp, int 
   const unsigned grid = (unsigned)(blocks < 16384 ? blocks : 16384);
   RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((gate_cols_kernel<T>), dim3(grid), dim3(256), 0, st, o, (const T*)P, ldp, g0, (T*)out, rows,
                                             n, scale))
+  return RAGGED_LAUNCH_OK();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// Short causal convolution over time per channel for whole rows: u_t = sum_j w[c, j] s_(t - taps + 1 + j) (+ bias), then
+// out = silu(u), s + u or u.  A thread walks RB neighbouring rows of one channel with the last taps - 1 inputs in registers
+// (TAPS = the number of taps, or 0 for any number: every tap is then read where it is needed).  A sequence's inputs before
+// this step come from `state` [slots, taps - 1, C] (the type of the source); `write_state` (every sequence brings exactly one
+// row) also shifts the state, otherwise ragged_conv_state does so behind this kernel.
+constexpr int CR_RB = 16;
+
+template <typename TI, typename TO, int TAPS>
+__global__ __launch_bounds__(256) void conv_rows_kernel(const TI* __restrict__ src, int64_t ld, int col0, const float* __restrict__ cw,
+                                                        const float* __restrict__ bias, TI* __restrict__ state, int ntaps, int C,
+                                                        TO* __restrict__ out, int add, int silu, int write_state, Batch bt) {
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= C) return;
+  const int taps = TAPS > 0 ? TAPS : ntaps, keep = taps - 1;
+  const int t0 = blockIdx.y * CR_RB, t1 = t0 + CR_RB < bt.T ? t0 + CR_RB : bt.T;
+  // the input `back` positions before row t (position pos of a sequence whose first `past` positions are older than the step)
+  auto input = [&](int t, int back, int pos, int past, int slot) -> float {
+    const int pp = pos - back;
+    if (pp >= past) return to_f(src[(int64_t)(t - back) * ld + col0 + c]);
+    if (pp >= 0) return to_f(state[((int64_t)slot * keep + (pp - past + keep)) * C + c]);
+    return 0.f;
+  };
+  float w[TAPS > 0 ? TAPS : 1], hist[TAPS > 1 ? TAPS - 1 : 1];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) w[j] = cw[(int64_t)c * TAPS + j];
+  const float b0 = bias ? bias[c] : 0.f;
+  for (int t = t0; t < t1; ++t) {
+    const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
+    const float cur = to_f(src[(int64_t)t * ld + col0 + c]);
+    float u = b0;
+    if (TAPS > 0) {
+      if (t == t0 || pos == past) {                          // (the same branch for the whole workgroup)
+#pragma unroll
+        for (int j = 0; j + 1 < TAPS; ++j) hist[j] = input(t, TAPS - 1 - j, pos, past, slot);
+      }
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j) u += w[j] * hist[j];
+      u += w[TAPS > 0 ? TAPS - 1 : 0] * cur;
+#pragma unroll
+      for (int j = 0; j + 2 < TAPS; ++j) hist[j] = hist[j + 1];
+      if (TAPS > 1) hist[TAPS > 1 ? TAPS - 2 : 0] = cur;
+      if (write_state) {
+#pragma unroll
+        for (int j = 0; j + 1 < TAPS; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(hist[j]);
+      }
+    } else {
+      for (int j = 0; j < taps; ++j) u += cw[(int64_t)c * taps + j] * input(t, taps - 1 - j, pos, past, slot);
+      if (write_state) {                                     // (row j + 1 is read before row j + 1 is written)
+        for (int j = 0; j < keep; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(input(t, keep - 1 - j, pos, past, slot));
+      }
+    }
+    if (silu) u = u / (1.0f + expf(-u));
+    out[(int64_t)t * C + c] = from_f<TO>(add ? cur + u : u);
+  }
+}
+
+template <typename TI, typename TO>
+static void launch_conv_rows(const void* src, int64_t ld, int col0, const float* cw, const float* bias, void* state, int taps, int C,
+                             void* out, int add, int silu, int write_state, Batch bt, hipStream_t st) {
+  const dim3 grid((C + 255) / 256, (bt.T + CR_RB - 1) / CR_RB);
+#define CR_CASE(N) hipLaunchKernelGGL((conv_rows_kernel<TI, TO, N>), grid, dim3(256), 0, st, (const TI*)src, ld, col0, cw, bias, \
+                                      (TI*)state, taps, C, (TO*)out, add, silu, write_state, bt)
+  if (taps == 1) CR_CASE(1);
+  else if (taps == 2) CR_CASE(2);
+  else if (taps == 3) CR_CASE(3);
+  else if (taps == 4) CR_CASE(4);
+  else CR_CASE(0);
+#undef CR_CASE
+}
+
+// the source's type is `src_dtype` (the projections' activation type, or float for the stream itself), the output's `dtype`
+extern "C" int ragged_conv_rows(const void* src, int64_t ld, int col0, const float* cw, const float* bias, void* state, int taps, int C,
+                                void* out, int add, int silu, int write_state, Batch bt, int src_dtype, int dtype, hipStream_t st) {
+  if (bt.T <= 0 || bt.T > 65535 * CR_RB || C <= 0 || col0 < 0 || ld < col0 + C || taps < 1 || taps > 16 || (taps > 1 && !state)) return -1;
+  if (src_dtype != dtype && src_dtype != 2) return -2;
+  if (taps == 1) write_state = 0;
+  RAGGED_DISPATCH(dtype,
+    if (src_dtype == 2) launch_conv_rows<float, T>(src, ld, col0, cw, bias, state, taps, C, out, add, silu, write_state, bt, st);
+    else launch_conv_rows<T, T>(src, ld, col0, cw, bias, state, taps, C, out, add, silu, write_state, bt, st))
+  return RAGGED_LAUNCH_OK();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// Output-norm form: x <- x + LN(y), LN(u) = (u - mean) / sqrt(mean((u - mean)^2) + eps) * w + b, on the float stream, then
+// xa = x as T for the product that reads the stream next.  With `cw` (every sequence brings exactly one row) xa is the
+// convolved stream x + sum_j cw[c, j] x_(t - taps + 1 + j) that the next layer's mixer reads: the older inputs come from
+// `hist` [slots, taps - 1, D], which is shifted in the same pass.  y null: xa = LN(x), the stream stays as it is.
+// One workgroup per row; NV as in post_norm_add_kernel.
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void ln_add_kernel(float* __restrict__ x, const T* __restrict__ y, const float* __restrict__ w,
+                                                     const float* __restrict__ bias, T* __restrict__ xa, int D, float eps,
+                                                     const float* __restrict__ cw, int taps, float* __restrict__ hist, Batch bt) {
+  __shared__ float red[8];
+  const int64_t row = blockIdx.x, base = row * D;
+  int slot = 0, pos = 0;
+  if (cw) { slot = bt.seq_slot[bt.tok_seq[row]]; pos = bt.tok_pos[row]; }
+  const int keep = taps - 1;
+  auto finish = [&](int c, float norm) {
+    const float v = y ? x[base + c] + norm : norm;
+    if (y) x[base + c] = v;
+    if (!xa) return;
+    float h = v;
+    if (cw) {
+      float u = 0.f;
+      for (int j = 0; j < keep; ++j) {                       // hist row j holds the input at position pos - keep + j
+        const int64_t o = ((int64_t)slot * keep + j) * D + c;
+        const float old = pos - keep + j >= 0 ? hist[o] : 0.f;
+        u += cw[(int64_t)c * taps + j] * old;
+        if (j > 0) hist[o - D] = old;
+      }
+      if (keep > 0) hist[((int64_t)slot * keep + keep - 1) * D + c] = v;
+      h = v + u + cw[(int64_t)c * taps + keep] * v;
+    }
+    xa[base + c] = from_f<T>(h);
+  };
+  if (NV > 0) {
+    float v[NV > 0 ? NV : 1];
+    float s = 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int c = threadIdx.x + 256 * u;
+      v[u] = c < D ? (y ? to_f(y[base + c]) : x[base + c]) : 0.f;
+      s += v[u];
+    }
+    const float mean = block_sum_256(s, red) / (float)D;
+    s = 0.f;
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      v[u] = threadIdx.x + 256 * u < D ? v[u] - mean : 0.f;
+      s += v[u] * v[u];
+    }
+    const float r = 1.0f / sqrtf(block_sum_256(s, red + 4) / (float)D + eps);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int c = threadIdx.x + 256 * u;
+      if (c < D) finish(c, v[u] * r * w[c] + bias[c]);
+    }
+    return;
+  }
+  float s = 0.f;
+  for (int c = threadIdx.x; c < D; c += 256) s += y ? to_f(y[base + c]) : x[base + c];
+  const float mean = block_sum_256(s, red) / (float)D;
+  s = 0.f;
+  for (int c = threadIdx.x; c < D; c += 256) { const float v = (y ? to_f(y[base + c]) : x[base + c]) - mean; s += v * v; }
+  const float r = 1.0f / sqrtf(block_sum_256(s, red + 4) / (float)D + eps);
+  for (int c = threadIdx.x; c < D; c += 256) finish(c, ((y ? to_f(y[base + c]) : x[base + c]) - mean) * r * w[c] + bias[c]);
+}
+
+extern "C" int ragged_ln_add(float* x, const void* y, const float* w, const float* bias, void* xa, int64_t rows, int D, float eps,
+                             const float* cw, int taps, float* hist, Batch bt, int dtype, hipStream_t st) {
+  if (rows <= 0 || D <= 0 || rows > 0x7fffffff || !x || !w || !bias || (!y && !xa)) return -1;
+  if (cw && (!xa || !y || taps < 1 || taps > 16 || (taps > 1 && !hist) || bt.T != rows || bt.B != rows)) return -1;
+  RAGGED_DISPATCH(dtype,
+    if (D <= 1024) hipLaunchKernelGGL((ln_add_kernel<T, 4>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias, (T*)xa, D,
+                                      eps, cw, taps, hist, bt);
+    else if (D <= 4096) hipLaunchKernelGGL((ln_add_kernel<T, 16>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias,
+                                           (T*)xa, D, eps, cw, taps, hist, bt);
+    else hipLaunchKernelGGL((ln_add_kernel<T, 0>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias, (T*)xa, D, eps, cw,
+                            taps, hist, bt))
+  return RAGGED_LAUNCH_OK();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+// Queries, keys and values of attention layers whose query / key norm covers the whole projection: one pass over a row's
+// [q | k | v] columns.  q and k: divided by the root mean square of all H d (G d) channels, times a weight per channel, then
+// the first `rot` channels of every head turned in pairs (i, i + rot / 2); q to a float buffer, k to its page.  v: with
+// `v_norm` every head divided by its root mean square; with `first_in` v <- (1 - lam) v + lam first (float values that an
+// earlier layer left in `first_out` [T, G vd] for the same rows); to its page.  One workgroup per token row.
+struct QkvRowsArgs {
+  const void* P;         // [T, ldp], columns 0 .. : q [H d] | k [G d] | v [G vd]
+  int64_t ldp;
+  int H, G, d, vd;
+  const float* qw;       // [H d]
+  const float* kw;       // [G d]
+  float eps;
+  int rot;
+  const float* cossin;   // [T, rot / 2, 2]
+  float* q_out;          // [T, H d]
+  void* kpages;          // [pages, G, PAGE, d]
+  void* vpages;          // [pages, G, PAGE, vd]
+  int v_norm;
+  const float* first_in;
+  float* first_out;
+  float lam;
+};
+
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRowsArgs a, Batch bt) {
+  extern __shared__ __attribute__((aligned(16))) float srow[];       // [q | k] of the row
+  __shared__ float red[8];
+  const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int nq = a.H * a.d, nk = a.G * a.d;
+  const T* row = (const T*)a.P + (int64_t)t * a.ldp;
+  const int b = bt.tok_seq[t], pos = bt.tok_pos[t];
+  const int64_t page = bt.pages[(int64_t)b * bt.max_pages + pos / PAGE];
+  float sq = 0.f, sk = 0.f;
+  if (VEC) {                                                 // 16 bytes per load; nq, nk and the row are multiples of the piece
+    constexpr int N = 16 / (int)sizeof(T);
+    for (int c = threadIdx.x * N; c < nq + nk; c += 256 * N) {
+      union { uint4 q; T e[N]; } p;
+      p.q = *reinterpret_cast<const uint4*>(row + c);
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < N; ++i) { const float v = to_f(p.e[i]); srow[c + i] = v; s += v * v; }
+      if (c < nq) sq += s; else sk += s;
+    }
+  } else {
+    for (int c = threadIdx.x; c < nq + nk; c += 256) {
+      const float v = to_f(row[c]);
+      srow[c] = v;
+      if (c < nq) sq += v * v; else sk += v * v;
+    }
+  }
+  const float rq = 1.0f / sqrtf(block_sum_256(sq, red) / (float)nq + a.eps);
+  const float rk = 1.0f / sqrtf(block_sum_256(sk, red + 4) / (float)nk + a.eps);      // (its barrier also covers srow)
+  const int half = a.rot >> 1;
+  const float2* turn = reinterpret_cast<const float2*>(a.cossin) + (int64_t)t * half;
+  for (int hd = wave; hd < a.H + a.G; hd += 4) {
+    const bool isq = hd < a.H;
+    const int g = hd - a.H;
+    const float* u = srow + hd * a.d;
+    const float* w = isq ? a.qw + hd * a.d : a.kw + g * a.d;
+    const float r = isq ? rq : rk;
+    float* qo = a.q_out + (int64_t)t * nq + hd * a.d;
+    T* ko = (T*)a.kpages + ((page * a.G + g) * PAGE + pos % PAGE) * a.d;
+    for (int c = lane; c < a.d; c += 64) {
+      float v = u[c] * r * w[c];
+      if (c < a.rot) {
+        const bool low = c < half;
+        const int o = low ? c + half : c - half;
+        const float2 cs = turn[low ? c : o];
+        const float other = u[o] * r * w[o];
+        v = low ? v * cs.x - other * cs.y : v * cs.x + other * cs.y;
+      }
+      if (isq) qo[c] = v;
+      else ko[c] = from_f<T>(v);
+    }
+  }
+  for (int g = wave; g < a.G; g += 4) {
+    const T* vr = row + nq + nk + g * a.vd;
+    float r = 1.f;
+    if (a.v_norm) {
+      float s = 0.f;
+      for (int c = lane; c < a.vd; c += 64) { const float v = to_f(vr[c]); s += v * v; }
+      r = 1.0f / sqrtf(wave_sum(s) / (float)a.vd + a.eps);
+    }
+    T* vo = (T*)a.vpages + ((page * a.G + g) * PAGE + pos % PAGE) * a.vd;
+    const int64_t f0 = ((int64_t)t * a.G + g) * a.vd;
+    for (int c = lane; c < a.vd; c += 64) {
+      float v = to_f(vr[c]) * r;
+      if (a.first_in) v = (1.0f - a.lam) * v + a.lam * a.first_in[f0 + c];
+      if (a.first_out) a.first_out[f0 + c] = v;
+      vo[c] = from_f<T>(v);
+    }
+  }
+}
+
+extern "C" int ragged_qkv_rows(QkvRowsArgs a, Batch bt, int dtype, hipStream_t st) {
+  if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.d <= 0 || a.vd <= 0 || a.rot < 0 || (a.rot & 1) || a.rot > a.d) return -1;
+  if (!a.qw || !a.kw || !a.q_out || !a.kpages || !a.vpages || (a.rot && !a.cossin)) return -1;
+  const int64_t n = (int64_t)(a.H + a.G) * a.d;
+  if (n * (int64_t)sizeof(float) > 60 * 1024 || a.ldp < n + (int64_t)a.G * a.vd) return -1;
+  const size_t sm = (size_t)n * sizeof(float);
+  RAGGED_DISPATCH(dtype,
+    constexpr int N = 16 / (int)sizeof(T);
+    const bool vec = (a.H * a.d) % N == 0 && (a.G * a.d) % N == 0 && a.ldp % N == 0 && ((uintptr_t)a.P % 16) == 0;
+    if (vec) hipLaunchKernelGGL((qkv_rows_kernel<T, true>), dim3((unsigned)bt.T), dim3(256), sm, st, a, bt);
+    else hipLaunchKernelGGL((qkv_rows_kernel<T, false>), dim3((unsigned)bt.T), dim3(256), sm, st, a, bt))
   return RAGGED_LAUNCH_OK();
 }

@@ -10,6 +10,7 @@ slots.  A layer declares what it keeps with a spec tuple:
     ("k", heads, key_row)                  pages  K alone (a layer whose values are part of its key rows)
     ("vector", size)                       slot   [slots, size]              float32
     ("tail", rows, channels)               slot   [slots, rows, channels]    activation type
+    ("stream_tail", rows, channels)        slot   [slots, rows, channels]    float32 (inputs of a convolution of the stream itself)
     ("matrix", heads, rows, cols)          slot   [slots, heads, rows, cols] float32
 
 The keys of the spec dictionary name layer executions (a layer that runs twice keeps two caches).  The pool also
@@ -40,6 +41,7 @@ class PagedStatePool:
         self.k: Dict[int, torch.Tensor] = {}
         self.v: Dict[int, torch.Tensor] = {}
         self.tail: Dict[int, torch.Tensor] = {}
+        self.stream_tail: Dict[int, torch.Tensor] = {}
         self.matrix: Dict[int, torch.Tensor] = {}
         self.vector: Dict[int, torch.Tensor] = {}
         for li, layer_specs in specs.items():
@@ -57,6 +59,9 @@ class PagedStatePool:
                 elif kind == "tail":
                     _, rows, channels = spec
                     self.tail[li] = torch.zeros(self.slots, rows, channels, dtype=act_dtype, device=self.device)
+                elif kind == "stream_tail":
+                    _, rows, channels = spec
+                    self.stream_tail[li] = torch.zeros(self.slots, rows, channels, dtype=torch.float32, device=self.device)
                 elif kind == "matrix":
                     _, heads, rows, cols = spec
                     self.matrix[li] = torch.zeros(self.slots, heads, rows, cols, dtype=torch.float32, device=self.device)
@@ -108,4 +113,4 @@ class PagedStatePool:
         return sum(self.len_of.values())
 
     def nbytes(self) -> int:
-        return sum(t.numel() * t.element_size() for d in (self.k, self.v, self.tail, self.matrix, self.vector) for t in d.values())
+        return sum(t.numel() * t.element_size() for d in (self.k, self.v, self.tail, self.stream_tail, self.matrix, self.vector) for t in d.values())

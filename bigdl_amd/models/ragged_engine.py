@@ -9,13 +9,15 @@ into arbitrary portions next to single decoded tokens run here instead:
   product runs once over all rows; the mixers read ``BatchMeta`` (row -> sequence, position, pages);
 * keys / values live in 64-token pages of a ``PagedStatePool``, per-sequence state in its slots;
 * the mixers are described by small dataclasses whose fields are the design's constants, so a new design is a new list
-  of them (``models/lipizen.py``, ``models/merusun.py``, ``models/filanex.py`` and ``models/dimelix.py`` build one from
-  a ``config.json``);
-* four residual forms: the post-sum norm x <- norm(alpha x + f(x)), the sandwich x <- x + norm_b(f(norm_a(x))), the
+  of them (``models/lipizen.py``, ``models/merusun.py``, ``models/filanex.py``, ``models/dimelix.py`` and
+  ``models/supisun.py`` build one from a ``config.json``);
+* five residual forms: the post-sum norm x <- norm(alpha x + f(x)), the sandwich x <- x + norm_b(f(norm_a(x))), the
   parallel pre-norm block u = norm(x), x <- x + mixer(u) + ff(u), and the sequential pre-norm block x <- x + f(norm(x))
-  per sublayer, whose stream may be kept in several copies that every sublayer reads and rewrites with learned weights;
+  per sublayer, whose stream may be kept in several copies that every sublayer reads and rewrites with learned weights,
+  and the output-norm block x <- x + LN(f(x)), whose mixers may read the stream behind a short causal convolution;
 * a run of layers may be executed several times with the same weights (every execution has its own cache), with the
-  embedding output mixed back into the stream in front of a pass; the embedding may add a row of a token-pair table;
+  embedding output mixed back into the stream in front of a pass; the embedding may add a row of a token-pair table or of
+  a table of learned positions;
 * matrix products are the library's (bf16 inputs with 32-bit accumulation, or plain float32), everything between them
   is ``ops/ragged.py``.
 """
@@ -67,6 +69,10 @@ class WindowAttention:
     head_sinks: bool = False       # every head has a learned sink score (``LayerTensors.sinks``) instead of the one number ``sink``
     dist_slopes: Optional[tuple] = None  # per head: slope * (i - j) is taken off the scaled score of query i and key j
     v_from_k: bool = False         # no value projection: the values are the key projections as they are before norm and rotation
+    qk_norm_rows: bool = False     # RMS norm over the whole query (key) projection at once, a weight per channel, before rotation
+    v_norm: bool = False           # each head's value divided by its root mean square (no weight)
+    v_mix: bool = False            # values of the stack's first such layer are mixed in: v <- (1 - lam) v + lam v_first of the same
+                                   # token (``LayerTensors.v_lam``; needs equal value sizes); what is cached is the mixture
 
 
 @dataclass
@@ -101,6 +107,36 @@ class DeltaRule:
     decay_rate: float = math.exp(-0.5)
     unit_eps: float = 1e-6
     out_scale: float = 1.0
+
+
+@dataclass
+class GatedDelta:
+    """Gated delta rule: queries and keys of ``kv_heads`` heads (head h reads h / (heads / kv_heads)), values of ``heads``, each
+    behind a short causal convolution over time and silu, q and k then unit vectors u / sqrt(|u|^2 + unit_eps), q times dim^-1/2.
+    Per head a decay g = exp(-e^A_log softplus(W_a h + dt_bias)) and a write strength beta = sigmoid(W_b h):
+    S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q.  Each head's output is divided by its root mean square, weighted
+    (one weight of ``vdim`` channels for all heads) and multiplied by silu of a projection of the mixer's input."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv_taps: int
+    unit_eps: float = 1e-6
+
+    @property
+    def conv_channels(self) -> int:
+        return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+
+
+@dataclass
+class SelectiveScan:
+    """Selective scan (Mamba): [x | z] = W_in h, x behind a short causal convolution with bias and silu, [low | B | C] = W_x x,
+    step sizes d = softplus(W_dt low + bias) per channel; S <- exp(d A) S + d x B, y = S C + D x per channel and state
+    (A = -e^A_log); output projection of y silu(z)."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv_taps: int
 
 
 @dataclass
@@ -204,13 +240,17 @@ class RaggedConfig:
     name: str = "ragged"
     embed_scale: float = 1.0
     block: str = "post_sum"        # "post_sum": x <- norm(alpha x + f(x)); "sandwich": x <- x + norm_b(f(norm_a(x)));
-                                   # "parallel": u = norm(x), x <- x + mixer(u) + ff(u); "pre_norm": x <- x + f(norm(x)) per sublayer
+                                   # "parallel": u = norm(x), x <- x + mixer(u) + ff(u); "pre_norm": x <- x + f(norm(x)) per sublayer;
+                                   # "output_norm": x <- x + LN(f(x)) per sublayer, LN with weight and bias, as is the final norm
     streams: int = 1               # "pre_norm": copies of the stream; every sublayer reads a weighted sum of them and writes
                                    # X[t] <- sum_s mix[s, t] X[s] + out[t] f(.) (``LayerTensors.hc1 / hc2``); the model's output is their sum
     runs: Optional[list] = None    # layer index of every layer execution, in order (None: every layer once); an execution
                                    # has its own cache / state, whatever weights it shares
     mix_in: tuple = ()             # executions in front of which x <- W_mix [x ; embedding output]
     pair_embed: Optional[PairEmbedding] = None
+    positions: int = 0             # > 0: a learned vector per position is added to the embedding; no sequence grows beyond this
+    stream_conv: int = 0           # "output_norm": a mixer reads x + conv(x), a causal convolution of this many taps per channel of
+                                   # the stream (``LayerTensors.stream_conv``; 0: it reads x)
 
     def layer_runs(self) -> list:
         return list(range(len(self.mixers))) if self.runs is None else list(self.runs)
@@ -252,6 +292,17 @@ class LayerTensors:
     w_decay: Optional[torch.Tensor] = None   # delta rule: second product of the decay's low-rank pair [heads dim, rank]
     decay_bias: Optional[torch.Tensor] = None  # float [heads dim]
     remove_bias: Optional[torch.Tensor] = None  # float [heads dim]
+    norm1_bias: Optional[torch.Tensor] = None  # output-norm form: LayerNorm biases beside norm1 and norm2
+    norm2_bias: Optional[torch.Tensor] = None
+    stream_conv: Optional[torch.Tensor] = None  # float [width, taps]
+    v_lam: float = 0.0                       # share of the first mixing layer's values
+    decay_rate: Optional[torch.Tensor] = None  # gated delta rule: e^A_log float [heads]; its step bias is decay_bias
+    conv_b: Optional[torch.Tensor] = None    # selective scan: bias of the convolution, float [inner]
+    w_low: Optional[torch.Tensor] = None     # [dt_rank + 2 state, inner]
+    w_dt: Optional[torch.Tensor] = None      # [inner, dt_rank]
+    dt_bias: Optional[torch.Tensor] = None   # float [inner]
+    ssm_a: Optional[torch.Tensor] = None     # float [inner, state]: -e^A_log log2(e)
+    ssm_d: Optional[torch.Tensor] = None     # float [inner]
     left: Optional["LayerTensors"] = None    # side-by-side mixers: what each of the two needs beyond the shared projections
     right: Optional["LayerTensors"] = None
 
@@ -285,11 +336,14 @@ class RaggedDecoder:
 
     def __init__(self, cfg: RaggedConfig, embed: torch.Tensor, layers: List[LayerTensors], final_norm: torch.Tensor,
                  head: torch.Tensor, act_dtype=torch.bfloat16, device="cuda", pair_table: Optional[torch.Tensor] = None,
-                 w_mix: Optional[torch.Tensor] = None):
+                 w_mix: Optional[torch.Tensor] = None, pos_table: Optional[torch.Tensor] = None,
+                 final_norm_bias: Optional[torch.Tensor] = None):
         """``pair_table`` [buckets + 1, width]: the token-pair embedding of ``cfg.pair_embed``; ``w_mix`` [width, 2 width]:
-        the projection of [stream ; embedding output] in front of the executions named in ``cfg.mix_in``."""
+        the projection of [stream ; embedding output] in front of the executions named in ``cfg.mix_in``; ``pos_table``
+        [positions, width]: learned positions; ``final_norm_bias``: the bias of an "output_norm" model's last norm."""
         self.cfg, self.embed, self.layers, self.final_norm, self.head = cfg, embed, layers, final_norm, head
-        self.pair_table, self.w_mix = pair_table, w_mix
+        self.pair_table, self.w_mix, self.pos_table, self.final_norm_bias = pair_table, w_mix, pos_table, final_norm_bias
+        self.max_positions = cfg.positions or None
         self.act = act_dtype
         self.device = torch.device(device)
         self.ops = R.ops_for(self.device)
@@ -301,6 +355,17 @@ class RaggedDecoder:
             raise ValueError("mixing the embedding output back in needs a [width, 2 width] projection and the parallel block")
         if cfg.pair_embed is not None and (pair_table is None or tuple(pair_table.shape) != (cfg.pair_embed.buckets + 1, cfg.width)):
             raise ValueError("the token-pair table must have buckets + 1 rows of the stream's width")
+        if cfg.positions and (pos_table is None or tuple(pos_table.shape) != (cfg.positions, cfg.width) or cfg.pair_embed is not None):
+            raise ValueError("learned positions need a [positions, width] table (and no token-pair table beside it)")
+        if cfg.block == "output_norm":
+            if final_norm_bias is None or any(lt.norm1_bias is None or (mlp is not None and lt.norm2_bias is None)
+                                              for lt, mlp in zip(layers, cfg.mlps)):
+                raise ValueError("the output-norm block's LayerNorms need weights and biases")
+            if cfg.stream_conv and any(lt.stream_conv is None or tuple(lt.stream_conv.shape) != (cfg.width, cfg.stream_conv) for lt in layers):
+                raise ValueError("every layer needs its [width, taps] convolution of the stream")
+        elif cfg.stream_conv:
+            raise ValueError("only the output-norm block convolves the stream")
+        self._check_value_mixing()
         self._kv_run = {}                  # execution -> the execution whose cache it reads (itself unless kv_from is set)
         latest = {}
         for ri, li in enumerate(self.runs):
@@ -334,6 +399,24 @@ class RaggedDecoder:
         self._graphs = {}
         self.graph_replays = 0
 
+    def _check_value_mixing(self):
+        self._v_first = None               # the first execution whose values the later mixing layers share
+        for ri, li in enumerate(self.runs):
+            m = self.cfg.mixers[li]
+            if not isinstance(m, WindowAttention):
+                continue
+            if m.qk_norm_rows:
+                if m.maps != 1 or m.conv_taps or m.gate or m.kv_from is not None or m.v_from_k or m.rot_neighbours or m.rot_amp != 1.0:
+                    raise ValueError(f"layer {li}: the norm over whole projections serves plain q / k / v projections of one map")
+            elif m.v_norm or m.v_mix:
+                raise ValueError(f"layer {li}: normed or mixed values come with the norm over whole projections")
+            if m.v_mix:
+                if self._v_first is None:
+                    self._v_first = ri
+                f = self.cfg.mixers[self.runs[self._v_first]]
+                if (f.kv_heads, f.vdim) != (m.kv_heads, m.vdim):
+                    raise ValueError(f"layer {li}: mixed values must have the first mixing layer's sizes")
+
     # ------------------------------------------------------------------ state
     def state_specs(self):
         """what every layer execution keeps, by execution index"""
@@ -346,6 +429,8 @@ class RaggedDecoder:
             kinds = [spec[0] if spec[0] != "kv" else "k" for spec in s]
             if len(set(kinds)) != len(kinds):
                 raise ValueError(f"layer {li}: mixers side by side must keep different kinds of state")
+            if self.cfg.stream_conv > 1:
+                s.append(("stream_tail", self.cfg.stream_conv - 1, self.cfg.width))
             specs[ri] = s
         return specs
 
@@ -365,6 +450,14 @@ class RaggedDecoder:
             s.append(("vector", m.heads))                   # the running maximum of every head
         elif isinstance(m, DeltaRule):
             s.append(("matrix", m.heads, m.dim, m.dim))
+        elif isinstance(m, GatedDelta):
+            s.append(("matrix", m.heads, m.dim, m.vdim))
+            if m.conv_taps > 1:
+                s.append(("tail", m.conv_taps - 1, m.conv_channels))
+        elif isinstance(m, SelectiveScan):
+            s.append(("matrix", 1, m.inner, m.state))
+            if m.conv_taps > 1:
+                s.append(("tail", m.conv_taps - 1, m.inner))
         return s
 
     @staticmethod
@@ -385,6 +478,8 @@ class RaggedDecoder:
     def _attention(self, li, m: WindowAttention, lt: LayerTensors, P, meta):
         """``li`` (here and in the other mixers): the execution's index, which names its cache / state in the pool"""
         ops, pool, eps = self.ops, self.pool, self.cfg.norm_eps
+        if m.qk_norm_rows:
+            return self._attention_rows(li, m, lt, P, meta)
         turn = dict(interleaved=m.rot_neighbours, rot_amp=m.rot_amp)
         cq = m.heads * m.maps * m.dim
         ck = m.kv_heads * m.maps * m.dim
@@ -410,6 +505,38 @@ class RaggedDecoder:
                               out_norm=m.out_norm, eps=eps, gate=P if m.gate else None, gate0=col, sink=m.sink,
                               chunk=m.chunk, softcap=m.softcap, gate_wide=m.gate and m.gate_channels,
                               sinks=lt.sinks if m.head_sinks else None, slopes=lt.slopes if m.dist_slopes is not None else None)
+
+    def _attention_rows(self, li, m: WindowAttention, lt: LayerTensors, P, meta):
+        """queries, keys and values of a row in one pass: norms over whole projections, rotation, value norm and mixing"""
+        ops, pool, eps = self.ops, self.pool, self.cfg.norm_eps
+        first = li == self._v_first
+        mix = m.v_mix and not first
+        q, v = ops.qkv_rows(P, lt.q_norm, lt.k_norm, eps, m.rot_dims, lt.inv_freq, pool.k[li], pool.v[li], meta, H=m.heads,
+                            G=m.kv_heads, d=m.dim, vd=m.vdim, v_norm=m.v_norm, first_in=meta.shared["values"] if mix else None,
+                            lam=lt.v_lam, want_first=first)
+        if first:
+            meta.shared["values"] = v
+        return ops.paged_attn(q, pool.k[li], pool.v[li], meta, maps=1, H=m.heads, G=m.kv_heads, d=m.dim, vd=m.vdim, window=m.window,
+                              keep_first=m.keep_first, scale=m.scale, lam=0.0, out_scale=m.out_scale, out_norm=m.out_norm, eps=eps,
+                              sink=m.sink, chunk=m.chunk, softcap=m.softcap, sinks=lt.sinks if m.head_sinks else None,
+                              slopes=lt.slopes if m.dist_slopes is not None else None)
+
+    def _gated_delta(self, li, m: GatedDelta, lt: LayerTensors, P, meta):
+        ops, pool = self.ops, self.pool
+        C, hv = m.conv_channels, m.heads * m.vdim
+        # columns of P: q | k | v | output gate | write strengths | step logits
+        qf, kf, v, gb = ops.gated_delta_prep(P, lt.conv_w, m.conv_taps, pool.tail.get(li), C + hv, C + hv + m.heads, lt.decay_rate,
+                                             lt.decay_bias, m.unit_eps, m.heads, m.kv_heads, m.dim, m.vdim, meta)
+        o = ops.gated_delta_scan(qf, kf, gb, m.kv_heads, v, pool.matrix[li], m.heads, m.dim, m.vdim, meta)
+        return ops.head_norm_gate(o, lt.o_norm, P, C, m.heads, m.vdim, self.cfg.norm_eps, self.act, gate="silu")
+
+    def _selective(self, li, m: SelectiveScan, lt: LayerTensors, P, meta):
+        ops, pool = self.ops, self.pool
+        # columns of P: x | z
+        x = ops.conv_rows(P, 0, lt.conv_w, lt.conv_b, pool.tail.get(li), meta, self.act, silu=True)
+        M = F.linear(x, lt.w_low)                    # low-rank step input | B | C
+        dt = self._linear_f32(M[:, :m.dt_rank], lt.w_dt)
+        return ops.selective_scan(x, dt, lt.dt_bias, M, m.dt_rank, m.dt_rank + m.state, lt.ssm_a, lt.ssm_d, P, m.inner, pool.matrix[li], meta)
 
     def _latent(self, li, m: LatentAttention, lt: LayerTensors, P, meta):
         """Scores of head h are q_h . [W_uk,h c | rotated part] = [W_uk,h^T q_h | rotated query part] . [c | rotated part]:
@@ -522,7 +649,11 @@ class RaggedDecoder:
         Returns float32 logits [wanted rows, vocab] in the order of entries and indices."""
         pool = self.pool
         pairs = self.cfg.pair_embed
+        positions = self.cfg.positions
         seqs, ids, prs = [], [], []
+        for slot, toks in entries:
+            if positions and pool.len_of[slot] + len(toks) > positions:
+                raise ValueError(f"a sequence of {pool.len_of[slot] + len(toks)} tokens does not fit the model's {positions} positions")
         for slot, toks in entries:
             if len(toks) == 0:
                 raise ValueError("an entry without tokens")
@@ -530,6 +661,8 @@ class RaggedDecoder:
             ids += list(toks)
             if pairs is not None:                    # the previous token is part of the sequence's state
                 prs += pairs.rows(pool.last_token[slot], toks)
+            elif positions:
+                prs += range(pool.len_of[slot], pool.len_of[slot] + len(toks))
         rows, at = [], 0
         for b, (_, _, n, _) in enumerate(seqs):
             idx = [n - 1] if want is None else want[b]
@@ -537,7 +670,7 @@ class RaggedDecoder:
                 raise ValueError("a wanted index outside its entry")
             rows += [at + i for i in idx]
             at += n
-        idt = torch.tensor(ids if pairs is None else [ids, prs], dtype=torch.int64)      # [T], or [2, T] with pair rows
+        idt = torch.tensor([ids, prs] if prs else ids, dtype=torch.int64)      # [T], or [2, T] with pair rows or positions
         if self.use_graph and collect is None and len(ids) == len(seqs) and rows == list(range(len(seqs))):
             logits = self._decode_step(seqs, idt)
         else:
@@ -592,12 +725,18 @@ class RaggedDecoder:
             return self._delta(li, m, lt, P, meta)
         if isinstance(m, SideBySide):
             return self._side_by_side(li, m, lt, P, meta)
+        if isinstance(m, GatedDelta):
+            return self._gated_delta(li, m, lt, P, meta)
+        if isinstance(m, SelectiveScan):
+            return self._selective(li, m, lt, P, meta)
         return self._hgrn2(li, m, lt, P, meta)
 
     def _forward(self, meta, idt, rows, collect):
         cfg, ops = self.cfg, self.ops
         if cfg.pair_embed is not None:
             x = ops.embed_rows(idt[0], self.embed, idt[1], self.pair_table, cfg.embed_scale)
+        elif cfg.positions:
+            x = ops.embed_rows(idt[0], self.embed, idt[1], self.pos_table, cfg.embed_scale)
         else:
             x = ops.embed_rows(idt, self.embed, scale=cfg.embed_scale)
         if cfg.block == "sandwich":
@@ -606,6 +745,8 @@ class RaggedDecoder:
             x = self._parallel_layers(x, meta, collect)
         elif cfg.block == "pre_norm":
             x = self._prenorm_layers(x, meta, collect)
+        elif cfg.block == "output_norm":
+            self._outnorm_layers(x, meta, collect)
         else:
             xa = x.to(self.act)
             for ri, li in enumerate(self.runs):
@@ -625,8 +766,11 @@ class RaggedDecoder:
             xr = x                                # (the final norm writes its own output)
         else:
             xr = x[torch.tensor(rows, dtype=torch.int64, device=self.device)].contiguous()
-        xo = torch.empty_like(xr)
-        xa = ops.sum_group_norm(xr, None, self.final_norm, cfg.norm_groups, 1.0, cfg.norm_eps, self.act, x_out=xo)
+        if cfg.block == "output_norm":
+            xa = ops.ln_add(xr, None, self.final_norm, self.final_norm_bias, cfg.norm_eps, self.act)
+        else:
+            xo = torch.empty_like(xr)
+            xa = ops.sum_group_norm(xr, None, self.final_norm, cfg.norm_groups, 1.0, cfg.norm_eps, self.act, x_out=xo)
         logits = F.linear(xa, self.head).float()
         if cfg.logit_softcap > 0:
             logits = torch.tanh(logits / cfg.logit_softcap) * cfg.logit_softcap
@@ -708,6 +852,39 @@ class RaggedDecoder:
                 collect.append(X.sum(1))
         return ops.hc_step(X, y, prev, self._sum_read, None, eps, self.act, want_u=True)[1]
 
+    def _outnorm_layers(self, x, meta, collect):
+        """x <- x + LN(mixer(h)), h = x + conv(x), then x <- x + LN(ff(x)) for every execution; x float32, in place.  The norm, the
+        residual sum and the next sublayer's operand are one kernel; in a step of single tokens so is the convolution of the
+        stream in front of the next mixer (prompt portions need their neighbours' rows first and get a kernel for it)."""
+        cfg, ops, eps, pool = self.cfg, self.ops, self.cfg.norm_eps, self.pool
+        n, taps = len(self.runs), cfg.stream_conv
+
+        def operand(ri):                             # what execution ri's mixer reads, from the stream as it is
+            if not taps:
+                return x.to(self.act)
+            return ops.conv_rows(x, 0, self.layers[self.runs[ri]].stream_conv, None, pool.stream_tail.get(ri), meta, self.act, add=True)
+
+        def join(y, w, b, ri):                       # x <- x + LN(y); returns the operand of execution ri's mixer (None behind the last)
+            if taps and meta.single and ri < n:
+                return ops.ln_add(x, y, w, b, eps, self.act, cw=self.layers[self.runs[ri]].stream_conv, tail=pool.stream_tail.get(ri), meta=meta)
+            xa = ops.ln_add(x, y, w, b, eps, self.act, want=not taps and ri < n)
+            return operand(ri) if taps and ri < n else xa
+
+        xa = operand(0) if n else None
+        for ri, li in enumerate(self.runs):
+            m, mlp, lt = cfg.mixers[li], cfg.mlps[li], self.layers[li]
+            y = F.linear(self._mixer(ri, m, lt, F.linear(xa, lt.w_in, lt.b_in), meta), lt.w_out)
+            if mlp is None:
+                xa = join(y, lt.norm1, lt.norm1_bias, ri + 1)
+            elif isinstance(mlp, DenseMlp):
+                a = F.linear(ops.ln_add(x, y, lt.norm1, lt.norm1_bias, eps, self.act), lt.w_ff)
+                y = F.linear(ops.act_cols(a, 0, mlp.ff, mlp.act, lt.act_params or (0.0, 0.0)), lt.w_down, lt.b_down)
+                xa = join(y, lt.norm2, lt.norm2_bias, ri + 1)
+            else:
+                raise ValueError("the output-norm block has no such feed-forward yet")
+            if collect is not None:
+                collect.append(x.clone())
+
     def _linear_f32(self, a, w):
         """a w^T with the operands in the activation type and a float32 result (no rounding of the 32-bit accumulator)"""
         if a.dtype == torch.float32 or a.device.type != "cuda":
@@ -739,7 +916,7 @@ class RaggedDecoder:
         return out
 
     def weight_bytes(self):
-        ts = [self.embed, self.head, self.final_norm] + [t for t in (self.pair_table, self.w_mix) if t is not None]
+        ts = [self.embed, self.head, self.final_norm] + [t for t in (self.pair_table, self.w_mix, self.pos_table) if t is not None]
         for lt in self.layers:
             ts += [t for t in vars(lt).values() if isinstance(t, torch.Tensor)]
         return sum(t.numel() * t.element_size() for t in ts)

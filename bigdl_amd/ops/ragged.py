@@ -96,6 +96,26 @@ class _AttnArgs(ctypes.Structure):
                 ("slopes", ctypes.c_void_p)]
 
 
+class _QkvRowsArgs(ctypes.Structure):
+    _fields_ = [("P", ctypes.c_void_p), ("ldp", ctypes.c_int64)] + [(n, ctypes.c_int) for n in ("H", "G", "d", "vd")] + \
+               [("qw", ctypes.c_void_p), ("kw", ctypes.c_void_p), ("eps", ctypes.c_float), ("rot", ctypes.c_int),
+                ("cossin", ctypes.c_void_p), ("q_out", ctypes.c_void_p), ("kpages", ctypes.c_void_p), ("vpages", ctypes.c_void_p),
+                ("v_norm", ctypes.c_int), ("first_in", ctypes.c_void_p), ("first_out", ctypes.c_void_p), ("lam", ctypes.c_float)]
+
+
+class _GatedDeltaArgs(ctypes.Structure):
+    _fields_ = [("P", ctypes.c_void_p), ("ldp", ctypes.c_int64), ("cw", ctypes.c_void_p), ("taps", ctypes.c_int), ("state", ctypes.c_void_p),
+                ("b0", ctypes.c_int), ("a0", ctypes.c_int), ("arate", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p), ("tiny", ctypes.c_float)] + \
+               [(n, ctypes.c_void_p) for n in ("qf", "kf", "vo", "gb")] + [(n, ctypes.c_int) for n in ("H", "G", "d", "vd", "write_state")]
+
+
+class _SelScanArgs(ctypes.Structure):
+    _fields_ = [("x", ctypes.c_void_p), ("ldx", ctypes.c_int64), ("dt", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p), ("bc", ctypes.c_void_p),
+                ("ldbc", ctypes.c_int64), ("b0", ctypes.c_int), ("c0", ctypes.c_int), ("A", ctypes.c_void_p), ("D", ctypes.c_void_p),
+                ("z", ctypes.c_void_p), ("ldz", ctypes.c_int64), ("z0", ctypes.c_int), ("state", ctypes.c_void_p), ("out", ctypes.c_void_p),
+                ("sum_dt", ctypes.c_void_p), ("C", ctypes.c_int), ("N", ctypes.c_int), ("keep_end", ctypes.c_int)]
+
+
 def lib():
     global _LIB
     if _LIB is None:
@@ -112,7 +132,7 @@ def lib():
         L.ragged_post_norm_add.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, ci, vp]
         L.ragged_mlstm_gates.argtypes = [vp, i64, ci, vp, cf, cf, vp, vp, vp, vp, ci, _Batch, ci, vp]
         L.ragged_mlstm_expand.argtypes = [vp, i64, ci, ci, vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
-        L.ragged_head_norm_gate.argtypes = [vp, vp, vp, i64, ci, vp, i64, ci, ci, cf, ci, vp, cf, cf, ci, vp]
+        L.ragged_head_norm_gate.argtypes = [vp, vp, vp, i64, ci, vp, i64, ci, ci, cf, ci, vp, cf, cf, ci, ci, vp]
         L.ragged_moe_route.argtypes = [vp, i64, vp, vp, vp, i64, ci, ci, ci, ci, ci, cf, ci, ci, ci, ci, vp]
         L.ragged_embed_rows.argtypes = [vp, vp, vp, vp, cf, vp, i64, ci, ci, vp]
         L.ragged_add_norm.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, ci, vp]
@@ -121,6 +141,13 @@ def lib():
         L.ragged_gate_cols.argtypes = [vp, vp, i64, ci, vp, i64, ci, cf, ci, vp]
         L.ragged_delta_gates.argtypes = [vp, i64, ci, ci, ci, vp, vp, vp, cf, cf, vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
         L.ragged_delta_scan.argtypes = [vp, vp, vp, vp, vp, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
+        L.ragged_gated_delta_prep.argtypes = [_GatedDeltaArgs, _Batch, ci, vp]
+        L.ragged_gated_delta_scan.argtypes = [vp, vp, vp, ci, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
+        L.ragged_conv_rows.argtypes = [vp, i64, ci, vp, vp, vp, ci, ci, vp, ci, ci, ci, _Batch, ci, ci, vp]
+        L.ragged_ln_add.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, vp, ci, vp, _Batch, ci, vp]
+        L.ragged_qkv_rows.argtypes = [_QkvRowsArgs, _Batch, ci, vp]
+        L.ragged_selective_scan.argtypes = [_SelScanArgs, _Batch, ci, ci, vp]
+        L.ragged_selective_chain.argtypes = [vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, vp]
         L.ragged_delta_chain_ok.argtypes = [ci]
         L.ragged_delta_chain.argtypes = [vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, vp]
         L.ragged_glu_pairs.argtypes = [vp, i64, vp, i64, ci, ci, vp]
@@ -153,6 +180,8 @@ class BatchMeta:
         self.device = device
         self.B = len(seqs)
         self.T = sum(n for _, _, n, _ in seqs)
+        self.single = self.T == self.B          # every sequence brings exactly one row
+        self.shared = {}                        # what one layer's mixer leaves for later layers of the same step
         self.max_pages = max_pages or max(1, max(len(pg) for *_, pg in seqs))
         T, B = self.T, self.B
         self._static = static
@@ -527,9 +556,9 @@ class HipOps:
             _ok(lib().ragged_relu2(A.data_ptr(), out.data_ptr(), A.numel(), _DT[A.dtype], _stream()), "relu2")
         return out
 
-    def head_norm_gate(self, o, w, P, g0, H, vd, eps, act, em=None, den_floor=0.0, scale=1.0):
-        """each head's rows of ``o`` divided by their root mean square, times ``w``, times sigmoid(gate columns of P), times
-        ``scale``.  With ``em`` [T, H]: ``o`` has vd + 1 columns per head and is first divided by max(|last column|, em) +
+    def head_norm_gate(self, o, w, P, g0, H, vd, eps, act, em=None, den_floor=0.0, scale=1.0, gate="sigmoid"):
+        """each head's rows of ``o`` divided by their root mean square, times ``w``, times sigmoid (``gate`` "silu": silu) of the
+        gate columns of P, times ``scale``.  With ``em`` [T, H]: ``o`` has vd + 1 columns per head and is first divided by max(|last column|, em) +
         den_floor."""
         _f32(o, w, em)
         _act(P)
@@ -540,7 +569,8 @@ class HipOps:
             raise ValueError("head outputs / gate columns do not fit")
         out = torch.empty(T, H * vd, dtype=act, device=o.device)
         _ok(lib().ragged_head_norm_gate(o.data_ptr(), w.data_ptr(), P.data_ptr(), P.stride(0), g0, out.data_ptr(), T, H, vd, eps,
-                                        ldo, None if em is None else em.data_ptr(), den_floor, float(scale), _DT[act],
+                                        ldo, None if em is None else em.data_ptr(), den_floor, float(scale),
+                                        {"sigmoid": 0, "silu": 1}[gate], _DT[act],
                                         _stream()), "head_norm_gate")
         return out
 
@@ -787,28 +817,50 @@ class HipOps:
         if any(a.shape != (meta.T, H * d) for a in arrays) or v0 + H * vd > P.shape[1] or P.shape[0] != meta.T \
                 or state.shape[1:] != (H, d, vd) or max(s[0] for s in meta.seqs) >= state.shape[0]:
             raise ValueError("recurrent state / scan arrays do not fit")
-        out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=P.device)
         L, dt, st = lib(), _DT[P.dtype], _stream()
         ptrs = [a.data_ptr() for a in arrays]
+
+        def scan(states, out, cols, values, batch, what):
+            _ok(L.ragged_delta_scan(*ptrs, P.data_ptr() if values else None, P.stride(0), v0, states.data_ptr(),
+                                    None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt, st), what)
+        return self._delta_passes(scan, state, H, d, vd, meta)
+
+    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta):
+        """S' = g S, u = beta (v - S'^T k), S <- S' + k u^T, o = S^T q per head (head h reads q / k head h / (H / G)): ``qf``,
+        ``kf`` [T, G d], ``gb`` [T, H, 2] = (g, beta), values V [T, H vd], ``state`` float [slots, H, d, vd]."""
+        _f32(qf, kf, gb, state)
+        _act(V)
+        if G <= 0 or H % G or qf.shape != (meta.T, G * d) or kf.shape != qf.shape or gb.shape != (meta.T, H, 2) \
+                or V.shape != (meta.T, H * vd) or state.shape[1:] != (H, d, vd) or max(s[0] for s in meta.seqs) >= state.shape[0]:
+            raise ValueError("recurrent state / scan arrays do not fit")
+        L, dt, st = lib(), _DT[V.dtype], _stream()
+
+        def scan(states, out, cols, values, batch, what):
+            _ok(L.ragged_gated_delta_scan(qf.data_ptr(), kf.data_ptr(), gb.data_ptr(), G, V.data_ptr() if values else None, V.stride(0), 0,
+                                          states.data_ptr(), None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt,
+                                          st), what)
+        return self._delta_passes(scan, state, H, d, vd, meta)
+
+    def _delta_passes(self, scan, state, H, d, vd, meta):
+        """``scan(states, out or None, columns, with values, batch, name)``: one pass of either delta rule"""
+        L, st, device = lib(), _stream(), state.device
+        out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=device)
         longest = max(n for _, _, n, _ in meta.seqs)
         if longest < self.delta_chunked_from:
-            _ok(L.ragged_delta_scan(*ptrs, P.data_ptr(), P.stride(0), v0, state.data_ptr(), out.data_ptr(), H, d, vd, 1, meta.c(),
-                                    dt, st), "delta_scan")
+            scan(state, out, vd, True, meta.c(), "delta_scan")
             return out
         # Long portions: chunks side by side.  A chunk maps its start state linearly, S_end = A S_start + L: L is the chunk
         # scanned from zero, A (d x d per head) the chunk scanned without inputs from the identity.  The chunk-start states
         # follow one after the other from those, and the chunks are scanned again from them for the outputs.
         nc, cstart, zeros, ones, cid, cfirst, last = meta.chunks(self._delta_chunk_length(meta, H, d, vd))
-        local = torch.empty(nc, H, d, vd, dtype=torch.float32, device=P.device)
-        trans = torch.eye(d, dtype=torch.float32, device=P.device).repeat(nc, H, 1, 1)
+        local = torch.empty(nc, H, d, vd, dtype=torch.float32, device=device)
+        trans = torch.eye(d, dtype=torch.float32, device=device).repeat(nc, H, 1, 1)
         begin = torch.empty_like(local)
 
         def chunk_batch(past):
             return _Batch(None, None, cstart.data_ptr(), past.data_ptr(), cid.data_ptr(), None, meta.T, nc, 0)
-        _ok(L.ragged_delta_scan(*ptrs, P.data_ptr(), P.stride(0), v0, local.data_ptr(), None, H, d, vd, 1, chunk_batch(zeros), dt, st),
-            "delta_scan (chunks from zero)")
-        _ok(L.ragged_delta_scan(*ptrs, None, 0, 0, trans.data_ptr(), None, H, d, d, 0, chunk_batch(ones), dt, st),
-            "delta_scan (transition matrices)")
+        scan(local, None, vd, True, chunk_batch(zeros), "delta_scan (chunks from zero)")
+        scan(trans, None, d, False, chunk_batch(ones), "delta_scan (transition matrices)")
         if self.delta_chain and L.ragged_delta_chain_ok(d):
             _ok(L.ragged_delta_chain(state.data_ptr(), local.data_ptr(), trans.data_ptr(), begin.data_ptr(), cfirst.data_ptr(),
                                      meta.seq_past.data_ptr(), meta.seq_slot.data_ptr(), meta.B, H, d, vd, st), "delta_chain")
@@ -816,18 +868,160 @@ class HipOps:
             first = [0]
             for _, _, n, _ in meta.seqs:
                 first.append(last[len(first) - 1] + 1)
-            slots = torch.tensor([s[0] for s in meta.seqs], dtype=torch.int64, device=P.device)
-            fresh = torch.tensor([s[1] == 0 for s in meta.seqs], device=P.device)
-            S = torch.where(fresh[:, None, None, None], torch.zeros((), device=P.device), state[slots])      # [B, H, d, vd]
+            slots = torch.tensor([s[0] for s in meta.seqs], dtype=torch.int64, device=device)
+            fresh = torch.tensor([s[1] == 0 for s in meta.seqs], device=device)
+            S = torch.where(fresh[:, None, None, None], torch.zeros((), device=device), state[slots])        # [B, H, d, vd]
             for j in range(max(first[b + 1] - first[b] for b in range(meta.B))):     # the j-th chunk of every sequence that has one
                 bs = [b for b in range(meta.B) if first[b + 1] - first[b] > j]
-                cs = torch.tensor([first[b] + j for b in bs], dtype=torch.int64, device=P.device)
-                bi = torch.tensor(bs, dtype=torch.int64, device=P.device)
+                cs = torch.tensor([first[b] + j for b in bs], dtype=torch.int64, device=device)
+                bi = torch.tensor(bs, dtype=torch.int64, device=device)
                 begin[cs] = S[bi]
                 S[bi] = torch.matmul(trans[cs], S[bi]) + local[cs]
             state[slots] = S
-        _ok(L.ragged_delta_scan(*ptrs, P.data_ptr(), P.stride(0), v0, begin.data_ptr(), out.data_ptr(), H, d, vd, 1,
-                                chunk_batch(ones), dt, st), "delta_scan (chunks from their start states)")
+        scan(begin, out, vd, True, chunk_batch(ones), "delta_scan (chunks from their start states)")
+        return out
+
+    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta):
+        """Inputs of ``gated_delta_scan`` from this step's projections, columns q [G d] | k [G d] | v [H vd] of P behind a causal
+        convolution (``cw`` [channels, taps], older inputs in ``tail`` [slots, taps - 1, channels]) and silu: (unit q times
+        d^-1/2, unit k, values of P's type, (exp(-arate softplus(a + dt_bias)), sigmoid(b)) with a, b = columns a0 .., b0 ..).
+        The tail moves on."""
+        _act(P, tail)
+        _f32(cw, arate, dt_bias)
+        C = 2 * G * d + H * vd
+        if P.dim() != 2 or P.shape[0] != meta.T or min(b0, a0) < C or max(b0, a0) + H > P.shape[1] or cw.shape != (C, taps) \
+                or arate.numel() != H or dt_bias.numel() != H or H % G:
+            raise ValueError("delta-rule columns / taps / gates do not fit")
+        self._tail_check(tail, taps, C, P.dtype, meta)
+        dev = P.device
+        qf = torch.empty(meta.T, G * d, dtype=torch.float32, device=dev)
+        kf = torch.empty_like(qf)
+        vo = torch.empty(meta.T, H * vd, dtype=P.dtype, device=dev)
+        gb = torch.empty(meta.T, H, 2, dtype=torch.float32, device=dev)
+        a = _GatedDeltaArgs(P.data_ptr(), P.stride(0), cw.data_ptr(), taps, None if tail is None else tail.data_ptr(), b0, a0,
+                            arate.data_ptr(), dt_bias.data_ptr(), float(tiny), qf.data_ptr(), kf.data_ptr(), vo.data_ptr(), gb.data_ptr(),
+                            H, G, d, vd, int(meta.single))
+        _ok(lib().ragged_gated_delta_prep(a, meta.c(), _DT[P.dtype], _stream()), "gated_delta_prep")
+        if taps > 1 and not meta.single:
+            self.conv_state(P, 0, tail, taps, C, meta)
+        return qf, kf, vo, gb
+
+    @staticmethod
+    def _tail_check(tail, taps, C, dtype, meta):
+        if taps < 1 or taps > 16 or (taps > 1 and (tail is None or tail.dtype != dtype or tail.shape[1:] != (taps - 1, C)
+                                                   or not tail.is_contiguous() or max(s[0] for s in meta.seqs) >= tail.shape[0])):
+            raise ValueError("convolution state does not fit")
+
+    def conv_rows(self, src, col0, cw, bias, tail, meta, act, add=False, silu=False):
+        """Causal convolution per channel of the columns col0 .. of ``src`` (the float stream or projections of type ``act``):
+        silu(conv + bias), src + conv (``add``) or conv, as ``act`` [T, channels]; the tail moves on."""
+        _act(src, tail)
+        _f32(cw, bias)
+        C, taps = cw.shape
+        if src.dim() != 2 or src.shape[0] != meta.T or col0 < 0 or col0 + C > src.shape[1] or src.dtype not in (act, torch.float32) \
+                or (bias is not None and bias.numel() != C):
+            raise ValueError("convolved columns / taps do not fit")
+        self._tail_check(tail, taps, C, src.dtype, meta)
+        out = torch.empty(meta.T, C, dtype=act, device=src.device)
+        _ok(lib().ragged_conv_rows(src.data_ptr(), src.stride(0), col0, cw.data_ptr(), None if bias is None else bias.data_ptr(),
+                                   None if tail is None else tail.data_ptr(), taps, C, out.data_ptr(), int(add), int(silu),
+                                   int(meta.single), meta.c(), _DT[src.dtype], _DT[act], _stream()), "conv_rows")
+        if taps > 1 and not meta.single:
+            self.conv_state(src, col0, tail, taps, C, meta)
+        return out
+
+    def ln_add(self, x, y, w, b, eps, act, want=True, cw=None, tail=None, meta=None):
+        """x <- x + LN(y) in place on the float stream; returns x as ``act`` (``want``), or with ``cw`` (a step of single tokens)
+        the stream plus its causal convolution, whose older inputs ``tail`` holds (it moves on).  y None: LN(x), x unchanged."""
+        _f32(x, w, b, cw, tail)
+        _act(y)
+        rows, D = x.shape
+        if (y is not None and (y.shape != x.shape or not y.is_contiguous() or y.dtype != act)) or w.numel() != D or b.numel() != D:
+            raise ValueError("sublayer output / norm weights do not fit the stream")
+        taps = 0
+        if cw is not None:
+            taps = cw.shape[1]
+            if not meta.single or meta.T != rows or cw.shape[0] != D or y is None or not want:
+                raise ValueError("the convolution of the stream is part of this pass only in a step of single tokens")
+            self._tail_check(tail, taps, D, torch.float32, meta)
+        xa = torch.empty(rows, D, dtype=act, device=x.device) if want else None
+        batch = meta.c() if cw is not None else _Batch(None, None, None, None, None, None, rows, rows, 0)
+        _ok(lib().ragged_ln_add(x.data_ptr(), None if y is None else y.data_ptr(), w.data_ptr(), b.data_ptr(),
+                                None if xa is None else xa.data_ptr(), rows, D, eps, None if cw is None else cw.data_ptr(), taps,
+                                None if tail is None else tail.data_ptr(), batch, _DT[act], _stream()), "ln_add")
+        return xa
+
+    def qkv_rows(self, P, qw, kw, eps, rot, inv_freq, kpages, vpages, meta, *, H, G, d, vd, v_norm=False, first_in=None, lam=0.0,
+                 want_first=False):
+        """Columns q [H d] | k [G d] | v [G vd] of P: q and k RMS-normed over the whole projection with a weight per channel, the
+        first ``rot`` channels of every head turned (pairs i, i + rot / 2); values RMS-normed per head (``v_norm``) and mixed with
+        ``first_in`` [T, G vd] as (1 - lam) v + lam first.  Keys and values go to their pages; returns (q float [T, H d], the
+        values as float if ``want_first`` else None)."""
+        _act(P, kpages, vpages)
+        _f32(qw, kw, inv_freq, first_in)
+        _page_check(meta, kpages)
+        _page_check(meta, vpages)
+        if P.dim() != 2 or P.shape[0] != meta.T or (H + G) * d + G * vd > P.shape[1] or qw.numel() != H * d or kw.numel() != G * d \
+                or kpages.shape[1:] != (G, PAGE, d) or vpages.shape[1:] != (G, PAGE, vd) or kpages.dtype != P.dtype or vpages.dtype != P.dtype \
+                or (first_in is not None and first_in.shape != (meta.T, G * vd)) or (rot and (inv_freq.numel() != rot // 2 or rot > d)):
+            raise ValueError("projections / norm weights / cache pages do not fit the head layout")
+        q = torch.empty(meta.T, H * d, dtype=torch.float32, device=P.device)
+        first = torch.empty(meta.T, G * vd, dtype=torch.float32, device=P.device) if want_first else None
+        a = _QkvRowsArgs(P.data_ptr(), P.stride(0), H, G, d, vd, qw.data_ptr(), kw.data_ptr(), eps, rot,
+                         meta.cossin(inv_freq).data_ptr() if rot else None, q.data_ptr(), kpages.data_ptr(), vpages.data_ptr(),
+                         int(bool(v_norm)), None if first_in is None else first_in.data_ptr(),
+                         None if first is None else first.data_ptr(), float(lam))
+        _ok(lib().ragged_qkv_rows(a, meta.c(), _DT[P.dtype], _stream()), "qkv_rows")
+        return q, first
+
+    selective_chunked_from = 128  # portions of at least this many tokens run the selective scan in chunks
+    selective_waves = 2048        # wavefronts of a pass that the chunk length aims at (eight per CU)
+
+    @staticmethod
+    def _states_per_lane(N, long):
+        """registers of state per lane: many for long portions (less work per state), few for single tokens (more lanes)"""
+        ns = 4
+        while (long and ns < 16 and ns < N) or (N > 64 * ns):
+            ns *= 2
+        return ns
+
+    def selective_scan(self, x, dt, dt_bias, M, b0, c0, A, D, P, z0, state, meta):
+        """S <- exp(d A) S + d x B, y = S C + D x, d = softplus(dt + dt_bias), per channel and state; returns y * silu(z) as x's
+        type.  x [T, C], dt float [T, C], B / C = columns b0 .. / c0 .. of M, z = columns z0 .. of P, A float [C, N] = log2(e) times
+        the (negative) rates, ``state`` float [slots, 1, C, N]."""
+        _act(x, M, P)
+        _f32(dt, dt_bias, A, D, state)
+        C, N = A.shape
+        if x.shape != (meta.T, C) or dt.shape != x.shape or M.shape[0] != meta.T or max(b0, c0) + N > M.shape[1] or P.shape[0] != meta.T \
+                or z0 + C > P.shape[1] or M.dtype != x.dtype or P.dtype != x.dtype or dt_bias.numel() != C or D.numel() != C \
+                or state.shape[1:] != (1, C, N) or max(s[0] for s in meta.seqs) >= state.shape[0] or N > 1024:
+            raise ValueError("recurrent state / scan inputs do not fit")
+        L, cdt, st = lib(), _DT[x.dtype], _stream()
+        out = torch.empty(meta.T, C, dtype=x.dtype, device=x.device)
+        a = _SelScanArgs(x.data_ptr(), x.stride(0), dt.data_ptr(), dt_bias.data_ptr(), M.data_ptr(), M.stride(0), b0, c0, A.data_ptr(),
+                         D.data_ptr(), P.data_ptr(), P.stride(0), z0, state.data_ptr(), out.data_ptr(), None, C, N, 1)
+        longest = max(n for _, _, n, _ in meta.seqs)
+        if longest < self.selective_chunked_from:
+            _ok(L.ragged_selective_scan(a, meta.c(), self._states_per_lane(N, longest >= 32), cdt, st), "selective_scan")
+            return out
+        # long portions: chunks from zero side by side, their start states from the chunks' decays, chunks again for the outputs
+        ns = self._states_per_lane(N, True)
+        waves = -(-C * (1 << max(0, -(-N // ns) - 1).bit_length()) // 64)
+        length = 32
+        while length < 256 and -(-meta.T // length) * waves > self.selective_waves:
+            length *= 2
+        nc, cstart, zeros, ones, cid, cfirst, _ = meta.chunks(length)
+        local = torch.empty(nc, C, N, dtype=torch.float32, device=x.device)
+        sums = torch.empty(nc, C, dtype=torch.float32, device=x.device)
+
+        def chunk_batch(past):
+            return _Batch(None, None, cstart.data_ptr(), past.data_ptr(), cid.data_ptr(), None, meta.T, nc, 0)
+        a.state, a.out, a.sum_dt = local.data_ptr(), None, sums.data_ptr()
+        _ok(L.ragged_selective_scan(a, chunk_batch(zeros), ns, cdt, st), "selective_scan (chunks from zero)")
+        _ok(L.ragged_selective_chain(state.data_ptr(), local.data_ptr(), sums.data_ptr(), A.data_ptr(), cfirst.data_ptr(),
+                                     meta.seq_past.data_ptr(), meta.seq_slot.data_ptr(), meta.B, C, N, st), "selective_chain")
+        a.out, a.sum_dt, a.keep_end = out.data_ptr(), None, 0
+        _ok(L.ragged_selective_scan(a, chunk_batch(ones), ns, cdt, st), "selective_scan (chunks from their start states)")
         return out
 
 
@@ -988,12 +1182,13 @@ class TorchOps:
     def relu2(self, A):
         return torch.relu(A.float()).pow(2).to(A.dtype)
 
-    def head_norm_gate(self, o, w, P, g0, H, vd, eps, act, em=None, den_floor=0.0, scale=1.0):
+    def head_norm_gate(self, o, w, P, g0, H, vd, eps, act, em=None, den_floor=0.0, scale=1.0, gate="sigmoid"):
         v = o.view(o.shape[0], H, -1)
         if em is not None:
             v = v[..., :vd] / (torch.maximum(v[..., vd].abs(), em) + den_floor)[..., None]
         v = (v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)).reshape(-1, H * vd)
-        return (v * w * scale * torch.sigmoid(P[:, g0:g0 + H * vd].float())).to(act)
+        z = P[:, g0:g0 + H * vd].float()
+        return (v * w * scale * (F.silu(z) if gate == "silu" else torch.sigmoid(z))).to(act)
 
     def mlstm_gates(self, P, i0, gate_bias, cap, m_start, H, mstate, meta):
         li = cap * torch.tanh((P[:, i0:i0 + H].float() + gate_bias[:H]) / cap)
@@ -1109,6 +1304,80 @@ class TorchOps:
                 out[t] = (S * rf[t].view(H, d, 1)).sum(1).reshape(-1)
             state[slot] = S
         return out
+
+    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta):
+        C, T = 2 * G * d + H * vd, meta.T
+        u = F.silu(self._segment(P, 0, meta, cw, taps, C, 0, tail, C))
+        if taps > 1:
+            self.conv_state(P, 0, tail, taps, C, meta)
+        unit = lambda v: (v / torch.sqrt(v.pow(2).sum(-1, keepdim=True) + tiny)).reshape(T, G * d)      # noqa: E731
+        g = torch.exp(-arate * F.softplus(P[:, a0:a0 + H].float() + dt_bias, threshold=80.0))
+        return unit(u[:, :G * d].reshape(T, G, d)) * d ** -0.5, unit(u[:, G * d:2 * G * d].reshape(T, G, d)), u[:, 2 * G * d:].to(P.dtype), \
+            torch.stack([g, torch.sigmoid(P[:, b0:b0 + H].float())], -1)
+
+    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta):
+        out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=V.device)
+        for b, (slot, past, n, _) in enumerate(meta.seqs):
+            S = state[slot].clone() if past > 0 else torch.zeros_like(state[slot])
+            for t in range(meta.start[b], meta.start[b] + n):
+                q, k = (a[t].view(G, d, 1).repeat_interleave(H // G, 0) for a in (qf, kf))
+                S = gb[t, :, 0].view(H, 1, 1) * S
+                S = S + k * (gb[t, :, 1].view(H, 1, 1) * (V[t].float().view(H, 1, vd) - (S * k).sum(1, keepdim=True)))
+                out[t] = (S * q).sum(1).reshape(-1)
+            state[slot] = S
+        return out
+
+    def conv_rows(self, src, col0, cw, bias, tail, meta, act, add=False, silu=False):
+        C, taps = cw.shape
+        u = self._segment(src, col0, meta, cw, taps, C, 0, tail, C)
+        if taps > 1:
+            self.conv_state(src, col0, tail, taps, C, meta)
+        if bias is not None:
+            u = u + bias
+        if silu:
+            u = F.silu(u)
+        return (src[:, col0:col0 + C].float() + u if add else u).to(act)
+
+    def ln_add(self, x, y, w, b, eps, act, want=True, cw=None, tail=None, meta=None):
+        v = F.layer_norm((x if y is None else y).float(), (x.shape[1],), w, b, eps)
+        if y is None:
+            return v.to(act)
+        x += v
+        if cw is not None:
+            return self.conv_rows(x, 0, cw, None, tail, meta, act, add=True)
+        return x.to(act) if want else None
+
+    def qkv_rows(self, P, qw, kw, eps, rot, inv_freq, kpages, vpages, meta, *, H, G, d, vd, v_norm=False, first_in=None, lam=0.0,
+                 want_first=False):
+        u = P.float()
+        nq, nk = H * d, G * d
+        rms = lambda v: v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)       # noqa: E731
+        qk = torch.cat([rms(u[:, :nq]) * qw, rms(u[:, nq:nq + nk]) * kw], 1).contiguous()
+        none = dict(cw=None, taps=0, C=0, ch0=0, state=None, normw=None, eps=eps)
+        q = torch.empty(meta.T, nq, dtype=torch.float32)
+        k = torch.empty(meta.T, nk, dtype=torch.float32)
+        self.conv_head(qk, 0, meta, ngroups=H, gsize=d, rot=rot, inv_freq=inv_freq, out_dense=q, **none)
+        self.conv_head(qk, nq, meta, ngroups=G, gsize=d, rot=rot, inv_freq=inv_freq, out_dense=k, **none)
+        v = u[:, nq + nk:nq + nk + G * vd].reshape(meta.T, G, vd)
+        v = (rms(v) if v_norm else v).reshape(meta.T, G * vd)
+        if first_in is not None:
+            v = (1.0 - lam) * v + lam * first_in
+        for rows, n, pages in ((k, d, kpages), (v.contiguous(), vd, vpages)):
+            self.conv_head(rows, 0, meta, ngroups=G, gsize=n, rot=0, inv_freq=None, pages=pages, **none)
+        return q, (v if want_first else None)
+
+    def selective_scan(self, x, dt, dt_bias, M, b0, c0, A, D, P, z0, state, meta):
+        C, N = A.shape
+        out = torch.empty(meta.T, C, dtype=torch.float32, device=x.device)
+        d = F.softplus(dt + dt_bias, threshold=80.0)
+        for b, (slot, past, n, _) in enumerate(meta.seqs):
+            S = state[slot, 0].clone() if past > 0 else torch.zeros_like(state[slot, 0])
+            for t in range(meta.start[b], meta.start[b] + n):
+                xt = x[t].float()
+                S = torch.exp2(d[t][:, None] * A) * S + (d[t] * xt)[:, None] * M[t, b0:b0 + N].float()
+                out[t] = S @ M[t, c0:c0 + N].float() + D * xt
+            state[slot, 0] = S
+        return (out * F.silu(P[:, z0:z0 + C].float())).to(x.dtype)
 
 
 def ops_for(device) -> object:

@@ -121,6 +121,9 @@ class ContinuousBatcher:
         if len(req.input_ids) + req.max_new_tokens > capacity:
             raise ValueError(f"request {req.request_id}: prompt + max_new_tokens exceeds the "
                              f"{'page pool' if self.ragged else 'slot capacity'} ({capacity})")
+        positions = getattr(self.engine, "max_positions", None)       # a learned position table ends somewhere
+        if positions and len(req.input_ids) + req.max_new_tokens - 1 > positions:      # (the last token is not fed back)
+            raise ValueError(f"request {req.request_id}: prompt + max_new_tokens exceeds the model's {positions} positions")
         if isinstance(req.eos_token_id, int):
             req.eos_token_id = [req.eos_token_id]
         self.waiting.append(req)
