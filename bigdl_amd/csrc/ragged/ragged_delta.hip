@@ -59,7 +59,8 @@ extern "C" int ragged_delta_gates(const void* P, int64_t ldp, int r0, int k0, in
 // behind a short causal convolution and silu): qf = unit(q) * d^(-1/2), kf = unit(k), float [rows, G d] each, with unit(u) =
 // u / sqrt(|u|^2 + tiny); vo of type T [rows, H vd]; gb float [rows, H, 2] = (exp(-arate softplus(a + dt bias)), sigmoid(b)).
 // The inputs before this step come from `state` [slots, taps - 1, C]; `write_state` (every sequence brings exactly one row)
-// also shifts it.  One wavefront per (row, item): 2 G unit vectors, blocks of 256 value channels, the gates.
+// also shifts it.  One wavefront per (block of rows, item): 2 G unit vectors, blocks
+// of value channels, the gates.
 struct GatedDeltaArgs {
   const void* P;
   int64_t ldp;
@@ -77,52 +78,115 @@ struct GatedDeltaArgs {
   int H, G, d, vd, write_state;
 };
 
-template <typename T>
-__global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a, int items, Batch bt) {
-  extern __shared__ float smem[];
+// K: 64-channel pieces of an item (a unit vector's d <= 64 K); a lane holds one channel of each.  RB rows are walked with the
+// last TAPS - 1 inputs in registers (TAPS = 0: any number of taps, every tap is read where it is needed).
+template <typename T, int K, int TAPS>
+__global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a, int items, int RB, Batch bt) {
+  constexpr int M = TAPS > 1 ? TAPS - 1 : 1, W = TAPS > 0 ? TAPS : 1;
   const int lane = threadIdx.x & 63;
-  float* buf = smem + (threadIdx.x >> 6) * a.d;
   const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (id >= (int64_t)bt.T * items) return;
-  const int t = (int)(id / items), it = (int)(id % items);
-  const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
+  const int t0 = (int)(id / items) * RB, it = (int)(id % items);
+  if (t0 >= bt.T) return;
+  const int t1 = t0 + RB < bt.T ? t0 + RB : bt.T;
   const T* P = (const T*)a.P;
-  const int C = 2 * a.G * a.d + a.H * a.vd, keep = a.taps - 1;
-  T* hist = (T*)a.state + (int64_t)slot * keep * C;
-  auto conv = [&](int ch) {                                  // silu of the convolved channel; with write_state shifts its history
-    float u = 0.f;
-    for (int j = 0; j < a.taps; ++j) {
-      const int back = keep - j, pp = pos - back;
-      T raw = from_f<T>(0.f);
-      if (pp >= past) raw = P[(int64_t)(t - back) * a.ldp + ch];
-      else if (pp >= 0) raw = hist[(int64_t)(pp - past + keep) * C + ch];
-      u += a.cw[(int64_t)ch * a.taps + j] * to_f(raw);
-      if (a.write_state && j > 0) hist[(int64_t)(j - 1) * C + ch] = raw;      // (row j - 1 has been read)
-    }
-    return u / (1.0f + expf(-u));
-  };
-  if (it < 2 * a.G) {
-    const bool isq = it < a.G;
-    float ss = 0.f;
-    for (int c = lane; c < a.d; c += 64) { const float v = conv(it * a.d + c); buf[c] = v; ss += v * v; }
-    float f = 1.0f / sqrtf(wave_sum(ss) + a.tiny);
-    if (isq) f *= 1.0f / sqrtf((float)a.d);
-    float* o = (isq ? a.qf : a.kf) + ((int64_t)t * a.G + (isq ? it : it - a.G)) * a.d;
-    for (int c = lane; c < a.d; c += 64) o[c] = buf[c] * f;          // (what this lane itself has stored)
-  } else if (it < items - 1) {
-    const int c0 = (it - 2 * a.G) * 256;
-    for (int c = c0 + lane; c < c0 + 256 && c < a.H * a.vd; c += 64)
-      ((T*)a.vo)[(int64_t)t * a.H * a.vd + c] = from_f<T>(conv(2 * a.G * a.d + c));
-  } else {
-    const T* row = P + (int64_t)t * a.ldp;
-    for (int h = lane; h < a.H; h += 64) {
+  if (it == items - 1) {                                     // decays and write strengths
+    for (int e = lane; e < (t1 - t0) * a.H; e += 64) {
+      const int t = t0 + e / a.H, h = e % a.H;
+      const T* row = P + (int64_t)t * a.ldp;
       const float z = to_f(row[a.a0 + h]) + a.dt_bias[h];
       const float sp = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
       float* o = a.gb + ((int64_t)t * a.H + h) * 2;
       o[0] = expf(-a.arate[h] * sp);
       o[1] = 1.0f / (1.0f + expf(-to_f(row[a.b0 + h])));
     }
+    return;
   }
+  const int C = 2 * a.G * a.d + a.H * a.vd, taps = TAPS > 0 ? TAPS : a.taps, keep = taps - 1;
+  const bool unit = it < 2 * a.G, isq = it < a.G;
+  const int v0 = (it - 2 * a.G) * 64 * K;                    // a value item's first value channel
+  const int ch0 = unit ? it * a.d : 2 * a.G * a.d + v0;
+  const int width = unit ? a.d : (a.H * a.vd - v0 < 64 * K ? a.H * a.vd - v0 : 64 * K);
+  T* S = (T*)a.state;
+  auto input = [&](int t, int back, int pos, int past, int slot, int ch) -> T {      // (the address is chosen first)
+    const int pp = pos - back;
+    const T* p = P + (int64_t)t * a.ldp + ch;
+    if (pp >= past) p -= back * a.ldp;
+    else if (pp >= 0) p = S + ((int64_t)slot * keep + (pp - past + keep)) * C + ch;
+    T v = *p;
+    if (pp < 0) v = from_f<T>(0.f);
+    return v;
+  };
+  int chs[K];
+  float w[K][W];
+  T hist[K][M];
+#pragma unroll
+  for (int k = 0; k < K; ++k) {
+    const int c = lane + 64 * k;
+    chs[k] = ch0 + (c < width ? c : width - 1);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[k][j] = a.cw[(int64_t)chs[k] * TAPS + j];
+  }
+  for (int t = t0; t < t1; ++t) {
+    const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
+    float u[K], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const T cur = P[(int64_t)t * a.ldp + chs[k]];
+      u[k] = 0.f;
+      const bool ok = lane + 64 * k < width;
+      if (TAPS > 0) {
+        if (TAPS > 1 && (t == t0 || pos == past)) {          // (the same branch for the whole wavefront)
+#pragma unroll
+          for (int j = 0; j < M; ++j) hist[k][j] = input(t, TAPS - 1 - j, pos, past, slot, chs[k]);
+        }
+        if (TAPS > 1) {
+#pragma unroll
+          for (int j = 0; j < M; ++j) u[k] += w[k][j] * to_f(hist[k][j]);
+        }
+        u[k] += w[k][W - 1] * to_f(cur);
+        if (TAPS > 1) {
+#pragma unroll
+          for (int j = 0; j + 1 < M; ++j) hist[k][j] = hist[k][j + 1];
+          hist[k][M - 1] = cur;
+          if (a.write_state && ok) {
+#pragma unroll
+            for (int j = 0; j < M; ++j) S[((int64_t)slot * keep + j) * C + chs[k]] = hist[k][j];
+          }
+        }
+      } else {
+        for (int j = 0; j < taps; ++j) {
+          const T raw = input(t, keep - j, pos, past, slot, chs[k]);
+          u[k] += a.cw[(int64_t)chs[k] * taps + j] * to_f(raw);
+          if (a.write_state && ok && j > 0) S[((int64_t)slot * keep + j - 1) * C + chs[k]] = raw;   // (row j - 1 has been read)
+        }
+      }
+      u[k] = ok ? u[k] / (1.0f + expf(-u[k])) : 0.f;
+      ss += u[k] * u[k];
+    }
+    if (unit) {
+      float f = 1.0f / sqrtf(wave_sum(ss) + a.tiny);
+      if (isq) f *= 1.0f / sqrtf((float)a.d);
+      float* o = (isq ? a.qf : a.kf) + ((int64_t)t * a.G + (isq ? it : it - a.G)) * a.d;
+#pragma unroll
+      for (int k = 0; k < K; ++k)
+        if (lane + 64 * k < width) o[lane + 64 * k] = u[k] * f;
+    } else {
+      T* o = (T*)a.vo + (int64_t)t * a.H * a.vd + v0;
+#pragma unroll
+      for (int k = 0; k < K; ++k)
+        if (lane + 64 * k < width) o[lane + 64 * k] = from_f<T>(u[k]);
+    }
+  }
+}
+
+template <typename T, int K>
+static void launch_gated_prep(GatedDeltaArgs a, Batch bt, hipStream_t st) {
+  const int items = 2 * a.G + (a.H * a.vd + 64 * K - 1) / (64 * K) + 1;
+  const int RB = bt.T >= 512 ? 8 : bt.T >= 64 ? 2 : 1;
+  const int64_t waves = (int64_t)((bt.T + RB - 1) / RB) * items;
+  const dim3 grid((unsigned)((waves + 3) / 4));
+  if (a.taps == 4) hipLaunchKernelGGL((gated_delta_prep_kernel<T, K, 4>), grid, dim3(256), 0, st, a, items, RB, bt);
+  else hipLaunchKernelGGL((gated_delta_prep_kernel<T, K, 0>), grid, dim3(256), 0, st, a, items, RB, bt);
 }
 
 extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hipStream_t st) {
@@ -130,12 +194,13 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
   if (!a.P || !a.cw || (a.taps > 1 && !a.state) || !a.arate || !a.dt_bias || !a.qf || !a.kf || !a.vo || !a.gb) return -1;
   const int C = 2 * a.G * a.d + a.H * a.vd;
   if (a.b0 < C || a.a0 < C || a.ldp < a.b0 + a.H || a.ldp < a.a0 + a.H || (a.write_state && bt.B != bt.T)) return -1;
+  if ((int64_t)bt.T * (2 * a.G + a.H * a.vd) > 0x7fffffff) return -1;
   if (a.taps == 1) a.write_state = 0;
-  const int items = 2 * a.G + (a.H * a.vd + 255) / 256 + 1;
-  const int64_t blocks = ((int64_t)bt.T * items + 3) / 4;
-  if (blocks > 0x7fffffff) return -1;
-  RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((gated_delta_prep_kernel<T>), dim3((unsigned)blocks), dim3(256), 4 * a.d * sizeof(float), st,
-                                            a, items, bt))
+  RAGGED_DISPATCH(dtype,
+    if (a.d <= 64) launch_gated_prep<T, 1>(a, bt, st);
+    else if (a.d <= 128) launch_gated_prep<T, 2>(a, bt, st);
+    else if (a.d <= 256) launch_gated_prep<T, 4>(a, bt, st);
+    else launch_gated_prep<T, 16>(a, bt, st))
   return RAGGED_LAUNCH_OK();
 }
 

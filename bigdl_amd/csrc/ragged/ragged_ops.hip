@@ -836,12 +836,15 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const TI* __restrict__ s
   if (c >= C) return;
   const int taps = TAPS > 0 ? TAPS : ntaps, keep = taps - 1;
   const int t0 = blockIdx.y * CR_RB, t1 = t0 + CR_RB < bt.T ? t0 + CR_RB : bt.T;
-  // the input `back` positions before row t (position pos of a sequence whose first `past` positions are older than the step)
+  // the input `back` positions before row t (position pos of a sequence whose first `past` positions are older than the step);
+  // the address is chosen first, so that the loads of all taps are in flight together
   auto input = [&](int t, int back, int pos, int past, int slot) -> float {
     const int pp = pos - back;
-    if (pp >= past) return to_f(src[(int64_t)(t - back) * ld + col0 + c]);
-    if (pp >= 0) return to_f(state[((int64_t)slot * keep + (pp - past + keep)) * C + c]);
-    return 0.f;
+    const TI* p = src + (int64_t)t * ld + col0 + c;
+    if (pp >= past) p -= back * ld;
+    else if (pp >= 0) p = state + ((int64_t)slot * keep + (pp - past + keep)) * C + c;
+    const float v = to_f(*p);
+    return pp >= 0 ? v : 0.f;
   };
   float w[TAPS > 0 ? TAPS : 1], hist[TAPS > 1 ? TAPS - 1 : 1];
 #pragma unroll
@@ -908,43 +911,40 @@ extern "C" int ragged_conv_rows(const void* src, int64_t ld, int col0, const flo
 // xa = x as T for the product that reads the stream next.  With `cw` (every sequence brings exactly one row) xa is the
 // convolved stream x + sum_j cw[c, j] x_(t - taps + 1 + j) that the next layer's mixer reads: the older inputs come from
 // `hist` [slots, taps - 1, D], which is shifted in the same pass.  y null: xa = LN(x), the stream stays as it is.
-// One workgroup per row; NV as in post_norm_add_kernel.
-template <typename T, int NV>
+// One workgroup per row; NV as in post_norm_add_kernel: every operand of the row, the stream's history included, is then
+// requested before the first sum.  TAPS: the taps of `cw` as a constant (0: no convolution, or any number of taps).
+template <typename T, int NV, int TAPS>
 __global__ __launch_bounds__(256) void ln_add_kernel(float* __restrict__ x, const T* __restrict__ y, const float* __restrict__ w,
                                                      const float* __restrict__ bias, T* __restrict__ xa, int D, float eps,
                                                      const float* __restrict__ cw, int taps, float* __restrict__ hist, Batch bt) {
   __shared__ float red[8];
   const int64_t row = blockIdx.x, base = row * D;
-  int slot = 0, pos = 0;
-  if (cw) { slot = bt.seq_slot[bt.tok_seq[row]]; pos = bt.tok_pos[row]; }
   const int keep = taps - 1;
-  auto finish = [&](int c, float norm) {
-    const float v = y ? x[base + c] + norm : norm;
-    if (y) x[base + c] = v;
-    if (!xa) return;
-    float h = v;
-    if (cw) {
-      float u = 0.f;
-      for (int j = 0; j < keep; ++j) {                       // hist row j holds the input at position pos - keep + j
-        const int64_t o = ((int64_t)slot * keep + j) * D + c;
-        const float old = pos - keep + j >= 0 ? hist[o] : 0.f;
-        u += cw[(int64_t)c * taps + j] * old;
-        if (j > 0) hist[o - D] = old;
-      }
-      if (keep > 0) hist[((int64_t)slot * keep + keep - 1) * D + c] = v;
-      h = v + u + cw[(int64_t)c * taps + keep] * v;
-    }
-    xa[base + c] = from_f<T>(h);
-  };
+  int pos = 0;
+  float* hp = hist;                                          // this sequence's history: row j holds position pos - keep + j
+  if (cw && keep > 0) {
+    const int b = bt.tok_seq[row];
+    pos = bt.tok_pos[row];
+    hp += (int64_t)bt.seq_slot[b] * keep * D;
+  }
   if (NV > 0) {
-    float v[NV > 0 ? NV : 1];
+    constexpr int K = TAPS > 1 ? TAPS - 1 : 1;
+    float v[NV > 0 ? NV : 1], xv[NV > 0 ? NV : 1], wv[NV > 0 ? NV : 1], bv[NV > 0 ? NV : 1], old[NV > 0 ? NV : 1][K];
     float s = 0.f;
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int c = threadIdx.x + 256 * u;
-      v[u] = c < D ? (y ? to_f(y[base + c]) : x[base + c]) : 0.f;
-      s += v[u];
+      const int c = threadIdx.x + 256 * u, cc = c < D ? c : D - 1;
+      xv[u] = x[base + cc];
+      v[u] = y ? to_f(y[base + cc]) : xv[u];
+      wv[u] = w[cc];
+      bv[u] = bias[cc];
+      if (TAPS > 1) {
+#pragma unroll
+        for (int j = 0; j < K; ++j) old[u][j] = hp[(int64_t)j * D + cc];
+      }
     }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) s += threadIdx.x + 256 * u < D ? v[u] : 0.f;
     const float mean = block_sum_256(s, red) / (float)D;
     s = 0.f;
 #pragma unroll
@@ -956,7 +956,33 @@ __global__ __launch_bounds__(256) void ln_add_kernel(float* __restrict__ x, cons
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int c = threadIdx.x + 256 * u;
-      if (c < D) finish(c, v[u] * r * w[c] + bias[c]);
+      if (c >= D) continue;
+      float h = v[u] * r * wv[u] + bv[u];
+      if (y) { h += xv[u]; x[base + c] = h; }
+      if (!xa) continue;
+      if (TAPS > 1) {
+        const float now = h;
+        float f = cw[(int64_t)c * TAPS + K] * now;
+#pragma unroll
+        for (int j = 0; j < K; ++j) {
+          const float o = pos - K + j >= 0 ? old[u][j] : 0.f;
+          f += cw[(int64_t)c * TAPS + j] * o;
+          if (j > 0) hp[(int64_t)(j - 1) * D + c] = o;
+        }
+        hp[(int64_t)(K - 1) * D + c] = now;
+        h = now + f;
+      } else if (cw) {
+        const float now = h;
+        float f = cw[(int64_t)c * taps + keep] * now;
+        for (int j = 0; j < keep; ++j) {
+          const float o = pos - keep + j >= 0 ? hp[(int64_t)j * D + c] : 0.f;
+          f += cw[(int64_t)c * taps + j] * o;
+          if (j > 0) hp[(int64_t)(j - 1) * D + c] = o;
+        }
+        if (keep > 0) hp[(int64_t)(keep - 1) * D + c] = now;
+        h = now + f;
+      }
+      xa[base + c] = from_f<T>(h);
     }
     return;
   }
@@ -966,7 +992,35 @@ __global__ __launch_bounds__(256) void ln_add_kernel(float* __restrict__ x, cons
   s = 0.f;
   for (int c = threadIdx.x; c < D; c += 256) { const float v = (y ? to_f(y[base + c]) : x[base + c]) - mean; s += v * v; }
   const float r = 1.0f / sqrtf(block_sum_256(s, red + 4) / (float)D + eps);
-  for (int c = threadIdx.x; c < D; c += 256) finish(c, ((y ? to_f(y[base + c]) : x[base + c]) - mean) * r * w[c] + bias[c]);
+  for (int c = threadIdx.x; c < D; c += 256) {
+    float h = ((y ? to_f(y[base + c]) : x[base + c]) - mean) * r * w[c] + bias[c];
+    if (y) { h += x[base + c]; x[base + c] = h; }
+    if (!xa) continue;
+    if (cw) {
+      const float now = h;
+      float f = cw[(int64_t)c * taps + keep] * now;
+      for (int j = 0; j < keep; ++j) {
+        const float o = pos - keep + j >= 0 ? hp[(int64_t)j * D + c] : 0.f;
+        f += cw[(int64_t)c * taps + j] * o;
+        if (j > 0) hp[(int64_t)(j - 1) * D + c] = o;
+      }
+      if (keep > 0) hp[(int64_t)(keep - 1) * D + c] = now;
+      h = now + f;
+    }
+    xa[base + c] = from_f<T>(h);
+  }
+}
+
+template <typename T, int TAPS>
+static void launch_ln_add(float* x, const void* y, const float* w, const float* bias, void* xa, int64_t rows, int D, float eps,
+                          const float* cw, int taps, float* hist, Batch bt, hipStream_t st) {
+#define LN_CASE(NV) hipLaunchKernelGGL((ln_add_kernel<T, NV, TAPS>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias, (T*)xa, D, \
+                                       eps, cw, taps, hist, bt)
+  if (D <= 1024) LN_CASE(4);
+  else if (D <= 2048) LN_CASE(8);
+  else if (D <= 4096) LN_CASE(16);
+  else LN_CASE(0);
+#undef LN_CASE
 }
 
 extern "C" int ragged_ln_add(float* x, const void* y, const float* w, const float* bias, void* xa, int64_t rows, int D, float eps,
@@ -974,12 +1028,8 @@ extern "C" int ragged_ln_add(float* x, const void* y, const float* w, const floa
   if (rows <= 0 || D <= 0 || rows > 0x7fffffff || !x || !w || !bias || (!y && !xa)) return -1;
   if (cw && (!xa || !y || taps < 1 || taps > 16 || (taps > 1 && !hist) || bt.T != rows || bt.B != rows)) return -1;
   RAGGED_DISPATCH(dtype,
-    if (D <= 1024) hipLaunchKernelGGL((ln_add_kernel<T, 4>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias, (T*)xa, D,
-                                      eps, cw, taps, hist, bt);
-    else if (D <= 4096) hipLaunchKernelGGL((ln_add_kernel<T, 16>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias,
-                                           (T*)xa, D, eps, cw, taps, hist, bt);
-    else hipLaunchKernelGGL((ln_add_kernel<T, 0>), dim3((unsigned)rows), dim3(256), 0, st, x, (const T*)y, w, bias, (T*)xa, D, eps, cw,
-                            taps, hist, bt))
+    if (cw && taps == 4) launch_ln_add<T, 4>(x, y, w, bias, xa, rows, D, eps, cw, taps, hist, bt, st);
+    else launch_ln_add<T, 0>(x, y, w, bias, xa, rows, D, eps, cw, taps, hist, bt, st))
   return RAGGED_LAUNCH_OK();
 }
 
