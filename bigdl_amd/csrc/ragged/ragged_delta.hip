@@ -84,8 +84,9 @@ template <typename T, int K, int TAPS>
 __global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a, int items, int RB, Batch bt) {
   constexpr int M = TAPS > 1 ? TAPS - 1 : 1, W = TAPS > 0 ? TAPS : 1;
   const int lane = threadIdx.x & 63;
-  const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int t0 = (int)(id / items) * RB, it = (int)(id % items);
+  // (the same for a whole wavefront: kept in scalar registers)
+  const unsigned id = __builtin_amdgcn_readfirstlane(blockIdx.x * 4 + (threadIdx.x >> 6));
+  const int t0 = (int)(id / (unsigned)items) * RB, it = (int)(id % (unsigned)items);
   if (t0 >= bt.T) return;
   const int t1 = t0 + RB < bt.T ? t0 + RB : bt.T;
   const T* P = (const T*)a.P;
@@ -126,12 +127,24 @@ __global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a,
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) w[k][j] = a.cw[(int64_t)chs[k] * TAPS + j];
   }
-  for (int t = t0; t < t1; ++t) {
-    const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
+  T next[K];                                                 // the row after the current one, requested early
+#pragma unroll
+  for (int k = 0; k < K; ++k) next[k] = P[(int64_t)t0 * a.ldp + chs[k]];
+  // what belongs to the rows' sequence is looked up once per sequence (a batch's sequences lie one behind the other)
+  int b = bt.tok_seq[t0], pos = bt.tok_pos[t0], past = bt.seq_past[b], slot = bt.seq_slot[b], end = bt.seq_start[b + 1];
+  const float qscale = isq ? 1.0f / sqrtf((float)a.d) : 1.0f;
+  for (int t = t0; t < t1; ++t, ++pos) {
+    if (t == end) { ++b; pos = past = bt.seq_past[b]; slot = bt.seq_slot[b]; end = bt.seq_start[b + 1]; }
     float u[K], ss = 0.f;
+    T row[K];
 #pragma unroll
     for (int k = 0; k < K; ++k) {
-      const T cur = P[(int64_t)t * a.ldp + chs[k]];
+      row[k] = next[k];
+      next[k] = P[(int64_t)(t + 1 < t1 ? t + 1 : t) * a.ldp + chs[k]];
+    }
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const T cur = row[k];
       u[k] = 0.f;
       const bool ok = lane + 64 * k < width;
       if (TAPS > 0) {
@@ -160,12 +173,11 @@ __global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a,
           if (a.write_state && ok && j > 0) S[((int64_t)slot * keep + j - 1) * C + chs[k]] = raw;   // (row j - 1 has been read)
         }
       }
-      u[k] = ok ? u[k] / (1.0f + expf(-u[k])) : 0.f;
+      u[k] = ok ? u[k] * sigmoidf_(u[k]) : 0.f;
       ss += u[k] * u[k];
     }
     if (unit) {
-      float f = 1.0f / sqrtf(wave_sum(ss) + a.tiny);
-      if (isq) f *= 1.0f / sqrtf((float)a.d);
+      const float f = qscale / sqrtf(wave_sum(ss) + a.tiny);
       float* o = (isq ? a.qf : a.kf) + ((int64_t)t * a.G + (isq ? it : it - a.G)) * a.d;
 #pragma unroll
       for (int k = 0; k < K; ++k)

@@ -822,20 +822,22 @@ extern "C" int ragged_gate_cols(const float* o, const void* P, int64_t ldp, int 
 
 // ---------------------------------------------------------------------------------------------------------------
 // Short causal convolution over time per channel for whole rows: u_t = sum_j w[c, j] s_(t - taps + 1 + j) (+ bias), then
-// out = silu(u), s + u or u.  A thread walks RB neighbouring rows of one channel with the last taps - 1 inputs in registers
+// out = silu(u), s + u or u.  A thread walks RB neighbouring rows of one channel (requested CR_U at a time) with the last
+// taps - 1 inputs in registers
 // (TAPS = the number of taps, or 0 for any number: every tap is then read where it is needed).  A sequence's inputs before
 // this step come from `state` [slots, taps - 1, C] (the type of the source); `write_state` (every sequence brings exactly one
 // row) also shifts the state, otherwise ragged_conv_state does so behind this kernel.
-constexpr int CR_RB = 16;
+constexpr int CR_U = 8;
 
 template <typename TI, typename TO, int TAPS>
 __global__ __launch_bounds__(256) void conv_rows_kernel(const TI* __restrict__ src, int64_t ld, int col0, const float* __restrict__ cw,
                                                         const float* __restrict__ bias, TI* __restrict__ state, int ntaps, int C,
-                                                        TO* __restrict__ out, int add, int silu, int write_state, Batch bt) {
+                                                        TO* __restrict__ out, int add, int silu, int write_state, int RB,
+                                                        Batch bt) {
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= C) return;
   const int taps = TAPS > 0 ? TAPS : ntaps, keep = taps - 1;
-  const int t0 = blockIdx.y * CR_RB, t1 = t0 + CR_RB < bt.T ? t0 + CR_RB : bt.T;
+  const int t0 = blockIdx.y * RB, t1 = t0 + RB < bt.T ? t0 + RB : bt.T;
   // the input `back` positions before row t (position pos of a sequence whose first `past` positions are older than the step);
   // the address is chosen first, so that the loads of all taps are in flight together
   auto input = [&](int t, int back, int pos, int past, int slot) -> float {
@@ -850,42 +852,54 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const TI* __restrict__ s
 #pragma unroll
   for (int j = 0; j < TAPS; ++j) w[j] = cw[(int64_t)c * TAPS + j];
   const float b0 = bias ? bias[c] : 0.f;
-  for (int t = t0; t < t1; ++t) {
-    const int b = bt.tok_seq[t], pos = bt.tok_pos[t], past = bt.seq_past[b], slot = bt.seq_slot[b];
-    const float cur = to_f(src[(int64_t)t * ld + col0 + c]);
-    float u = b0;
-    if (TAPS > 0) {
-      if (t == t0 || pos == past) {                          // (the same branch for the whole workgroup)
+  // what belongs to the rows' sequence is looked up once per sequence (a batch's sequences lie one behind the other)
+  int b = bt.tok_seq[t0], pos = bt.tok_pos[t0], past = bt.seq_past[b], slot = bt.seq_slot[b], end = bt.seq_start[b + 1];
+  for (int g0 = t0; g0 < t1; g0 += CR_U) {
+    TI now[CR_U];
 #pragma unroll
-        for (int j = 0; j + 1 < TAPS; ++j) hist[j] = input(t, TAPS - 1 - j, pos, past, slot);
+    for (int i = 0; i < CR_U; ++i) now[i] = src[(int64_t)(g0 + i < t1 ? g0 + i : t1 - 1) * ld + col0 + c];
+#pragma unroll
+    for (int i = 0; i < CR_U; ++i) {
+      const int t = g0 + i;
+      if (t >= t1) break;
+      if (t == end) { ++b; pos = past = bt.seq_past[b]; slot = bt.seq_slot[b]; end = bt.seq_start[b + 1]; }
+      const float cur = to_f(now[i]);
+      float u = b0;
+      if (TAPS > 0) {
+        if (t == t0 || pos == past) {                        // (the same branch for the whole workgroup)
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS; ++j) hist[j] = input(t, TAPS - 1 - j, pos, past, slot);
+        }
+#pragma unroll
+        for (int j = 0; j + 1 < TAPS; ++j) u += w[j] * hist[j];
+        u += w[TAPS > 0 ? TAPS - 1 : 0] * cur;
+#pragma unroll
+        for (int j = 0; j + 2 < TAPS; ++j) hist[j] = hist[j + 1];
+        if (TAPS > 1) hist[TAPS > 1 ? TAPS - 2 : 0] = cur;
+        if (write_state) {
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(hist[j]);
+        }
+      } else {
+        for (int j = 0; j < taps; ++j) u += cw[(int64_t)c * taps + j] * input(t, taps - 1 - j, pos, past, slot);
+        if (write_state) {                                   // (row j + 1 is read before row j + 1 is written)
+          for (int j = 0; j < keep; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(input(t, keep - 1 - j, pos, past, slot));
+        }
       }
-#pragma unroll
-      for (int j = 0; j + 1 < TAPS; ++j) u += w[j] * hist[j];
-      u += w[TAPS > 0 ? TAPS - 1 : 0] * cur;
-#pragma unroll
-      for (int j = 0; j + 2 < TAPS; ++j) hist[j] = hist[j + 1];
-      if (TAPS > 1) hist[TAPS > 1 ? TAPS - 2 : 0] = cur;
-      if (write_state) {
-#pragma unroll
-        for (int j = 0; j + 1 < TAPS; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(hist[j]);
-      }
-    } else {
-      for (int j = 0; j < taps; ++j) u += cw[(int64_t)c * taps + j] * input(t, taps - 1 - j, pos, past, slot);
-      if (write_state) {                                     // (row j + 1 is read before row j + 1 is written)
-        for (int j = 0; j < keep; ++j) state[((int64_t)slot * keep + j) * C + c] = from_f<TI>(input(t, keep - 1 - j, pos, past, slot));
-      }
+      if (silu) u *= sigmoidf_(u);
+      out[(int64_t)t * C + c] = from_f<TO>(add ? cur + u : u);
+      ++pos;
     }
-    if (silu) u = u / (1.0f + expf(-u));
-    out[(int64_t)t * C + c] = from_f<TO>(add ? cur + u : u);
   }
 }
 
 template <typename TI, typename TO>
 static void launch_conv_rows(const void* src, int64_t ld, int col0, const float* cw, const float* bias, void* state, int taps, int C,
                              void* out, int add, int silu, int write_state, Batch bt, hipStream_t st) {
-  const dim3 grid((C + 255) / 256, (bt.T + CR_RB - 1) / CR_RB);
+  const int RB = bt.T == bt.B || bt.T < 128 ? 1 : 2 * CR_U;
+  const dim3 grid((C + 255) / 256, (bt.T + RB - 1) / RB);
 #define CR_CASE(N) hipLaunchKernelGGL((conv_rows_kernel<TI, TO, N>), grid, dim3(256), 0, st, (const TI*)src, ld, col0, cw, bias, \
-                                      (TI*)state, taps, C, (TO*)out, add, silu, write_state, bt)
+                                      (TI*)state, taps, C, (TO*)out, add, silu, write_state, RB, bt)
   if (taps == 1) CR_CASE(1);
   else if (taps == 2) CR_CASE(2);
   else if (taps == 3) CR_CASE(3);
@@ -897,7 +911,7 @@ static void launch_conv_rows(const void* src, int64_t ld, int col0, const float*
 // the source's type is `src_dtype` (the projections' activation type, or float for the stream itself), the output's `dtype`
 extern "C" int ragged_conv_rows(const void* src, int64_t ld, int col0, const float* cw, const float* bias, void* state, int taps, int C,
                                 void* out, int add, int silu, int write_state, Batch bt, int src_dtype, int dtype, hipStream_t st) {
-  if (bt.T <= 0 || bt.T > 65535 * CR_RB || C <= 0 || col0 < 0 || ld < col0 + C || taps < 1 || taps > 16 || (taps > 1 && !state)) return -1;
+  if (bt.T <= 0 || bt.T > (bt.T == bt.B ? 65535 : 65535 * 2 * CR_U) || C <= 0 || col0 < 0 || ld < col0 + C || taps < 1 || taps > 16 || (taps > 1 && !state)) return -1;
   if (src_dtype != dtype && src_dtype != 2) return -2;
   if (taps == 1) write_state = 0;
   RAGGED_DISPATCH(dtype,
