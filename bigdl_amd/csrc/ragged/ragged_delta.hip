@@ -420,110 +420,132 @@ extern "C" int ragged_gated_delta_scan(const float* qf, const float* kf, const f
 // leaves the last S in the sequence's slot.  A workgroup holds 16 columns of S in LDS; thread (i0, j) makes rows
 // i0, i0 + 16, ... of column j.  Grid: (column blocks, heads, sequences); cfirst[b] .. cfirst[b + 1] - 1 are b's chunks.
 constexpr int DC_COLS = 16;
-constexpr int DC_LDS_D = 120;                              // up to this many rows a chunk's A is staged in LDS
-constexpr int DC_APRE = (DC_LDS_D * DC_LDS_D + 255) / 256;
-constexpr int DC_LPRE = (DC_LDS_D + 15) / 16;              // rows of a column that a thread makes
+constexpr int DC_LDS_D = 128;                              // up to this many rows a chunk's A is staged in LDS
 
-// LDSA: A_c is brought into LDS by the whole workgroup (coalesced) and A_c and the thread's elements of L_c are requested
-// one chunk ahead into registers, so a chunk's step waits for no memory; otherwise every thread reads its rows of A_c and
-// its elements of L_c from memory as it goes.
-template <bool LDSA>
+// NU > 0: a thread makes rows i0 + 16 u, u < NU (16 NU >= d).  A_c is brought into LDS by the whole workgroup (coalesced) and
+// A_c and the thread's elements of L_c are requested one chunk ahead into registers, so a chunk's step waits for no memory;
+// S lies transposed, [column][row], so that both operands are read four channels at a time.
+// NU = 0: any d; every thread reads its rows of A_c and its elements of L_c from memory as it goes.
+template <int NU>
 __global__ __launch_bounds__(256) void delta_chain_kernel(float* __restrict__ state, const float* __restrict__ local,
                                                           const float* __restrict__ trans, float* __restrict__ begin,
                                                           const int* __restrict__ cfirst, const int* __restrict__ seq_past,
                                                           const int* __restrict__ seq_slot, int H, int d, int vd) {
-  extern __shared__ __attribute__((aligned(16))) float smem[];   // two buffers [d][DC_COLS], then A [d][d + 1]
+  extern __shared__ __attribute__((aligned(16))) float smem[];   // two buffers [DC_COLS][ld] of S, then A [d][ld]
+  constexpr int U = NU > 0 ? NU : 1, NA = NU * NU > 0 ? NU * NU : 1;      // d d <= 256 NU NU
   const int b = blockIdx.z, h = blockIdx.y;
   const int j = threadIdx.x % DC_COLS, i0 = threadIdx.x / DC_COLS, col = blockIdx.x * DC_COLS + j;
   const bool colok = col < vd;
   const int cc = colok ? col : vd - 1;
+  const int ld = ((d + 3) & ~3) + 4;                         // (a row's padding stays zero; the odd multiple of 4 spreads the banks)
   float* cur = smem;
-  float* nxt = smem + d * DC_COLS;
-  float* As = smem + 2 * d * DC_COLS;
-  const int lda = d + 1;
+  float* nxt = smem + DC_COLS * ld;
+  float* As = smem + 2 * DC_COLS * ld;
   float* sp = state + ((int64_t)seq_slot[b] * H + h) * d * vd;
   const bool old = seq_past[b] > 0;
-  for (int i = i0; i < d; i += 256 / DC_COLS) cur[i * DC_COLS + j] = old ? sp[(int64_t)i * vd + cc] : 0.f;
+  for (int e = threadIdx.x; e < (2 * DC_COLS + (NU > 0 ? d : 0)) * ld; e += 256) smem[e] = 0.f;
+  __syncthreads();
+  for (int i = i0; i < d; i += 16) cur[j * ld + i] = old ? sp[(int64_t)i * vd + cc] : 0.f;
   const int c0 = cfirst[b], c1 = cfirst[b + 1];
-  float apre[LDSA ? DC_APRE : 1], lpre[LDSA ? DC_LPRE : 1], lcur[LDSA ? DC_LPRE : 1];
+  float apre[NA], lpre[U], acc[U];
   auto fetch = [&](int c) {
     const float* A = trans + ((int64_t)c * H + h) * d * d;
     const float* L = local + ((int64_t)c * H + h) * d * vd;
 #pragma unroll
-    for (int u = 0; u < DC_APRE; ++u) {
-      if (256 * u >= d * d) break;
+    for (int u = 0; u < NA; ++u) {
       const int e = threadIdx.x + 256 * u;
-      apre[u] = e < d * d ? A[e] : 0.f;
+      apre[u] = A[e < d * d ? e : d * d - 1];
     }
 #pragma unroll
-    for (int u = 0; u < DC_LPRE; ++u) {
+    for (int u = 0; u < U; ++u) {
       const int i = i0 + 16 * u;
-      lpre[u] = i < d ? L[(int64_t)i * vd + cc] : 0.f;
+      lpre[u] = L[(int64_t)(i < d ? i : d - 1) * vd + cc];
     }
   };
   const int step_r = 256 / d, step_c = 256 % d;
-  if (LDSA && c0 < c1) fetch(c0);
+  if (NU > 0 && c0 < c1) fetch(c0);
   __syncthreads();
   for (int c = c0; c < c1; ++c) {
-    const float* A = trans + ((int64_t)c * H + h) * d * d;
-    const float* L = local + ((int64_t)c * H + h) * d * vd;
     float* B = begin + ((int64_t)c * H + h) * d * vd;
-    if (LDSA) {
-      int ar_ = threadIdx.x / d, ac_ = threadIdx.x % d;      // element e = threadIdx.x + 256 u of A sits at (e / d, e % d)
+    if (NU > 0) {
+      int ar = threadIdx.x / d, ac = threadIdx.x % d;        // element e = threadIdx.x + 256 u of A sits at (e / d, e % d)
 #pragma unroll
-      for (int u = 0; u < DC_APRE; ++u) {
-        if (256 * u >= d * d) break;
-        if (ar_ < d) As[ar_ * lda + ac_] = apre[u];
-        ar_ += step_r;
-        ac_ += step_c;
-        if (ac_ >= d) { ac_ -= d; ++ar_; }
+      for (int u = 0; u < NA; ++u) {
+        if (ar < d) As[ar * ld + ac] = apre[u];
+        ar += step_r;
+        ac += step_c;
+        if (ac >= d) { ac -= d; ++ar; }
       }
 #pragma unroll
-      for (int u = 0; u < DC_LPRE; ++u) lcur[u] = lpre[u];
+      for (int u = 0; u < U; ++u) acc[u] = lpre[u];
       __syncthreads();
       if (c + 1 < c1) fetch(c + 1);
-    }
-#pragma unroll 1
-    for (int i = i0, u = 0; i < d; i += 256 / DC_COLS, ++u) {
-      if (colok) B[(int64_t)i * vd + col] = cur[i * DC_COLS + j];
-      float first = 0.f;
-      if (LDSA) {
+      for (int l = 0; l < d; l += 4) {
+        const float4 s = *reinterpret_cast<const float4*>(cur + j * ld + l);
 #pragma unroll
-        for (int uu = 0; uu < DC_LPRE; ++uu) first = uu == u ? lcur[uu] : first;     // (a register, not an indexed array)
-      } else {
-        first = L[(int64_t)i * vd + cc];
+        for (int u = 0; u < U; ++u) {
+          const int i = i0 + 16 * u;
+          const float4 a = *reinterpret_cast<const float4*>(As + (i < d ? i : d - 1) * ld + l);
+          acc[u] += (a.x * s.x + a.y * s.y) + (a.z * s.z + a.w * s.w);
+        }
       }
-      float acc[4] = {first, 0.f, 0.f, 0.f};
-      const float* ar = LDSA ? As + i * lda : A + (int64_t)i * d;
-      int l = 0;
-      for (; l + 4 <= d; l += 4) {
-        acc[0] += ar[l] * cur[l * DC_COLS + j];
-        acc[1] += ar[l + 1] * cur[(l + 1) * DC_COLS + j];
-        acc[2] += ar[l + 2] * cur[(l + 2) * DC_COLS + j];
-        acc[3] += ar[l + 3] * cur[(l + 3) * DC_COLS + j];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int i = i0 + 16 * u;
+        if (i < d) {
+          if (colok) B[(int64_t)i * vd + col] = cur[j * ld + i];
+          nxt[j * ld + i] = acc[u];
+        }
       }
-      for (; l < d; ++l) acc[0] += ar[l] * cur[l * DC_COLS + j];
-      nxt[i * DC_COLS + j] = (acc[0] + acc[1]) + (acc[2] + acc[3]);
+    } else {
+      const float* A = trans + ((int64_t)c * H + h) * d * d;
+      const float* L = local + ((int64_t)c * H + h) * d * vd;
+      for (int i = i0; i < d; i += 16) {
+        if (colok) B[(int64_t)i * vd + col] = cur[j * ld + i];
+        float s4[4] = {L[(int64_t)i * vd + cc], 0.f, 0.f, 0.f};
+        const float* ar = A + (int64_t)i * d;
+        int l = 0;
+        for (; l + 4 <= d; l += 4) {
+#pragma unroll
+          for (int k = 0; k < 4; ++k) s4[k] += ar[l + k] * cur[j * ld + l + k];
+        }
+        for (; l < d; ++l) s4[0] += ar[l] * cur[j * ld + l];
+        nxt[j * ld + i] = (s4[0] + s4[1]) + (s4[2] + s4[3]);
+      }
     }
     __syncthreads();
     float* t = cur; cur = nxt; nxt = t;
   }
-  for (int i = i0; i < d; i += 256 / DC_COLS)
-    if (colok) sp[(int64_t)i * vd + col] = cur[i * DC_COLS + j];
+  for (int i = i0; i < d; i += 16)
+    if (colok) sp[(int64_t)i * vd + col] = cur[j * ld + i];
 }
 
 extern "C" int ragged_delta_chain_ok(int d) { return d > 0 && d <= 384; }
 
+template <int NU>
+static int launch_delta_chain(float* state, const float* local, const float* trans, float* begin, const int* cfirst, const int* seq_past,
+                              const int* seq_slot, int B, int H, int d, int vd, hipStream_t st) {
+  const size_t ld = ((d + 3) & ~3) + 4, sm = (2 * DC_COLS + (NU > 0 ? d : 0)) * ld * sizeof(float);
+  if (sm > 64 * 1024) {                                      // (asked for once per process and kernel)
+    static const hipError_t asked = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_chain_kernel<NU>),
+                                                        hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024);
+    if (asked != hipSuccess) return -3;
+  }
+  hipLaunchKernelGGL(delta_chain_kernel<NU>, dim3((vd + DC_COLS - 1) / DC_COLS, H, B), dim3(256), sm, st, state, local, trans, begin, cfirst,
+                     seq_past, seq_slot, H, d, vd);
+  return RAGGED_LAUNCH_OK();
+}
+
 extern "C" int ragged_delta_chain(float* state, const float* local, const float* trans, float* begin, const int* cfirst,
                                   const int* seq_past, const int* seq_slot, int B, int H, int d, int vd, hipStream_t st) {
   if (B <= 0 || H <= 0 || vd <= 0 || !ragged_delta_chain_ok(d)) return -1;
-  const dim3 grid((vd + DC_COLS - 1) / DC_COLS, H, B);
-  if (d <= DC_LDS_D) {
-    const size_t sm = (2 * (size_t)d * DC_COLS + (size_t)d * (d + 1)) * sizeof(float);
-    hipLaunchKernelGGL(delta_chain_kernel<true>, grid, dim3(256), sm, st, state, local, trans, begin, cfirst, seq_past, seq_slot, H, d, vd);
-  } else {
-    const size_t sm = 2 * (size_t)d * DC_COLS * sizeof(float);
-    hipLaunchKernelGGL(delta_chain_kernel<false>, grid, dim3(256), sm, st, state, local, trans, begin, cfirst, seq_past, seq_slot, H, d, vd);
-  }
-  return RAGGED_LAUNCH_OK();
+#define DC_CASE(NU) return launch_delta_chain<NU>(state, local, trans, begin, cfirst, seq_past, seq_slot, B, H, d, vd, st)
+  if (d <= 16) DC_CASE(1);
+  if (d <= 32) DC_CASE(2);
+  if (d <= 48) DC_CASE(3);
+  if (d <= 64) DC_CASE(4);
+  if (d <= 96) DC_CASE(6);
+  if (d <= DC_LDS_D) DC_CASE(8);
+  DC_CASE(0);
+#undef DC_CASE
 }

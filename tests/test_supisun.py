@@ -461,7 +461,7 @@ def test_selective_scan_across_portions_and_in_a_used_slot(device, C, N):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("H,G,d,e,taps", [(4, 2, 16, 24, 4), (1, 1, 48, 8, 1), (3, 1, 40, 64, 3), (2, 2, 130, 33, 4), (6, 3, 5, 7, 2),
-                                          (2, 1, 300, 20, 4)])
+                                          (2, 1, 300, 20, 4), (2, 1, 128, 128, 4), (1, 1, 117, 16, 4), (2, 2, 64, 64, 4)])
 def test_gated_delta_rule_across_portions_and_in_a_used_slot(device, H, G, d, e, taps):
     """preparation (convolutions, unit vectors, gates) and scan against the token-by-token statement: portions of 1, 2 and many
     tokens, a second sequence in the first one's slot, long portions in chunks, decays near one"""
