@@ -975,7 +975,7 @@ class HipOps:
         return q, first
 
     selective_chunked_from = 128  # portions of at least this many tokens run the selective scan in chunks
-    selective_waves = 2048        # wavefronts of a pass that the chunk length aims at (eight per CU)
+    selective_waves = 4096        # wavefronts of a pass that the chunk length aims at (sixteen per CU)
 
     @staticmethod
     def _states_per_lane(N, long):
