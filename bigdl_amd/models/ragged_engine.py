@@ -70,7 +70,7 @@ class WindowAttention:
     dist_slopes: Optional[tuple] = None  # per head: slope * (i - j) is taken off the scaled score of query i and key j
     v_from_k: bool = False         # no value projection: the values are the key projections as they are before norm and rotation
     qk_norm_rows: bool = False     # RMS norm over the whole query (key) projection at once, a weight per channel, before rotation
-    v_norm: bool = False           # each head's value divided by its root mean square (no weight)
+    v_norm: bool = False           # values RMS-normed per head, without a weight
     v_mix: bool = False            # values of the stack's first such layer are mixed in: v <- (1 - lam) v + lam v_first of the same
                                    # token (``LayerTensors.v_lam``; needs equal value sizes); what is cached is the mixture
 

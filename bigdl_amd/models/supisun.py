@@ -7,7 +7,7 @@ channel of the stream; a last LayerNorm and an output projection of its own.
 Mixers (``type`` of a layer):
 
 * ``attention``: grouped key/value heads; queries and keys RMS-normed over the whole projection with a weight per channel, the
-  first ``rot.dims`` channels of every head turned in pairs (i, i + dims / 2); every value head divided by its root mean square;
+  first ``rot.dims`` channels of every head turned in pairs (i, i + dims / 2); values RMS-normed per head without a weight;
   with ``v_mix`` the values of the first such layer are mixed in, v <- (1 - lambda) v + lambda v_first; softmax inside blocks of
   ``mask.size`` positions counted from the sequence's start;
 * ``mamba1``: selective scan (``SelectiveScan``);
