@@ -33,6 +33,8 @@ struct AttnArgs {
   const float* sinks;    // [H] or null: with `sink`, head h's own sink score instead of sink_score
   const float* slopes;   // [H] or null: slopes[h] * (i - j) is taken off the scaled score of query i and key j (in front of
                          // the cap, if there is one): a bias that grows with the distance
+  const float* dist_bias;  // [H][n_bias] or null: dist_bias[h][min(i - j, n_bias - 1)] joins the scaled score in front of the cap
+  int n_bias;
 };
 
 namespace ragged {

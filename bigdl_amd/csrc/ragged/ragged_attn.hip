@@ -126,6 +126,12 @@ __global__ __launch_bounds__(512) void paged_attn_kernel(AttnArgs a, Batch bt, i
       }
     };
     load_values(va, 0);                               // in flight during the scores
+    float bias[REP];                                  // by distance, requested with them
+    if (a.dist_bias) {
+      const int dist = i - kp < 0 ? 0 : i - kp < a.n_bias ? i - kp : a.n_bias - 1;
+#pragma unroll
+      for (int r = 0; r < REP; ++r) bias[r] = a.dist_bias[(int64_t)(h0 + r) * a.n_bias + dist];
+    }
     float s[REP][MAPS];
     if (VEC && coal) {
       const int kpi = 64 / cpr;                       // keys per load instruction
@@ -200,6 +206,12 @@ __global__ __launch_bounds__(512) void paged_attn_kernel(AttnArgs a, Batch bt, i
       for (int r = 0; r < REP; ++r)
 #pragma unroll
         for (int mp = 0; mp < MAPS; ++mp) s[r][mp] -= a.slopes[h0 + r] * dist;
+    }
+    if (a.dist_bias) {
+#pragma unroll
+      for (int r = 0; r < REP; ++r)
+#pragma unroll
+        for (int mp = 0; mp < MAPS; ++mp) s[r][mp] += bias[r];
     }
     if (a.softcap > 0.f) {
       const float inv_cap = 1.0f / a.softcap;
@@ -379,7 +391,8 @@ static void launch_rows(AttnArgs a, Batch bt, int nrows, hipStream_t st, int* rc
 
 extern "C" int ragged_paged_attn(AttnArgs a, Batch bt, int maps, int dtype, hipStream_t st) {
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.d <= 0 || a.vd <= 0 || a.vd > 128 * MAX_VRP) return -1;
-  if ((maps != 1 && maps != 2) || a.ldv < a.vd || a.chunk < 0 || (a.gate_wide && !a.gate) || (a.sinks && !a.sink)) return -1;
+  if ((maps != 1 && maps != 2) || a.ldv < a.vd || a.chunk < 0 || (a.gate_wide && !a.gate) || (a.sinks && !a.sink) ||
+      (a.dist_bias && a.n_bias <= 0)) return -1;
   const int nrows = a.rows ? a.n_rows : bt.T;
   if (nrows <= 0 || (int64_t)nrows * a.H > 0x7fffffff) return -1;
   int rc = 0;

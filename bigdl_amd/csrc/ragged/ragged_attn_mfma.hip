@@ -13,6 +13,8 @@
 //    16 bits of p and the upper 16 bits of the exact remainder (2^-16 relative), so the second product loses nothing
 //    beyond the values' own 16 bits.
 //  * both maps of a differential head share the K page walk and the value tile.
+//  * a learned bias by distance: the head's table lies in LDS (a table too long for it is read where it is); pages whose keys are all
+//    at the table's last distance or farther take that one number.
 #include "ragged_attn.h"
 
 using namespace ragged;
@@ -37,8 +39,12 @@ __device__ __forceinline__ uint16_t bf_bits(float f) { return from_f<bf16>(f).b;
 // overflow trouble (e^(2x) = inf gives 1, 0 gives -1)
 __device__ __forceinline__ float fast_tanh(float x) { return 1.0f - 2.0f * __builtin_amdgcn_rcpf(__expf(2.0f * x) + 1.0f); }
 
-template <int MAPS, int DK>
+constexpr int MF_BIAS = 4096;  // entries of a head's distance-bias table that LDS takes
+
+// BIAS: no distance-bias table (0), one that lies in LDS (1) or one that is read from memory (2)
+template <int MAPS, int DK, int BIAS>
 __global__ __launch_bounds__(256) void paged_attn_mfma_kernel(AttnArgs a, Batch bt) {
+  extern __shared__ float bias_lds[];                        // BIAS 1: n_bias floats
   __shared__ __attribute__((aligned(16))) uint16_t vt[MF_NEB * 16 * MF_LDV];      // V^T [vd][PAGE (+ pad)]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int lq = lane & 15, g4 = lane >> 4;
@@ -88,6 +94,11 @@ __global__ __launch_bounds__(256) void paged_attn_mfma_kernel(AttnArgs a, Batch 
   const float inv_cap = capped ? 1.0f / a.softcap : 0.f;
   const bool biased = a.slopes != nullptr;                   // scores fall with the distance between query and key
   const float slope = biased ? a.slopes[h] : 0.f;
+  const float* btab = BIAS ? a.dist_bias + (int64_t)h * a.n_bias : nullptr;
+  if (BIAS == 1) {                                           // (the page loop's first barrier stands in front of the first use)
+    for (int e = threadIdx.x; e < a.n_bias; e += 256) bias_lds[e] = btab[e];
+  }
+  const float bias_far = BIAS ? btab[a.n_bias - 1] : 0.f;
 
   const bf16* K = (const bf16*)a.kpages;
   const bf16* V = (const bf16*)a.vpages;
@@ -181,6 +192,20 @@ __global__ __launch_bounds__(256) void paged_attn_mfma_kernel(AttnArgs a, Batch 
     Frag phi[MAPS][2], plo[MAPS][2];
     // a page whose 64 keys every row of this wavefront sees needs no mask arithmetic
     const bool inner = k0 + PAGE - 1 <= w_first && (!win || k0 >= w_lo_last || k0 + PAGE - 1 < keep);
+    float bias[4][4];
+    if (BIAS) {
+      const bool all_far = w_first - (k0 + PAGE - 1) >= a.n_bias - 1;
+#pragma unroll
+      for (int kb = 0; kb < 4; ++kb)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          bias[kb][i] = bias_far;
+          if (!all_far) {
+            const int dist = qpos - (k0 + 16 * kb + 4 * g4 + i), e = dist < 0 ? 0 : dist < a.n_bias ? dist : a.n_bias - 1;
+            bias[kb][i] = BIAS == 1 ? bias_lds[e] : btab[e];
+          }
+        }
+    }
 #pragma unroll
     for (int mp = 0; mp < MAPS; ++mp) {
       float mx = -1e30f;
@@ -190,6 +215,7 @@ __global__ __launch_bounds__(256) void paged_attn_mfma_kernel(AttnArgs a, Batch 
         for (int i = 0; i < 4; ++i) {
           float sc = S[mp][kb][i] * a.scale;
           if (biased) sc -= slope * (float)(qpos - (k0 + 16 * kb + 4 * g4 + i));
+          if (BIAS) sc += bias[kb][i];
           if (capped) sc = a.softcap * fast_tanh(sc * inv_cap);
           if (!inner) {
             const int key = k0 + 16 * kb + 4 * g4 + i;
@@ -501,7 +527,7 @@ static int launch_wide(AttnArgs a, Batch bt, unsigned grid, hipStream_t st) {
 
 extern "C" int ragged_paged_attn_mfma_wide(AttnArgs a, Batch bt, hipStream_t st) {
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || !ragged_paged_attn_mfma_wide_ok(a.d, a.vd)) return -1;
-  if (a.ldv < a.vd || a.ldv % 8 || a.keep_first > 0 || a.out_norm || a.gate || a.chunk > 0 || a.softcap > 0.f || a.sinks || a.slopes) return -1;
+  if (a.ldv < a.vd || a.ldv % 8 || a.keep_first > 0 || a.out_norm || a.gate || a.chunk > 0 || a.softcap > 0.f || a.sinks || a.slopes || a.dist_bias) return -1;
   if (!a.tiles || a.n_tiles <= 0 || (int64_t)a.n_tiles * a.H > 0x7fffffff) return -1;
   const unsigned grid = (unsigned)(a.n_tiles * a.H);
   const int dk = (a.d + 31) / 32, neb = a.vd / 16;
@@ -697,7 +723,7 @@ static int launch_heads(AttnArgs a, Batch bt, unsigned grid, hipStream_t st) {
 // token rows a.rows[0 .. n_rows) (all T rows without a list)
 extern "C" int ragged_paged_attn_mfma_heads(AttnArgs a, Batch bt, hipStream_t st) {
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || !ragged_paged_attn_mfma_wide_ok(a.d, a.vd)) return -1;
-  if (a.ldv < a.vd || a.ldv % 8 || a.keep_first > 0 || a.out_norm || a.gate || a.chunk > 0 || a.softcap > 0.f || a.sinks || a.slopes) return -1;
+  if (a.ldv < a.vd || a.ldv % 8 || a.keep_first > 0 || a.out_norm || a.gate || a.chunk > 0 || a.softcap > 0.f || a.sinks || a.slopes || a.dist_bias) return -1;
   const int nrows = a.rows ? a.n_rows : bt.T;
   const int nblk = (a.H / a.G + 15) / 16;
   if (nrows <= 0 || (int64_t)nrows * a.G * nblk > 0x7fffffff) return -1;
@@ -718,23 +744,27 @@ extern "C" int ragged_paged_attn_mfma_ok(int d, int vd) {
   return d % 8 == 0 && d <= 32 * MF_DK && vd % 16 == 0 && vd <= 16 * MF_NEB;
 }
 
-template <int MAPS>
+template <int MAPS, int BIAS>
 static void launch_mfma(AttnArgs a, Batch bt, unsigned grid, hipStream_t st) {
   const int dk = (a.d + 31) / 32;
-  if (dk == 1) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 1>), dim3(grid), dim3(256), 0, st, a, bt);
-  else if (dk == 2) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 2>), dim3(grid), dim3(256), 0, st, a, bt);
-  else if (dk == 3) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 3>), dim3(grid), dim3(256), 0, st, a, bt);
-  else hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 4>), dim3(grid), dim3(256), 0, st, a, bt);
+  const size_t lds = BIAS == 1 ? a.n_bias * sizeof(float) : 0;         // (beside the value tile: 34 KB at most)
+  if (dk == 1) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 1, BIAS>), dim3(grid), dim3(256), lds, st, a, bt);
+  else if (dk == 2) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 2, BIAS>), dim3(grid), dim3(256), lds, st, a, bt);
+  else if (dk == 3) hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 3, BIAS>), dim3(grid), dim3(256), lds, st, a, bt);
+  else hipLaunchKernelGGL((paged_attn_mfma_kernel<MAPS, 4, BIAS>), dim3(grid), dim3(256), lds, st, a, bt);
 }
 
 extern "C" int ragged_paged_attn_mfma(AttnArgs a, Batch bt, int maps, hipStream_t st) {
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || !ragged_paged_attn_mfma_ok(a.d, a.vd)) return -1;
   if (a.ldv < a.vd || a.ldv % 8) return -1;                  // value rows are read 16 bytes at a time
   // per-channel gate logits are read 8 bytes at a time
-  if (a.chunk < 0 || (a.gate_wide && (!a.gate || a.ldg % 4 || a.gate0 % 4)) || (a.sinks && !a.sink)) return -1;
+  if (a.chunk < 0 || (a.gate_wide && (!a.gate || a.ldg % 4 || a.gate0 % 4)) || (a.sinks && !a.sink) ||
+      (a.dist_bias && (a.n_bias <= 0 || maps != 1))) return -1;
   if ((maps != 1 && maps != 2) || !a.tiles || a.n_tiles <= 0 || (int64_t)a.n_tiles * a.H > 0x7fffffff) return -1;
   const unsigned grid = (unsigned)(a.n_tiles * a.H);
-  if (maps == 2) launch_mfma<2>(a, bt, grid, st);
-  else launch_mfma<1>(a, bt, grid, st);
+  if (maps == 2) launch_mfma<2, 0>(a, bt, grid, st);
+  else if (!a.dist_bias) launch_mfma<1, 0>(a, bt, grid, st);
+  else if (a.n_bias <= MF_BIAS) launch_mfma<1, 1>(a, bt, grid, st);
+  else launch_mfma<1, 2>(a, bt, grid, st);
   return RAGGED_LAUNCH_OK();
 }

@@ -57,6 +57,7 @@ __device__ __forceinline__ float lane_value(float v, int j) {
 }
 
 __device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + __expf(-x)); }
+__device__ __forceinline__ float softplusf_(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
 // Per-step description of the batch, all int32, one device buffer:
 //   tok_seq[T] tok_pos[T] | seq_start[B + 1] seq_past[B] seq_slot[B] | pages[B][max_pages]

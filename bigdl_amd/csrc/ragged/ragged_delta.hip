@@ -5,7 +5,9 @@
 // (decay, removal rate, unit key, state, outputs) is float whatever the activation type T is.
 // The gated delta rule is its relative with one decay g and one write strength beta per head,
 //     S' = g S,   u = beta (v - S'^T k),   S <- S' + k u^T,   o = S^T q,     k, q unit vectors behind short convolutions:
-// the same scan with two arrays and two scalars per token instead of five arrays.
+// the same scan with two arrays and two scalars per token instead of five arrays, or with three where g has a number per key
+// channel.  The state space recurrence (Mamba-2) is the one without the forgetting term,
+//     S <- exp(-a d) S + d B x^T,   y = S^T C + D x,     d = softplus(step logit + bias) per head.
 #include "ragged_common.h"
 
 using namespace ragged;
@@ -58,9 +60,10 @@ extern "C" int ragged_delta_gates(const void* P, int64_t ldp, int r0, int k0, in
 // The gated delta rule's inputs from this step's projections (columns 0 .. of P: q [G d] | k [G d] | v [H vd], all of them
 // behind a short causal convolution and silu): qf = unit(q) * d^(-1/2), kf = unit(k), float [rows, G d] each, with unit(u) =
 // u / sqrt(|u|^2 + tiny); vo of type T [rows, H vd]; gb float [rows, H, 2] = (exp(-arate softplus(a + dt bias)), sigmoid(b)).
+// With a decay per key channel: wf float [rows, H d] = exp(-arate_h softplus(wl + dt bias)), wl float logits, and gb = (1, sigmoid(b)).
 // The inputs before this step come from `state` [slots, taps - 1, C]; `write_state` (every sequence brings exactly one row)
 // also shifts it.  One wavefront per (block of rows, item): 2 G unit vectors, blocks
-// of value channels, the gates.
+// of value channels, blocks of decay channels, the gates.
 struct GatedDeltaArgs {
   const void* P;
   int64_t ldp;
@@ -69,8 +72,10 @@ struct GatedDeltaArgs {
   void* state;
   int b0, a0;            // columns of P: write strengths and step logits, H each
   const float* arate;    // [H]
-  const float* dt_bias;  // [H]
+  const float* dt_bias;  // [H], or with wl [H d]
   float tiny;
+  const float* wl;       // [rows, H d] or null: decay logits per key channel
+  float* wf;             // [rows, H d]
   float* qf;
   float* kf;
   void* vo;
@@ -94,11 +99,28 @@ __global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a,
     for (int e = lane; e < (t1 - t0) * a.H; e += 64) {
       const int t = t0 + e / a.H, h = e % a.H;
       const T* row = P + (int64_t)t * a.ldp;
-      const float z = to_f(row[a.a0 + h]) + a.dt_bias[h];
-      const float sp = fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
       float* o = a.gb + ((int64_t)t * a.H + h) * 2;
-      o[0] = expf(-a.arate[h] * sp);
+      o[0] = a.wl ? 1.f : expf(-a.arate[h] * softplusf_(to_f(row[a.a0 + h]) + a.dt_bias[h]));
       o[1] = 1.0f / (1.0f + expf(-to_f(row[a.b0 + h])));
+    }
+    return;
+  }
+  const int vitems = (a.H * a.vd + 64 * K - 1) / (64 * K);
+  if (it >= 2 * a.G + vitems) {                              // decays per key channel
+    const int HD = a.H * a.d, c0 = (it - 2 * a.G - vitems) * 64 * K + lane;
+    float rate[K], bias[K];
+#pragma unroll
+    for (int k = 0; k < K; ++k) {
+      const int c = c0 + 64 * k < HD ? c0 + 64 * k : HD - 1;
+      rate[k] = a.arate[c / a.d];
+      bias[k] = a.dt_bias[c];
+    }
+    for (int t = t0; t < t1; ++t) {
+#pragma unroll
+      for (int k = 0; k < K; ++k) {
+        const int c = c0 + 64 * k;
+        if (c < HD) a.wf[(int64_t)t * HD + c] = expf(-rate[k] * softplusf_(a.wl[(int64_t)t * HD + c] + bias[k]));
+      }
     }
     return;
   }
@@ -193,11 +215,12 @@ __global__ __launch_bounds__(256) void gated_delta_prep_kernel(GatedDeltaArgs a,
 
 template <typename T, int K>
 static void launch_gated_prep(GatedDeltaArgs a, Batch bt, hipStream_t st) {
-  const int items = 2 * a.G + (a.H * a.vd + 64 * K - 1) / (64 * K) + 1;
+  const int items = 2 * a.G + (a.H * a.vd + 64 * K - 1) / (64 * K) + (a.wl ? (a.H * a.d + 64 * K - 1) / (64 * K) : 0) + 1;
   const int RB = bt.T >= 512 ? 8 : bt.T >= 64 ? 2 : 1;
   const int64_t waves = (int64_t)((bt.T + RB - 1) / RB) * items;
   const dim3 grid((unsigned)((waves + 3) / 4));
   if (a.taps == 4) hipLaunchKernelGGL((gated_delta_prep_kernel<T, K, 4>), grid, dim3(256), 0, st, a, items, RB, bt);
+  else if (a.taps == 3) hipLaunchKernelGGL((gated_delta_prep_kernel<T, K, 3>), grid, dim3(256), 0, st, a, items, RB, bt);
   else hipLaunchKernelGGL((gated_delta_prep_kernel<T, K, 0>), grid, dim3(256), 0, st, a, items, RB, bt);
 }
 
@@ -205,8 +228,8 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.d <= 0 || a.d > 1024 || a.vd <= 0 || a.taps < 1 || a.taps > 16) return -1;
   if (!a.P || !a.cw || (a.taps > 1 && !a.state) || !a.arate || !a.dt_bias || !a.qf || !a.kf || !a.vo || !a.gb) return -1;
   const int C = 2 * a.G * a.d + a.H * a.vd;
-  if (a.b0 < C || a.a0 < C || a.ldp < a.b0 + a.H || a.ldp < a.a0 + a.H || (a.write_state && bt.B != bt.T)) return -1;
-  if ((int64_t)bt.T * (2 * a.G + a.H * a.vd) > 0x7fffffff) return -1;
+  if (a.b0 < C || a.ldp < a.b0 + a.H || (!a.wl && (a.a0 < C || a.ldp < a.a0 + a.H)) || (a.wl && !a.wf) || (a.write_state && bt.B != bt.T)) return -1;
+  if ((int64_t)bt.T * (2 * a.G + a.H * (a.vd + a.d)) > 0x7fffffff) return -1;
   if (a.taps == 1) a.write_state = 0;
   RAGGED_DISPATCH(dtype,
     if (a.d <= 64) launch_gated_prep<T, 1>(a, bt, st);
@@ -226,22 +249,39 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
 // while the previous block is scanned (register look-ahead, two LDS buffers) and read back as 16-byte broadcasts.
 // Grid: (column blocks, heads, sequences).  `values` = 0: v is taken as 0 (the state only decays and forgets: from an
 // identity state this yields a chunk's transition matrix).
-// NA = 5: the generalised rule.  NA = 2: the gated rule; the arrays are q and k of G heads (head h reads head h / (H / G)),
-// `gb` holds every token's decay and write strength per head, and the four arrays of the general form shrink to k and scalars:
-// w = g, n = k, b = beta g k, and k v takes the factor beta.
+// MODE: which recurrence.
+//   general  five arrays, as above.
+//   gated    q and k of G heads (head h reads head h / (H / G)); `gb` holds every token's decay and write strength per head, and the
+//            four arrays of the general form shrink to k and scalars: w = g, n = k, b = beta g k, and k v takes the factor beta.
+//   channel  the gated rule with a decay per key channel: q, k and the decays w of H heads; of `gb` only the write strength counts.
+//   space    the state space recurrence: q and k are the rows C and B of G groups, columns c0 .. and b0 .. of P (type T); a token's
+//            decay and step size per head come from its step logit (`ss`), the read-out takes D v on top.
+enum DeltaMode { DL_GENERAL, DL_GATED, DL_CHANNEL, DL_SPACE };
+
+struct SpaceArgs {
+  const void* dt;        // step logits: row t, column h of a [rows, lddt] matrix of type T
+  int64_t lddt;
+  const float* dt_bias;  // [H]
+  const float* rate;     // [H]
+  const float* D;        // [H]
+  int b0, c0;
+};
+
 constexpr int DL_DR = 32;
 constexpr int DL_SEG = DL_DR + 4;   // LDS floats per lane group and token (padding shifts the banks between groups)
 constexpr int DL_TBR = 32;          // TB * R <= this
 
-template <typename T, int NW, int NA>
+template <typename T, int NW, int MODE>
 __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ rf, const float* __restrict__ wf,
                                                          const float* __restrict__ nf, const float* __restrict__ bf,
                                                          const float* __restrict__ kf, const float* __restrict__ gb, int G,
                                                          const T* __restrict__ P, int64_t ldp, int v0,
                                                          float* __restrict__ state, float* __restrict__ out, int H, int d, int vd,
-                                                         int R, int TB, int values, Batch bt) {
+                                                         int R, int TB, int values, SpaceArgs ss, Batch bt) {
+  constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2, KI = MODE == DL_GENERAL ? 4 : 1;    // arrays, k's place among them
+  constexpr bool GB = MODE != DL_GENERAL;                    // two scalars per token
   constexpr int NT = 64 * NW, DL_PRE = NA * DL_TBR * DL_DR / NT;
-  extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k (r, k): [TB][R][SEG] each, v[TB][wcols], (g, beta)[TB] }
+  extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k (r, k, w): [TB][R][SEG] each, v[TB][wcols], (g, beta)[TB] }
   const int b = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63;
   const int cols = 64 / R, wcols = NW * cols;
@@ -250,9 +290,11 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
   const int start = bt.seq_start[b], n = bt.seq_start[b + 1] - start, past = bt.seq_past[b], slot = bt.seq_slot[b];
   const bool colok = col < vd;
   const int row0 = r * DL_DR;
-  const int HD = NA == 2 ? G * d : H * d, hd0 = NA == 2 ? h / (H / G) * d : h * d;      // floats of an array's row, this head's first
+  const int gh = GB ? h / (H / G) : h;                       // the head of q and k that this head reads
+  const int HD = GB ? G * d : H * d, hd0 = gh * d;           // floats of an array's row, this head's first
   const int qsz = TB * R * DL_SEG;                         // floats of one array in a buffer
-  const int bufsz = NA * qsz + TB * wcols + (NA == 2 ? (2 * TB + 3) & ~3 : 0);
+  const int bufsz = NA * qsz + TB * wcols + (GB ? (2 * TB + 3) & ~3 : 0);
+  const float rate = MODE == DL_SPACE ? ss.rate[h] : 0.f, dtb = MODE == DL_SPACE ? ss.dt_bias[h] : 0.f, skip = MODE == DL_SPACE ? ss.D[h] : 0.f;
   float S[DL_DR];
   float* sp = state + (((int64_t)slot * H + h) * d) * vd;
   {
@@ -278,12 +320,27 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
       const int tk = ta / NA, which = ta - tk * NA;
       float v = NA == 5 && which == 1 ? 1.f : 0.f;         // padding: w = 1, everything else 0
       if (e < live && row < d) {
-        const float* src = which == 0 ? rf : NA == 2 ? kf : which == 1 ? wf : which == 2 ? nf : which == 3 ? bf : kf;
-        v = src[(int64_t)(start + i0 + tk) * HD + hd0 + row];
+        const int64_t t = start + i0 + tk;
+        if (MODE == DL_SPACE) {
+          v = to_f(P[t * ldp + (which == 0 ? ss.c0 : ss.b0) + hd0 + row]);
+        } else if (MODE == DL_CHANNEL && which == 2) {
+          v = wf[t * (H * d) + h * d + row];
+        } else {
+          const float* src = which == 0 ? rf : GB ? kf : which == 1 ? wf : which == 2 ? nf : which == 3 ? bf : kf;
+          v = src[t * HD + hd0 + row];
+        }
       }
       pre[u] = v;
     }
-    if (NA == 2 && tid < 2 * TB && i0 + (tid >> 1) < n) preg = gb[((int64_t)(start + i0 + (tid >> 1)) * H + h) * 2 + (tid & 1)];
+    if (GB && tid < 2 * TB && i0 + (tid >> 1) < n) {
+      const int64_t t = start + i0 + (tid >> 1);
+      if (MODE == DL_SPACE) {
+        const float step = softplusf_(to_f(((const T*)ss.dt)[t * ss.lddt + h]) + dtb);
+        preg = (tid & 1) ? step : expf(-rate * step);
+      } else {
+        preg = gb[(t * H + h) * 2 + (tid & 1)];
+      }
+    }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
       const int e = tid + NT * u;
@@ -312,7 +369,7 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
       const int e = tid + NT * u;
       if (e < TB * wcols) buf[NA * qsz + e] = prev[u];
     }
-    if (NA == 2 && tid < 2 * TB) buf[NA * qsz + TB * wcols + tid] = preg;
+    if (GB && tid < 2 * TB) buf[NA * qsz + TB * wcols + tid] = preg;
   };
   if (n > 0) { fetch(0); stash(smem, 0); }
   __syncthreads();
@@ -325,23 +382,40 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
     for (int tk = 0; tk < nt; ++tk) {
       const int seg = (tk * R + r) * DL_SEG;
       const float4* r4 = reinterpret_cast<const float4*>(buf + seg);
-      const float4* k4 = reinterpret_cast<const float4*>(buf + (NA - 1) * qsz + seg);
-      const float4* w4 = reinterpret_cast<const float4*>(buf + qsz + seg);               // (NA == 5)
+      const float4* k4 = reinterpret_cast<const float4*>(buf + KI * qsz + seg);
+      const float4* w4 = reinterpret_cast<const float4*>(buf + (NA == 3 ? 2 : 1) * qsz + seg);      // (NA == 5, 3)
       const float4* n4 = NA == 5 ? reinterpret_cast<const float4*>(buf + 2 * qsz + seg) : k4;
       const float4* b4 = reinterpret_cast<const float4*>(buf + (NA == 5 ? 3 * qsz : 0) + seg);   // (NA == 5)
       const float v = buf[NA * qsz + tk * wcols + lc];
-      // n . s over the old state
-      float acc[4] = {0.f, 0.f, 0.f, 0.f};
+      // n . s over the old state (with a decay per channel over the decayed state)
+      float acc[4] = {0.f, 0.f, 0.f, 0.f}, dot = 0.f;
+      if (MODE != DL_SPACE) {
 #pragma unroll
-      for (int k = 0; k < DL_DR / 4; ++k) {
-        const float4 a = n4[k];
-        acc[0] += S[4 * k] * a.x; acc[1] += S[4 * k + 1] * a.y; acc[2] += S[4 * k + 2] * a.z; acc[3] += S[4 * k + 3] * a.w;
+        for (int k = 0; k < DL_DR / 4; ++k) {
+          if (MODE == DL_CHANNEL) {
+            const float4 w = w4[k];
+            S[4 * k] *= w.x; S[4 * k + 1] *= w.y; S[4 * k + 2] *= w.z; S[4 * k + 3] *= w.w;
+          }
+          const float4 a = n4[k];
+          acc[0] += S[4 * k] * a.x; acc[1] += S[4 * k + 1] * a.y; acc[2] += S[4 * k + 2] * a.z; acc[3] += S[4 * k + 3] * a.w;
+        }
+        dot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
+        acc[0] = acc[1] = acc[2] = acc[3] = 0.f;
       }
-      const float dot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
-      acc[0] = acc[1] = acc[2] = acc[3] = 0.f;
-      if (NA == 2) {
+      if (MODE == DL_CHANNEL) {
+        const float c = buf[NA * qsz + TB * wcols + 2 * tk + 1] * (v - dot);
+#pragma unroll
+        for (int k = 0; k < DL_DR / 4; ++k) {
+          const float4 kk = k4[k], q = r4[k];
+          S[4 * k] += kk.x * c;
+          S[4 * k + 1] += kk.y * c;
+          S[4 * k + 2] += kk.z * c;
+          S[4 * k + 3] += kk.w * c;
+          acc[0] += S[4 * k] * q.x; acc[1] += S[4 * k + 1] * q.y; acc[2] += S[4 * k + 2] * q.z; acc[3] += S[4 * k + 3] * q.w;
+        }
+      } else if (GB) {
         const float2 gs = *reinterpret_cast<const float2*>(buf + NA * qsz + TB * wcols + 2 * tk);
-        const float w = gs.x, c = gs.y * (v - w * dot);
+        const float w = gs.x, c = MODE == DL_SPACE ? gs.y * v : gs.y * (v - w * dot);
 #pragma unroll
         for (int k = 0; k < DL_DR / 4; ++k) {
           const float4 kk = k4[k], q = r4[k];
@@ -362,7 +436,7 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
           acc[0] += S[4 * k] * q.x; acc[1] += S[4 * k + 1] * q.y; acc[2] += S[4 * k + 2] * q.z; acc[3] += S[4 * k + 3] * q.w;
         }
       }
-      const float tot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
+      const float tot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R) + (MODE == DL_SPACE ? skip * v : 0.f);
       if (out && r == 0 && colok) out[(int64_t)(start + i0 + tk) * (H * vd) + h * vd + col] = tot;
     }
     if (more) stash(smem + (cur ^ 1) * bufsz, i0 + TB);
@@ -376,10 +450,11 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
   }
 }
 
-template <int NA>
+template <int MODE>
 static int launch_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const float* gb, int G,
-                             const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
-                             int dtype, hipStream_t st) {
+                             const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, SpaceArgs ss,
+                             Batch bt, int dtype, hipStream_t st) {
+  constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2;
   if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 32 || (values && !P)) return -1;
   int R = 1;
   while (R * DL_DR < d) R <<= 1;
@@ -388,14 +463,14 @@ static int launch_delta_scan(const float* rf, const float* wf, const float* nf, 
   int TB = DL_TBR / R < 16 ? DL_TBR / R : 16;
   if (TB * wcols > 4 * 64 * nw) TB = 4 * 64 * nw / wcols;   // the value look-ahead holds 4 floats per thread
   if (TB < 1) return -1;
-  // (2 TB <= 32 threads bring the gated rule's scalars; TB wcols and a buffer's parts are multiples of 16 bytes)
-  const size_t sm = 2 * (size_t)(NA * TB * R * DL_SEG + TB * wcols + (NA == 2 ? (2 * TB + 3) & ~3 : 0)) * sizeof(float);
+  // (2 TB <= 32 threads bring a token's two scalars; TB wcols and a buffer's parts are multiples of 16 bytes)
+  const size_t sm = 2 * (size_t)(NA * TB * R * DL_SEG + TB * wcols + (MODE != DL_GENERAL ? (2 * TB + 3) & ~3 : 0)) * sizeof(float);
   const dim3 grid((vd + wcols - 1) / wcols, H, bt.B);
   RAGGED_DISPATCH(dtype,
-    if (nw == 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, NA>), grid, dim3(128), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp,
-                                    v0, state, out, H, d, vd, R, TB, values, bt);
-    else hipLaunchKernelGGL((delta_scan_kernel<T, 4, NA>), grid, dim3(256), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp, v0,
-                            state, out, H, d, vd, R, TB, values, bt))
+    if (nw == 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, MODE>), grid, dim3(128), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp,
+                                    v0, state, out, H, d, vd, R, TB, values, ss, bt);
+    else hipLaunchKernelGGL((delta_scan_kernel<T, 4, MODE>), grid, dim3(256), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp, v0,
+                            state, out, H, d, vd, R, TB, values, ss, bt))
   return RAGGED_LAUNCH_OK();
 }
 
@@ -403,14 +478,24 @@ static int launch_delta_scan(const float* rf, const float* wf, const float* nf, 
 extern "C" int ragged_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const void* P,
                                  int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
                                  int dtype, hipStream_t st) {
-  return launch_delta_scan<5>(rf, wf, nf, bf, kf, nullptr, H, P, ldp, v0, state, out, H, d, vd, values, bt, dtype, st);
+  return launch_delta_scan<DL_GENERAL>(rf, wf, nf, bf, kf, nullptr, H, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt, dtype, st);
 }
 
-// the gated rule: qf, kf [rows, G d], gb [rows, H, 2]
-extern "C" int ragged_gated_delta_scan(const float* qf, const float* kf, const float* gb, int G, const void* P, int64_t ldp, int v0,
+// the gated rule: qf, kf [rows, G d], gb [rows, H, 2]; wf [rows, H d] or null: a decay per key channel
+extern "C" int ragged_gated_delta_scan(const float* qf, const float* kf, const float* wf, const float* gb, int G, const void* P, int64_t ldp, int v0,
                                        float* state, float* out, int H, int d, int vd, int values, Batch bt, int dtype, hipStream_t st) {
   if (G <= 0 || H % G || !gb) return -1;
-  return launch_delta_scan<2>(qf, nullptr, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, bt, dtype, st);
+  if (wf) return launch_delta_scan<DL_CHANNEL>(qf, wf, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt,
+                                               dtype, st);
+  return launch_delta_scan<DL_GATED>(qf, nullptr, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt, dtype, st);
+}
+
+// the state space recurrence: X [rows, ldx] of type T holds x (columns 0 .. H vd), B and C (columns b0 .., c0 .., G d each)
+extern "C" int ragged_state_space_scan(SpaceArgs ss, const void* X, int64_t ldx, int G, float* state, float* out, int H, int d, int vd,
+                                       Batch bt, int dtype, hipStream_t st) {
+  if (G <= 0 || H % G || !ss.dt || !ss.dt_bias || !ss.rate || !ss.D || ss.lddt < H || ss.b0 < 0 || ss.c0 < 0) return -1;
+  if (ldx < (int64_t)H * vd || ldx < ss.b0 + (int64_t)G * d || ldx < ss.c0 + (int64_t)G * d || !out) return -1;
+  return launch_delta_scan<DL_SPACE>(nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, G, X, ldx, 0, state, out, H, d, vd, 1, ss, bt, dtype, st);
 }
 
 // ---------------------------------------------------------------------------------------------------------------

@@ -13,12 +13,17 @@ constexpr int MOE_SLOTS = MOE_MAX_E / 64;
 // the bfloat16 rounding of the normed stream).  Experts form `groups` equal runs of neighbours; a group's score is the sum
 // of its `group_top` (1 or 2) best experts' scores; the `top` best experts of the `keep` best groups are chosen, best
 // first, with weight s * scale, or (renorm) s / (sum of the chosen s + 1e-20) * scale.  Ties go to the lower lane.
+// `corr` [E] or null: what is compared, for groups and experts alike, is s + corr (of either sign); the weights are made of s.
+// `wg` [D] or null: one more router row, gate_out[t] = sigmoid(wg . x) (how much of a shared expert a row takes).
 // One workgroup of four wavefronts per row: the wavefronts share the router's rows, wavefront 0 chooses.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x, int64_t ldx, const float* __restrict__ wr,
                                                         int* __restrict__ idx, float* __restrict__ wts, int D, int E, int groups,
-                                                        int keep, int top, float scale, int score_fn, int group_top, int renorm) {
+                                                        int keep, int top, float scale, int score_fn, int group_top, int renorm,
+                                                        const float* __restrict__ corr, const float* __restrict__ wg,
+                                                        float* __restrict__ gate_out) {
   __shared__ float z[MOE_MAX_E];
+  __shared__ float zc[MOE_MAX_E];                                  // what the choice compares
   __shared__ float gbest[64];
   extern __shared__ __attribute__((aligned(16))) float xs[];       // the row as floats
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -57,7 +62,14 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
     if (lane == 0) { z[e0] = a0; z[e1] = a1; }
   }
   __syncthreads();
+  if (wg && wave == 3) {
+    float g = 0.f;
+    for (int c = lane; c < D; c += 64) g += wg[c] * xs[c];
+    g = wave_sum(g);
+    if (lane == 0) gate_out[t] = 1.0f / (1.0f + expf(-g));
+  }
   if (wave != 0) return;
+  constexpr float NONE = -INFINITY;
   float s[MOE_SLOTS];
   if (score_fn == 1) {
 #pragma unroll
@@ -90,22 +102,28 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
       if (e < E) z[e] = s[k];
     }
   }
+#pragma unroll
+  for (int k = 0; k < MOE_SLOTS; ++k) {
+    const int e = lane + 64 * k;
+    s[k] = e < E ? s[k] + (corr ? corr[e] : 0.f) : NONE;
+    if (e < E) zc[e] = s[k];
+  }
   // (a wavefront's LDS requests are served in order: the scores written above are what is read below)
   const int gsz = E / groups;
   if (groups > 1 && keep < groups) {
-    float g = -1.f;
+    float g = NONE;
     if (lane < groups) {
-      float second = 0.f;                                   // (scores are not negative: a group of one adds nothing)
+      float second = NONE;
       for (int j = 0; j < gsz; ++j) {
-        const float v = z[lane * gsz + j];
-        if (v > g) { second = g > 0.f ? g : 0.f; g = v; }
+        const float v = zc[lane * gsz + j];
+        if (v > g) { second = g; g = v; }
         else if (v > second) second = v;
       }
-      if (group_top == 2) g += second;
+      if (group_top == 2 && gsz > 1) g += second;           // (a group of one adds nothing)
     }
     bool kept = false;
     for (int it = 0; it < keep; ++it) {
-      const float best = wave_max(kept ? -1.f : g);
+      const float best = wave_max(kept ? NONE : g);
       const unsigned long long who = __ballot(!kept && g == best && lane < groups);
       if (lane == __ffsll((long long)who) - 1) kept = true;
     }
@@ -113,12 +131,9 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
 #pragma unroll
     for (int k = 0; k < MOE_SLOTS; ++k) {
       const int e = lane + 64 * k;
-      if (e < E && gbest[e / gsz] == 0.f) s[k] = -1.f;
+      if (e < E && gbest[e / gsz] == 0.f) s[k] = NONE;
     }
   }
-#pragma unroll
-  for (int k = 0; k < MOE_SLOTS; ++k)
-    if (lane + 64 * k >= E) s[k] = -1.f;
   float total = 0.f, kept_w = 0.f;                         // lane `it` keeps the score of the it-th choice (top <= 64 with renorm)
   for (int it = 0; it < top; ++it) {
     float mine = s[0];
@@ -128,27 +143,31 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
       if (s[k] > mine) { mine = s[k]; at = k; }
     const float best = wave_max(mine);
     const unsigned long long who = __ballot(mine == best);
-    total += best;
-    if (lane == (it & 63)) kept_w = best;
-    if (lane == __ffsll((long long)who) - 1) {
-      idx[(int64_t)t * top + it] = lane + 64 * at;
-      if (!renorm) wts[(int64_t)t * top + it] = best * scale;
+    const int winner = who ? __ffsll((long long)who) - 1 : 0;       // (scores that are no numbers: some expert, never an index outside)
+    const int e = __shfl(lane + 64 * at, winner, 64);
+    const float score = z[e < E ? e : 0];
+    total += score;
+    if (lane == (it & 63)) kept_w = score;
+    if (lane == winner) {
+      idx[(int64_t)t * top + it] = e < E ? e : 0;
+      if (!renorm) wts[(int64_t)t * top + it] = score * scale;
 #pragma unroll
       for (int k = 0; k < MOE_SLOTS; ++k)
-        if (k == at) s[k] = -2.f;
+        if (k == at) s[k] = NONE;
     }
   }
   if (renorm && lane < top) wts[(int64_t)t * top + lane] = kept_w / (total + 1e-20f) * scale;
 }
 
 extern "C" int ragged_moe_route(const void* x, int64_t ldx, const float* wr, int* idx, float* wts, int64_t rows, int D, int E,
-                                int groups, int keep, int top, float scale, int score_fn, int group_top, int renorm, int dtype,
-                                hipStream_t st) {
+                                int groups, int keep, int top, float scale, int score_fn, int group_top, int renorm, const float* corr,
+                                const float* wg, float* gate_out, int dtype, hipStream_t st) {
+  if (wg && !gate_out) return -1;
   if (score_fn < 0 || score_fn > 1 || group_top < 1 || group_top > 2 || (renorm && top > 64)) return -1;
   if (rows <= 0 || rows > 0x7fffffff || D <= 0 || D > 12288 || E <= 0 || E > MOE_MAX_E || groups <= 0 || groups > 64 || E % groups) return -1;
   if (keep <= 0 || keep > groups || top <= 0 || top > keep * (E / groups)) return -1;
   RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((moe_route_kernel<T>), dim3((unsigned)rows), dim3(256), D * sizeof(float), st, (const T*)x, ldx, wr, idx,
-                                            wts, D, E, groups, keep, top, scale, score_fn, group_top, renorm))
+                                            wts, D, E, groups, keep, top, scale, score_fn, group_top, renorm, corr, wg, gate_out))
   return RAGGED_LAUNCH_OK();
 }
 

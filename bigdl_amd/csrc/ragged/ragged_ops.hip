@@ -535,26 +535,34 @@ extern "C" int ragged_row_norm(const float* x, const float* w, void* out, int64_
 
 // ---------------------------------------------------------------------------------------------------------------
 // Embedding rows as the float stream: x[t] = scale * table[ids[t]] (+ table2[ids2[t]]), summed in float.  The second
-// table serves embeddings of token pairs (a row chosen by a hash of the previous and the current token).
+// table serves embeddings of token pairs (a row chosen by a hash of the previous and the current token).  With `norm` the
+// row is divided by its root mean square and weighted.
 template <typename T>
 __global__ __launch_bounds__(256) void embed_rows_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
                                                          const int64_t* __restrict__ ids2, const T* __restrict__ table2,
-                                                         float scale, float* __restrict__ x, int D) {
+                                                         float scale, const float* __restrict__ norm, float eps,
+                                                         float* __restrict__ x, int D) {
+  __shared__ float red[4];
   const int64_t t = blockIdx.x;
   const T* r1 = table + ids[t] * D;
   const T* r2 = table2 ? table2 + ids2[t] * D : nullptr;
+  float ss = 0.f;
   for (int c = threadIdx.x; c < D; c += 256) {
     float v = to_f(r1[c]) * scale;
     if (r2) v += to_f(r2[c]);
     x[t * D + c] = v;
+    ss += v * v;
   }
+  if (!norm) return;
+  const float r = 1.0f / sqrtf(block_sum_256(ss, red) / (float)D + eps);
+  for (int c = threadIdx.x; c < D; c += 256) x[t * D + c] *= r * norm[c];      // (what this thread has written itself)
 }
 
 extern "C" int ragged_embed_rows(const int64_t* ids, const void* table, const int64_t* ids2, const void* table2, float scale,
-                                 float* x, int64_t rows, int D, int dtype, hipStream_t st) {
+                                 const float* norm, float eps, float* x, int64_t rows, int D, int dtype, hipStream_t st) {
   if (rows <= 0 || rows > 0x7fffffff || D <= 0 || !ids || !table || !x || (table2 && !ids2)) return -1;
   RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((embed_rows_kernel<T>), dim3((unsigned)rows), dim3(256), 0, st, ids, (const T*)table, ids2,
-                                            (const T*)table2, scale, x, D))
+                                            (const T*)table2, scale, norm, eps, x, D))
   return RAGGED_LAUNCH_OK();
 }
 
@@ -619,11 +627,247 @@ extern "C" int ragged_add_norm(float* x, const void* y1, const void* y2, const f
 }
 
 // ---------------------------------------------------------------------------------------------------------------
+// Parallel block with a norm per sublayer: x <- x + u + y2 on the float stream, u = y or mix * (rms(ya) wa + rms(yb) wb) (two
+// mixers side by side whose outputs are normed over the row), then u1 = rms(x) w1 and u2 = rms(x) w2 for the products that read
+// the stream next (w2 null: only u1; w1 null: neither).  Without any y it norms the stream as it is.  One workgroup per row.
+// V channels per load and NU such pieces per thread stay in registers (NU V 256 >= D); NU = 0: any D, the passes re-read.
+struct JoinArgs {
+  float* x;
+  const void* y;
+  const void* y2;
+  const void* ya;
+  const void* yb;
+  const float* wa;
+  const float* wb;
+  float mix;
+  const float* w1;
+  const float* w2;
+  void* u1;
+  void* u2;
+  int D;
+  float eps;
+};
+
+template <typename T, int V> __device__ __forceinline__ void load_piece(const T* p, float (&o)[V]) {
+  if (V == 4 && sizeof(T) == 2) {
+    const uint2 q = *reinterpret_cast<const uint2*>(p);
+    o[0] = __uint_as_float(q.x << 16);
+    o[1 % V] = __uint_as_float(q.x & 0xffff0000u);
+    o[2 % V] = __uint_as_float(q.y << 16);
+    o[3 % V] = __uint_as_float(q.y & 0xffff0000u);
+  } else if (V == 4) {
+    const float4 q = *reinterpret_cast<const float4*>(p);
+    o[0] = q.x; o[1 % V] = q.y; o[2 % V] = q.z; o[3 % V] = q.w;
+  } else {
+    o[0] = to_f(*p);
+  }
+}
+template <typename T, int V> __device__ __forceinline__ void store_piece(T* p, const float (&v)[V]) {
+  if (V == 4 && sizeof(T) == 2) {
+    uint2 q;
+    q.x = (uint32_t)from_f<bf16>(v[0]).b | ((uint32_t)from_f<bf16>(v[1 % V]).b << 16);
+    q.y = (uint32_t)from_f<bf16>(v[2 % V]).b | ((uint32_t)from_f<bf16>(v[3 % V]).b << 16);
+    *reinterpret_cast<uint2*>(p) = q;
+  } else if (V == 4) {
+    *reinterpret_cast<float4*>(p) = float4{v[0], v[1 % V], v[2 % V], v[3 % V]};
+  } else {
+    *p = from_f<T>(v[0]);
+  }
+}
+
+template <typename T, int NU, int V>
+__global__ __launch_bounds__(256) void join_norms_kernel(JoinArgs a) {
+  __shared__ float red[12];
+  const int D = a.D;
+  const int64_t base = (int64_t)blockIdx.x * D;
+  float* x = a.x + base;
+  const T* y = a.y ? (const T*)a.y + base : nullptr;
+  const T* y2 = a.y2 ? (const T*)a.y2 + base : nullptr;
+  const T* ya = a.ya ? (const T*)a.ya + base : nullptr;
+  const T* yb = a.yb ? (const T*)a.yb + base : nullptr;
+  const bool adds = y || y2 || ya;
+  if (NU > 0) {
+    constexpr int U = NU > 0 ? NU : 1;
+    float xv[U][V], av[U][V], bv[U][V], sa = 0.f, sb = 0.f, ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = (threadIdx.x + 256 * u) * V;
+      if (c < D) {                                           // (D is a multiple of V)
+        load_piece<float, V>(x + c, xv[u]);
+        if (ya) { load_piece<T, V>(ya + c, av[u]); load_piece<T, V>(yb + c, bv[u]); }
+        if (y) load_piece<T, V>(y + c, av[u]);
+        if (y2) {
+          float t[V];
+          load_piece<T, V>(y2 + c, t);
+#pragma unroll
+          for (int i = 0; i < V; ++i) xv[u][i] += t[i];
+        }
+#pragma unroll
+        for (int i = 0; i < V; ++i) {
+          if (ya) { sa += av[u][i] * av[u][i]; sb += bv[u][i] * bv[u][i]; }
+          if (y) xv[u][i] += av[u][i];
+        }
+      }
+    }
+    if (ya) {
+      const float ra = a.mix / sqrtf(block_sum_256(sa, red) / (float)D + a.eps), rb = a.mix / sqrtf(block_sum_256(sb, red + 4) / (float)D + a.eps);
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int c = (threadIdx.x + 256 * u) * V;
+        if (c < D) {
+          float wa[V], wb[V];
+          load_piece<float, V>(a.wa + c, wa);
+          load_piece<float, V>(a.wb + c, wb);
+#pragma unroll
+          for (int i = 0; i < V; ++i) xv[u][i] += av[u][i] * ra * wa[i] + bv[u][i] * rb * wb[i];
+        }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = (threadIdx.x + 256 * u) * V;
+      if (c < D) {
+        if (adds) store_piece<float, V>(x + c, xv[u]);
+#pragma unroll
+        for (int i = 0; i < V; ++i) ss += xv[u][i] * xv[u][i];
+      }
+    }
+    if (!a.u1) return;
+    const float r = 1.0f / sqrtf(block_sum_256(ss, red + 8) / (float)D + a.eps);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = (threadIdx.x + 256 * u) * V;
+      if (c < D) {
+        float w[V], o[V];
+        load_piece<float, V>(a.w1 + c, w);
+#pragma unroll
+        for (int i = 0; i < V; ++i) o[i] = xv[u][i] * r * w[i];
+        store_piece<T, V>((T*)a.u1 + base + c, o);
+        if (a.u2) {
+          load_piece<float, V>(a.w2 + c, w);
+#pragma unroll
+          for (int i = 0; i < V; ++i) o[i] = xv[u][i] * r * w[i];
+          store_piece<T, V>((T*)a.u2 + base + c, o);
+        }
+      }
+    }
+    return;
+  }
+  float ra = 0.f, rb = 0.f, ss = 0.f;
+  if (ya) {
+    float sa = 0.f, sb = 0.f;
+    for (int c = threadIdx.x; c < D; c += 256) {
+      const float p = to_f(ya[c]), q = to_f(yb[c]);
+      sa += p * p;
+      sb += q * q;
+    }
+    ra = a.mix / sqrtf(block_sum_256(sa, red) / (float)D + a.eps);
+    rb = a.mix / sqrtf(block_sum_256(sb, red + 4) / (float)D + a.eps);
+  }
+  for (int c = threadIdx.x; c < D; c += 256) {
+    float v = x[c] + (y2 ? to_f(y2[c]) : 0.f);
+    if (y) v += to_f(y[c]);
+    if (ya) v += to_f(ya[c]) * ra * a.wa[c] + to_f(yb[c]) * rb * a.wb[c];
+    if (adds) x[c] = v;
+    ss += v * v;
+  }
+  if (!a.u1) return;
+  const float r = 1.0f / sqrtf(block_sum_256(ss, red + 8) / (float)D + a.eps);
+  for (int c = threadIdx.x; c < D; c += 256) {               // (each thread re-reads what it has written itself)
+    const float v = x[c] * r;
+    ((T*)a.u1)[base + c] = from_f<T>(v * a.w1[c]);
+    if (a.u2) ((T*)a.u2)[base + c] = from_f<T>(v * a.w2[c]);
+  }
+}
+
+extern "C" int ragged_join_norms(JoinArgs a, int64_t rows, int dtype, hipStream_t st) {
+  if (rows <= 0 || rows > 0x7fffffff || a.D <= 0 || !a.x || (a.y && a.ya) || (a.ya && (!a.yb || !a.wa || !a.wb))) return -1;
+  if ((a.u1 && !a.w1) || (a.u2 && (!a.w2 || !a.u1))) return -1;
+  auto aligned = [](const void* p, size_t n) { return ((uintptr_t)p % n) == 0; };
+  RAGGED_DISPATCH(dtype,
+    const size_t n = 4 * sizeof(T);
+    const bool vec = a.D % 4 == 0 && aligned(a.x, 16) && aligned(a.wa, 16) && aligned(a.wb, 16) && aligned(a.w1, 16) && aligned(a.w2, 16) &&
+                     aligned(a.y, n) && aligned(a.y2, n) && aligned(a.ya, n) && aligned(a.yb, n) && aligned(a.u1, n) && aligned(a.u2, n);
+    const dim3 grid((unsigned)rows);
+    if (vec && a.D <= 1024) hipLaunchKernelGGL((join_norms_kernel<T, 1, 4>), grid, dim3(256), 0, st, a);
+    else if (vec && a.D <= 2048) hipLaunchKernelGGL((join_norms_kernel<T, 2, 4>), grid, dim3(256), 0, st, a);
+    else if (vec && a.D <= 4096) hipLaunchKernelGGL((join_norms_kernel<T, 4, 4>), grid, dim3(256), 0, st, a);
+    else if (a.D <= 1024) hipLaunchKernelGGL((join_norms_kernel<T, 4, 1>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((join_norms_kernel<T, 0, 1>), grid, dim3(256), 0, st, a))
+  return RAGGED_LAUNCH_OK();
+}
+
+// out = w * groupnorm(y * silu(P[:, z0 ..])) over `groups` equal parts of a row (each by its own root mean square): float head
+// outputs y [rows, n], gated before the norm.  One workgroup per (row, part); NU V 256 >= n / groups, or NU = 0 for any size.
+template <typename T, int NU, int V>
+__global__ __launch_bounds__(256) void gate_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ P, int64_t ldp, int z0,
+                                                              const float* __restrict__ w, T* __restrict__ out, int n, int groups, float eps) {
+  __shared__ float red[4];
+  const int row = blockIdx.x / groups, g = blockIdx.x % groups, dg = n / groups, c0 = g * dg;
+  const float* yr = y + (int64_t)row * n + c0;
+  const T* zr = P + (int64_t)row * ldp + z0 + c0;
+  T* orow = out + (int64_t)row * n + c0;
+  float ss = 0.f;
+  if (NU > 0) {
+    constexpr int U = NU > 0 ? NU : 1;
+    float v[U][V];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = (threadIdx.x + 256 * u) * V;
+      if (c < dg) {
+        float z[V];
+        load_piece<float, V>(yr + c, v[u]);
+        load_piece<T, V>(zr + c, z);
+#pragma unroll
+        for (int i = 0; i < V; ++i) { v[u][i] *= z[i] / (1.0f + expf(-z[i])); ss += v[u][i] * v[u][i]; }
+      }
+    }
+    const float r = 1.0f / sqrtf(block_sum_256(ss, red) / (float)dg + eps);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int c = (threadIdx.x + 256 * u) * V;
+      if (c < dg) {
+        float wv[V];
+        load_piece<float, V>(w + c0 + c, wv);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[u][i] *= r * wv[i];
+        store_piece<T, V>(orow + c, v[u]);
+      }
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < dg; c += 256) { const float z = to_f(zr[c]), v = yr[c] * (z / (1.0f + expf(-z))); ss += v * v; }
+  const float r = 1.0f / sqrtf(block_sum_256(ss, red) / (float)dg + eps);
+  for (int c = threadIdx.x; c < dg; c += 256) {
+    const float z = to_f(zr[c]);
+    orow[c] = from_f<T>(yr[c] * (z / (1.0f + expf(-z))) * r * w[c0 + c]);
+  }
+}
+
+extern "C" int ragged_gate_group_norm(const float* y, const void* P, int64_t ldp, int z0, const float* w, void* out, int64_t rows, int n,
+                                      int groups, float eps, int dtype, hipStream_t st) {
+  if (rows <= 0 || n <= 0 || groups <= 0 || n % groups || rows * groups > 0x7fffffff || z0 < 0 || ldp < z0 + n || !y || !P || !w || !out) return -1;
+  const int dg = n / groups;
+  RAGGED_DISPATCH(dtype,
+    const size_t b = 4 * sizeof(T);
+    const bool vec = dg % 4 == 0 && ldp % 4 == 0 && z0 % 4 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)w % 16 == 0 && (uintptr_t)P % b == 0 &&
+                     (uintptr_t)out % b == 0;
+    const dim3 grid((unsigned)(rows * groups));
+#define GN_CASE(NU, V) hipLaunchKernelGGL((gate_group_norm_kernel<T, NU, V>), grid, dim3(256), 0, st, y, (const T*)P, ldp, z0, w, (T*)out, n, groups, eps)
+    if (vec && dg <= 1024) GN_CASE(1, 4);
+    else if (vec && dg <= 4096) GN_CASE(4, 4);
+    else if (dg <= 1024) GN_CASE(4, 1);
+    else GN_CASE(0, 1))
+#undef GN_CASE
+  return RAGGED_LAUNCH_OK();
+}
+
+// ---------------------------------------------------------------------------------------------------------------
 // Activations of a feed-forward's inner channels.  act_cols: out[r, c] = act(P[r, col0 + c]), c < n, with
 // kind 0: gelu through erf, 0.5 z (1 + erf(z / sqrt 2));  1: gelu through tanh, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
 // 2: relu(z)^2;  3: a unit with two curvatures (p0, p1 >= 0 are handed in): p0 z^2 + z / 2 right of zero,
 // (1/2 + p1) (e^z - 1 - z) + z / 2 left of it (both branches and their slopes meet at 0);  4: tanh(z).
-// glu_pairs: the inner channels come as neighbouring (gate, up) pairs, out[r, c] = silu(P[r, 2 c]) * P[r, 2 c + 1].
+// glu_pairs: the inner channels come as neighbouring (gate, up) pairs, out[r, c] = silu(P[r, 2 c]) * P[r, 2 c + 1] (* row_gate[r]).
 __device__ __forceinline__ float act_value(float z, int kind, float p0, float p1) {
   if (kind == 3) return z > 0.f ? p0 * z * z + 0.5f * z : (0.5f + p1) * (expm1f(z) - z) + 0.5f * z;
   if (kind == 4) return tanhf(z);
@@ -656,13 +900,14 @@ __global__ __launch_bounds__(256) void act_cols_kernel(const T* __restrict__ P, 
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void glu_pairs_kernel(const T* __restrict__ P, int64_t ldp, T* __restrict__ out, int64_t rows, int n) {
+__global__ __launch_bounds__(256) void glu_pairs_kernel(const T* __restrict__ P, int64_t ldp, const float* __restrict__ row_gate,
+                                                        T* __restrict__ out, int64_t rows, int n) {
   const int64_t total = rows * n;
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < total; i += (int64_t)gridDim.x * 256) {
     const int64_t r = i / n;
     const int c = (int)(i % n);
     const float g = to_f(P[r * ldp + 2 * c]), u = to_f(P[r * ldp + 2 * c + 1]);
-    out[i] = from_f<T>(g / (1.0f + expf(-g)) * u);
+    out[i] = from_f<T>(g / (1.0f + expf(-g)) * u * (row_gate ? row_gate[r] : 1.0f));
   }
 }
 
@@ -684,11 +929,12 @@ extern "C" int ragged_act_cols(const void* P, int64_t ldp, int col0, void* out, 
   return RAGGED_LAUNCH_OK();
 }
 
-extern "C" int ragged_glu_pairs(const void* P, int64_t ldp, void* out, int64_t rows, int n, int dtype, hipStream_t st) {
+extern "C" int ragged_glu_pairs(const void* P, int64_t ldp, const float* row_gate, void* out, int64_t rows, int n, int dtype, hipStream_t st) {
   if (rows <= 0 || n <= 0 || ldp < 2 * n) return -1;
   const int64_t blocks = (rows * n + 255) / 256;
   const unsigned grid = (unsigned)(blocks < 16384 ? blocks : 16384);
-  RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((glu_pairs_kernel<T>), dim3(grid), dim3(256), 0, st, (const T*)P, ldp, (T*)out, rows, n))
+  RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((glu_pairs_kernel<T>), dim3(grid), dim3(256), 0, st, (const T*)P, ldp, row_gate, (T*)out, rows,
+                                            n))
   return RAGGED_LAUNCH_OK();
 }
 
@@ -1048,17 +1294,19 @@ extern "C" int ragged_ln_add(float* x, const void* y, const float* w, const floa
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// Queries, keys and values of attention layers whose query / key norm covers the whole projection: one pass over a row's
-// [q | k | v] columns.  q and k: divided by the root mean square of all H d (G d) channels, times a weight per channel, then
-// the first `rot` channels of every head turned in pairs (i, i + rot / 2); q to a float buffer, k to its page.  v: with
+// Queries, keys and values of attention layers without a convolution: one pass over a row's
+// [q | k | v] columns.  q and k: divided by the root mean square of all H d (G d) channels, times a weight per channel
+// (`head_norms`: every head by its own, times a weight of d channels that all heads share), then
+// the first `rot` channels of every head turned in pairs (i, i + rot / 2); q to a float buffer (times 1 + temp_coef
+// ln(floor((pos + 1) / temp_every) + 1) with `temp_every`), k to its page.  v: with
 // `v_norm` every head divided by its root mean square; with `first_in` v <- (1 - lam) v + lam first (float values that an
 // earlier layer left in `first_out` [T, G vd] for the same rows); to its page.  One workgroup per token row.
 struct QkvRowsArgs {
   const void* P;         // [T, ldp], columns 0 .. : q [H d] | k [G d] | v [G vd]
   int64_t ldp;
   int H, G, d, vd;
-  const float* qw;       // [H d]
-  const float* kw;       // [G d]
+  const float* qw;       // [H d], or [d] with head_norms
+  const float* kw;       // [G d], or [d] with head_norms
   float eps;
   int rot;
   const float* cossin;   // [T, rot / 2, 2]
@@ -1069,6 +1317,9 @@ struct QkvRowsArgs {
   const float* first_in;
   float* first_out;
   float lam;
+  int head_norms;
+  int temp_every;        // 0: no temperature
+  float temp_coef;
 };
 
 template <typename T, bool VEC>
@@ -1098,6 +1349,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRowsArgs a, Batch bt) 
       if (c < nq) sq += v * v; else sk += v * v;
     }
   }
+  const float temp = a.temp_every > 0 ? 1.0f + a.temp_coef * logf((float)((pos + 1) / a.temp_every + 1)) : 1.0f;
   const float rq = 1.0f / sqrtf(block_sum_256(sq, red) / (float)nq + a.eps);
   const float rk = 1.0f / sqrtf(block_sum_256(sk, red + 4) / (float)nk + a.eps);      // (its barrier also covers srow)
   const int half = a.rot >> 1;
@@ -1106,8 +1358,14 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRowsArgs a, Batch bt) 
     const bool isq = hd < a.H;
     const int g = hd - a.H;
     const float* u = srow + hd * a.d;
-    const float* w = isq ? a.qw + hd * a.d : a.kw + g * a.d;
-    const float r = isq ? rq : rk;
+    const float* w = a.head_norms ? (isq ? a.qw : a.kw) : isq ? a.qw + hd * a.d : a.kw + g * a.d;
+    float r = isq ? rq : rk;
+    if (a.head_norms) {
+      float s = 0.f;
+      for (int c = lane; c < a.d; c += 64) s += u[c] * u[c];
+      r = 1.0f / sqrtf(wave_sum(s) / (float)a.d + a.eps);
+    }
+    if (isq) r *= temp;
     float* qo = a.q_out + (int64_t)t * nq + hd * a.d;
     T* ko = (T*)a.kpages + ((page * a.G + g) * PAGE + pos % PAGE) * a.d;
     for (int c = lane; c < a.d; c += 64) {
@@ -1144,7 +1402,7 @@ __global__ __launch_bounds__(256) void qkv_rows_kernel(QkvRowsArgs a, Batch bt) 
 
 extern "C" int ragged_qkv_rows(QkvRowsArgs a, Batch bt, int dtype, hipStream_t st) {
   if (bt.T <= 0 || a.H <= 0 || a.G <= 0 || a.H % a.G || a.d <= 0 || a.vd <= 0 || a.rot < 0 || (a.rot & 1) || a.rot > a.d) return -1;
-  if (!a.qw || !a.kw || !a.q_out || !a.kpages || !a.vpages || (a.rot && !a.cossin)) return -1;
+  if (!a.qw || !a.kw || !a.q_out || !a.kpages || !a.vpages || (a.rot && !a.cossin) || a.temp_every < 0) return -1;
   const int64_t n = (int64_t)(a.H + a.G) * a.d;
   if (n * (int64_t)sizeof(float) > 60 * 1024 || a.ldp < n + (int64_t)a.G * a.vd) return -1;
   const size_t sm = (size_t)n * sizeof(float);

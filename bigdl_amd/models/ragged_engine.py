@@ -9,10 +9,11 @@ into arbitrary portions next to single decoded tokens run here instead:
   product runs once over all rows; the mixers read ``BatchMeta`` (row -> sequence, position, pages);
 * keys / values live in 64-token pages of a ``PagedStatePool``, per-sequence state in its slots;
 * the mixers are described by small dataclasses whose fields are the design's constants, so a new design is a new list
-  of them (``models/lipizen.py``, ``models/merusun.py``, ``models/filanex.py``, ``models/dimelix.py`` and
-  ``models/supisun.py`` build one from a ``config.json``);
+  of them (``models/lipizen.py``, ``models/merusun.py``, ``models/filanex.py``, ``models/dimelix.py``, ``models/supisun.py`` and
+  ``models/lifenex.py`` build one from a ``config.json``);
 * five residual forms: the post-sum norm x <- norm(alpha x + f(x)), the sandwich x <- x + norm_b(f(norm_a(x))), the
-  parallel pre-norm block u = norm(x), x <- x + mixer(u) + ff(u), and the sequential pre-norm block x <- x + f(norm(x))
+  parallel pre-norm block u = norm(x), x <- x + mixer(u) + ff(u) (or with a norm of its own for each of the two), and the
+  sequential pre-norm block x <- x + f(norm(x))
   per sublayer, whose stream may be kept in several copies that every sublayer reads and rewrites with learned weights,
   and the output-norm block x <- x + LN(f(x)), whose mixers may read the stream behind a short causal convolution;
 * a run of layers may be executed several times with the same weights (every execution has its own cache), with the
@@ -73,6 +74,10 @@ class WindowAttention:
     v_norm: bool = False           # values RMS-normed per head, without a weight
     v_mix: bool = False            # values of the stack's first such layer are mixed in: v <- (1 - lam) v + lam v_first of the same
                                    # token (``LayerTensors.v_lam``; needs equal value sizes); what is cached is the mixture
+    one_pass: bool = False         # ``qk_norm`` per head (plain projections, one map): queries, keys and values of a row in one kernel
+    q_temp: Optional[tuple] = None  # (coef, every): the query of position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)
+    dist_far: int = 0              # > 0: a learned bias by distance, ``LayerTensors.dist_bias`` [heads, dist_far + 1], joins the scaled
+                                   # score of query i and key j at min(i - j, dist_far)
 
 
 @dataclass
@@ -115,13 +120,17 @@ class GatedDelta:
     behind a short causal convolution over time and silu, q and k then unit vectors u / sqrt(|u|^2 + unit_eps), q times dim^-1/2.
     Per head a decay g = exp(-e^A_log softplus(W_a h + dt_bias)) and a write strength beta = sigmoid(W_b h):
     S <- g S, u = beta (v - S^T k), S <- S + k u^T, o = S^T q.  Each head's output is divided by its root mean square, weighted
-    (one weight of ``vdim`` channels for all heads) and multiplied by silu of a projection of the mixer's input."""
+    (one weight of ``vdim`` channels for all heads) and multiplied by silu of a projection of the mixer's input.
+    ``decay_rank`` > 0: one decay per head and key channel (S <- diag(g) S), its logits W_a2 (W_a1 h) through a pair of products of
+    that rank; ``gate_rank`` > 0: the output gate comes through such a pair too and is a sigmoid."""
     heads: int
     kv_heads: int
     dim: int
     vdim: int
     conv_taps: int
     unit_eps: float = 1e-6
+    decay_rank: int = 0
+    gate_rank: int = 0
 
     @property
     def conv_channels(self) -> int:
@@ -140,12 +149,38 @@ class SelectiveScan:
 
 
 @dataclass
+class StateSpace:
+    """Mamba-2: [z | x | B | C | step logits] = W_in h with x of ``heads`` x ``vdim`` channels, B and C of ``groups`` x ``state``, one step
+    logit per head; x, B and C behind a short causal convolution with bias and silu, d = softplus(logits + dt_bias); per head (head h
+    uses group h / (heads / groups)) S <- exp(-e^A_log d) S + d B x^T, y = S^T C + D x.  y silu(z) is RMS-normed in ``norm_groups``
+    equal parts of all channels, weighted, and projected."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    norm_groups: int
+    conv_taps: int
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def conv_channels(self) -> int:
+        return self.inner + 2 * self.groups * self.state
+
+
+@dataclass
 class SideBySide:
     """Two mixers that read the same input; their outputs are summed, each with its own weight (carried by the mixers'
     ``out_scale``, so that one output projection [W_left | W_right] serves both).  The two must keep different kinds of
-    state (pages against a matrix), since an execution has one cache of each kind."""
+    state (pages against a matrix), since an execution has one cache of each kind.
+    ``out_norms``: each has an output projection of its own whose result is RMS-normed over the width with a weight
+    (``LayerTensors.out_norm``) before the two are summed and multiplied by ``mix`` (parallel block with two norms)."""
     left: object
     right: object
+    out_norms: bool = False
+    mix: float = 1.0
 
 
 @dataclass
@@ -185,7 +220,9 @@ class RoutedExperts:
     over all experts' router logits or a sigmoid per expert (32-bit); experts come in ``groups`` equal runs of neighbours,
     a group scores as the sum of its ``group_top`` best experts, and the ``top`` best experts inside the ``keep`` best
     groups are used, weighted by score * ``scale``, the scores first divided by their sum (+ 1e-20) with ``renorm``.
-    ``shared_ff`` > 0: one more expert of that inner size that every token uses with weight 1."""
+    ``correction``: a number per expert is added to the scores for the choice of groups and experts (which may turn them negative),
+    not to the weights.  ``shared_ff`` > 0: one more expert of that inner size that every token uses with weight 1, or with
+    ``shared_gate`` with the sigmoid of a router row of its own."""
     experts: int
     top: int
     ff: int
@@ -197,6 +234,8 @@ class RoutedExperts:
     group_top: int = 1
     renorm: bool = False
     act: str = "relu2"             # or "swiglu"
+    correction: bool = False
+    shared_gate: bool = False
 
 
 @dataclass
@@ -249,6 +288,9 @@ class RaggedConfig:
     mix_in: tuple = ()             # executions in front of which x <- W_mix [x ; embedding output]
     pair_embed: Optional[PairEmbedding] = None
     positions: int = 0             # > 0: a learned vector per position is added to the embedding; no sequence grows beyond this
+    two_norms: bool = False        # "parallel": the feed-forward reads a norm of its own, x <- x + mixer(norm1(x)) + ff(norm2(x))
+    embed_norm: bool = False       # the embedding output is RMS-normed with a weight before the first layer
+    logit_scale: float = 1.0
     stream_conv: int = 0           # "output_norm": a mixer reads x + conv(x), a causal convolution of this many taps per channel of
                                    # the stream (``LayerTensors.stream_conv``; 0: it reads x)
 
@@ -296,13 +338,19 @@ class LayerTensors:
     norm2_bias: Optional[torch.Tensor] = None
     stream_conv: Optional[torch.Tensor] = None  # float [width, taps]
     v_lam: float = 0.0                       # share of the first mixing layer's values
-    decay_rate: Optional[torch.Tensor] = None  # gated delta rule: e^A_log float [heads]; its step bias is decay_bias
+    decay_rate: Optional[torch.Tensor] = None  # gated delta rule, state space: e^A_log float [heads]; the delta rule's step bias is
+                                             # decay_bias, its pair's second product (``decay_rank``) w_decay [heads dim, rank]
+    w_gate: Optional[torch.Tensor] = None    # gated delta rule with ``gate_rank``: second product of the gate's pair [heads vdim, rank]
+    dist_bias: Optional[torch.Tensor] = None  # float [heads, dist_far + 1]: score bias by distance
+    out_norm: Optional[torch.Tensor] = None  # side-by-side mixers with ``out_norms``: float [width]
+    correction: Optional[torch.Tensor] = None  # float [experts]
+    w_sgate: Optional[torch.Tensor] = None   # shared expert's gate row, float [width]
     conv_b: Optional[torch.Tensor] = None    # selective scan: bias of the convolution, float [inner]
     w_low: Optional[torch.Tensor] = None     # [dt_rank + 2 state, inner]
     w_dt: Optional[torch.Tensor] = None      # [inner, dt_rank]
-    dt_bias: Optional[torch.Tensor] = None   # float [inner]
+    dt_bias: Optional[torch.Tensor] = None   # float [inner] (state space: [heads])
     ssm_a: Optional[torch.Tensor] = None     # float [inner, state]: -e^A_log log2(e)
-    ssm_d: Optional[torch.Tensor] = None     # float [inner]
+    ssm_d: Optional[torch.Tensor] = None     # float [inner] (state space: [heads])
     left: Optional["LayerTensors"] = None    # side-by-side mixers: what each of the two needs beyond the shared projections
     right: Optional["LayerTensors"] = None
 
@@ -337,12 +385,14 @@ class RaggedDecoder:
     def __init__(self, cfg: RaggedConfig, embed: torch.Tensor, layers: List[LayerTensors], final_norm: torch.Tensor,
                  head: torch.Tensor, act_dtype=torch.bfloat16, device="cuda", pair_table: Optional[torch.Tensor] = None,
                  w_mix: Optional[torch.Tensor] = None, pos_table: Optional[torch.Tensor] = None,
-                 final_norm_bias: Optional[torch.Tensor] = None):
+                 final_norm_bias: Optional[torch.Tensor] = None, embed_norm: Optional[torch.Tensor] = None):
         """``pair_table`` [buckets + 1, width]: the token-pair embedding of ``cfg.pair_embed``; ``w_mix`` [width, 2 width]:
         the projection of [stream ; embedding output] in front of the executions named in ``cfg.mix_in``; ``pos_table``
-        [positions, width]: learned positions; ``final_norm_bias``: the bias of an "output_norm" model's last norm."""
+        [positions, width]: learned positions; ``final_norm_bias``: the bias of an "output_norm" model's last norm; ``embed_norm`` float [width]: the weight of
+        ``cfg.embed_norm``."""
         self.cfg, self.embed, self.layers, self.final_norm, self.head = cfg, embed, layers, final_norm, head
         self.pair_table, self.w_mix, self.pos_table, self.final_norm_bias = pair_table, w_mix, pos_table, final_norm_bias
+        self.embed_norm = embed_norm
         self.max_positions = cfg.positions or None
         self.act = act_dtype
         self.device = torch.device(device)
@@ -365,6 +415,12 @@ class RaggedDecoder:
                 raise ValueError("every layer needs its [width, taps] convolution of the stream")
         elif cfg.stream_conv:
             raise ValueError("only the output-norm block convolves the stream")
+        if cfg.embed_norm and (embed_norm is None or embed_norm.numel() != cfg.width):
+            raise ValueError("the norm of the embedding output needs a weight of the stream's width")
+        if cfg.two_norms and (cfg.block != "parallel" or cfg.mix_in or any(lt.norm2 is None for lt, mlp in zip(layers, cfg.mlps) if mlp is not None)):
+            raise ValueError("two norms belong to the parallel block (without mixing the embedding output back in), one weight each")
+        if any(isinstance(m, SideBySide) and m.out_norms for m in cfg.mixers) and not cfg.two_norms:
+            raise ValueError("mixers side by side with norms of their own outputs come in the parallel block with two norms")
         self._check_value_mixing()
         self._kv_run = {}                  # execution -> the execution whose cache it reads (itself unless kv_from is set)
         latest = {}
@@ -403,11 +459,18 @@ class RaggedDecoder:
         self._v_first = None               # the first execution whose values the later mixing layers share
         for ri, li in enumerate(self.runs):
             m = self.cfg.mixers[li]
+            m = m.left if isinstance(m, SideBySide) else m
             if not isinstance(m, WindowAttention):
                 continue
             if m.qk_norm_rows:
                 if m.maps != 1 or m.conv_taps or m.gate or m.kv_from is not None or m.v_from_k or m.rot_neighbours or m.rot_amp != 1.0:
                     raise ValueError(f"layer {li}: the norm over whole projections serves plain q / k / v projections of one map")
+            elif m.one_pass:
+                if not m.qk_norm or m.maps != 1 or m.conv_taps or m.gate or m.kv_from is not None or m.v_from_k or m.rot_neighbours \
+                        or m.rot_amp != 1.0 or m.v_norm or m.v_mix:
+                    raise ValueError(f"layer {li}: one pass over a row's projections serves plain q / k / v projections of one map, normed per head")
+            elif m.q_temp is not None:
+                raise ValueError(f"layer {li}: the query temperature comes with the pass over a row's projections")
             elif m.v_norm or m.v_mix:
                 raise ValueError(f"layer {li}: normed or mixed values come with the norm over whole projections")
             if m.v_mix:
@@ -454,6 +517,10 @@ class RaggedDecoder:
             s.append(("matrix", m.heads, m.dim, m.vdim))
             if m.conv_taps > 1:
                 s.append(("tail", m.conv_taps - 1, m.conv_channels))
+        elif isinstance(m, StateSpace):
+            s.append(("matrix", m.heads, m.state, m.vdim))
+            if m.conv_taps > 1:
+                s.append(("tail", m.conv_taps - 1, m.conv_channels))
         elif isinstance(m, SelectiveScan):
             s.append(("matrix", 1, m.inner, m.state))
             if m.conv_taps > 1:
@@ -478,7 +545,7 @@ class RaggedDecoder:
     def _attention(self, li, m: WindowAttention, lt: LayerTensors, P, meta):
         """``li`` (here and in the other mixers): the execution's index, which names its cache / state in the pool"""
         ops, pool, eps = self.ops, self.pool, self.cfg.norm_eps
-        if m.qk_norm_rows:
+        if m.qk_norm_rows or m.one_pass:
             return self._attention_rows(li, m, lt, P, meta)
         turn = dict(interleaved=m.rot_neighbours, rot_amp=m.rot_amp)
         cq = m.heads * m.maps * m.dim
@@ -504,31 +571,48 @@ class RaggedDecoder:
                               window=m.window, keep_first=m.keep_first, scale=m.scale, lam=m.lam, out_scale=m.out_scale,
                               out_norm=m.out_norm, eps=eps, gate=P if m.gate else None, gate0=col, sink=m.sink,
                               chunk=m.chunk, softcap=m.softcap, gate_wide=m.gate and m.gate_channels,
-                              sinks=lt.sinks if m.head_sinks else None, slopes=lt.slopes if m.dist_slopes is not None else None)
+                              sinks=lt.sinks if m.head_sinks else None, slopes=lt.slopes if m.dist_slopes is not None else None,
+                              dist_bias=lt.dist_bias if m.dist_far else None)
 
     def _attention_rows(self, li, m: WindowAttention, lt: LayerTensors, P, meta):
-        """queries, keys and values of a row in one pass: norms over whole projections, rotation, value norm and mixing"""
+        """queries, keys and values of a row in one pass: norms (over whole projections or per head), rotation, query temperature,
+        value norm and mixing"""
         ops, pool, eps = self.ops, self.pool, self.cfg.norm_eps
         first = li == self._v_first
         mix = m.v_mix and not first
         q, v = ops.qkv_rows(P, lt.q_norm, lt.k_norm, eps, m.rot_dims, lt.inv_freq, pool.k[li], pool.v[li], meta, H=m.heads,
                             G=m.kv_heads, d=m.dim, vd=m.vdim, v_norm=m.v_norm, first_in=meta.shared["values"] if mix else None,
-                            lam=lt.v_lam, want_first=first)
+                            lam=lt.v_lam, want_first=first, head_norms=not m.qk_norm_rows, q_temp=m.q_temp)
         if first:
             meta.shared["values"] = v
         return ops.paged_attn(q, pool.k[li], pool.v[li], meta, maps=1, H=m.heads, G=m.kv_heads, d=m.dim, vd=m.vdim, window=m.window,
                               keep_first=m.keep_first, scale=m.scale, lam=0.0, out_scale=m.out_scale, out_norm=m.out_norm, eps=eps,
                               sink=m.sink, chunk=m.chunk, softcap=m.softcap, sinks=lt.sinks if m.head_sinks else None,
-                              slopes=lt.slopes if m.dist_slopes is not None else None)
+                              slopes=lt.slopes if m.dist_slopes is not None else None, dist_bias=lt.dist_bias if m.dist_far else None)
 
     def _gated_delta(self, li, m: GatedDelta, lt: LayerTensors, P, meta):
         ops, pool = self.ops, self.pool
         C, hv = m.conv_channels, m.heads * m.vdim
-        # columns of P: q | k | v | output gate | write strengths | step logits
-        qf, kf, v, gb = ops.gated_delta_prep(P, lt.conv_w, m.conv_taps, pool.tail.get(li), C + hv, C + hv + m.heads, lt.decay_rate,
-                                             lt.decay_bias, m.unit_eps, m.heads, m.kv_heads, m.dim, m.vdim, meta)
-        o = ops.gated_delta_scan(qf, kf, gb, m.kv_heads, v, pool.matrix[li], m.heads, m.dim, m.vdim, meta)
-        return ops.head_norm_gate(o, lt.o_norm, P, C, m.heads, m.vdim, self.cfg.norm_eps, self.act, gate="silu")
+        # columns of P: q | k | v | low-rank input of the decays (if any) | output gate or its low-rank input | write strengths | step
+        # logits (unless the decays have a rank)
+        g0 = C + m.decay_rank
+        b0 = g0 + (m.gate_rank or hv)
+        a0 = b0 + m.heads
+        wl = self._linear_f32(P[:, C:g0], lt.w_decay) if m.decay_rank else None
+        qf, kf, v, gb, *wf = ops.gated_delta_prep(P, lt.conv_w, m.conv_taps, pool.tail.get(li), b0, a0, lt.decay_rate, lt.decay_bias,
+                                                  m.unit_eps, m.heads, m.kv_heads, m.dim, m.vdim, meta, wl=wl)
+        o = ops.gated_delta_scan(qf, kf, gb, m.kv_heads, v, pool.matrix[li], m.heads, m.dim, m.vdim, meta, wf=wf[0] if wf else None)
+        if not m.gate_rank:
+            return ops.head_norm_gate(o, lt.o_norm, P, g0, m.heads, m.vdim, self.cfg.norm_eps, self.act, gate="silu")
+        return ops.head_norm_gate(o, lt.o_norm, F.linear(P[:, g0:g0 + m.gate_rank], lt.w_gate), 0, m.heads, m.vdim, self.cfg.norm_eps, self.act)
+
+    def _state_space(self, li, m: StateSpace, lt: LayerTensors, P, meta):
+        ops, pool, C, GN = self.ops, self.pool, m.inner, m.groups * m.state
+        # columns of P: z | x | B | C | step logits
+        X = ops.conv_rows(P, C, lt.conv_w, lt.conv_b, pool.tail.get(li), meta, self.act, silu=True)
+        y = ops.state_space_scan(X, C, C + GN, P, 2 * C + 2 * GN, lt.dt_bias, lt.decay_rate, lt.ssm_d, pool.matrix[li], m.heads, m.groups,
+                                 m.state, m.vdim, meta)
+        return ops.gate_group_norm(y, P, 0, lt.o_norm, m.norm_groups, self.cfg.norm_eps, self.act)
 
     def _selective(self, li, m: SelectiveScan, lt: LayerTensors, P, meta):
         ops, pool = self.ops, self.pool
@@ -581,7 +665,8 @@ class RaggedDecoder:
 
     def _side_by_side(self, li, m: SideBySide, lt: LayerTensors, P, meta):
         nl = lt.left.w_in.shape[0]                   # the left mixer's rows of the stacked projection
-        return torch.cat([self._mixer(li, m.left, lt.left, P[:, :nl], meta), self._mixer(li, m.right, lt.right, P[:, nl:], meta)], 1)
+        a, b = self._mixer(li, m.left, lt.left, P[:, :nl], meta), self._mixer(li, m.right, lt.right, P[:, nl:], meta)
+        return (F.linear(a, lt.left.w_out), F.linear(b, lt.right.w_out)) if m.out_norms else torch.cat([a, b], 1)
 
     def _mlstm(self, li, m: Mlstm, lt: LayerTensors, P, meta):
         ops, pool = self.ops, self.pool
@@ -601,11 +686,12 @@ class RaggedDecoder:
     def _experts(self, f: RoutedExperts, lt: LayerTensors, xa, meta):
         ops = self.ops
         gated = f.act == "swiglu"
-        idx, wts = ops.moe_route(xa, lt.w_router, f.groups, f.keep, f.top, f.scale, f.score, f.group_top, f.renorm)
+        idx, wts, *row_gate = ops.moe_route(xa, lt.w_router, f.groups, f.keep, f.top, f.scale, f.score, f.group_top, f.renorm,
+                                            correction=lt.correction if f.correction else None, w_gate=lt.w_sgate if f.shared_gate else None)
         base = None
         if f.shared_ff:
             a = F.linear(xa, lt.w_sup)
-            base = F.linear(ops.glu_pairs(a) if gated else ops.relu2(a), lt.w_sdn)
+            base = F.linear(ops.glu_pairs(a, *row_gate) if gated else ops.relu2(a), lt.w_sdn)
         if meta.T * f.top < self.moe_dense_rows * f.experts:
             return ops.moe_rows(xa, idx, wts, lt.w_up, lt.w_dn, base, gated)
         y = ops.moe_sorted(xa, idx, wts, lt.w_up, lt.w_dn, base, gated)         # bfloat16: one grouped product per projection
@@ -729,6 +815,8 @@ class RaggedDecoder:
             return self._gated_delta(li, m, lt, P, meta)
         if isinstance(m, SelectiveScan):
             return self._selective(li, m, lt, P, meta)
+        if isinstance(m, StateSpace):
+            return self._state_space(li, m, lt, P, meta)
         return self._hgrn2(li, m, lt, P, meta)
 
     def _forward(self, meta, idt, rows, collect):
@@ -738,9 +826,11 @@ class RaggedDecoder:
         elif cfg.positions:
             x = ops.embed_rows(idt[0], self.embed, idt[1], self.pos_table, cfg.embed_scale)
         else:
-            x = ops.embed_rows(idt, self.embed, scale=cfg.embed_scale)
+            x = ops.embed_rows(idt, self.embed, scale=cfg.embed_scale, norm=self.embed_norm if cfg.embed_norm else None, eps=cfg.norm_eps)
         if cfg.block == "sandwich":
             self._sandwich_layers(x, meta, collect)
+        elif cfg.block == "parallel" and cfg.two_norms:
+            self._two_norm_layers(x, meta, collect)
         elif cfg.block == "parallel":
             x = self._parallel_layers(x, meta, collect)
         elif cfg.block == "pre_norm":
@@ -774,7 +864,7 @@ class RaggedDecoder:
         logits = F.linear(xa, self.head).float()
         if cfg.logit_softcap > 0:
             logits = torch.tanh(logits / cfg.logit_softcap) * cfg.logit_softcap
-        return logits
+        return logits if cfg.logit_scale == 1.0 else logits.mul_(cfg.logit_scale)
 
     def _sandwich_layers(self, x, meta, collect):
         """x <- x + norm_b(f(norm_a(x))) for the mixer and the feed-forward of every layer; x float32, in place.  The norm
@@ -824,6 +914,38 @@ class RaggedDecoder:
             if collect is not None:
                 collect.append(x.clone())
         return x
+
+    def _two_norm_layers(self, x, meta, collect):
+        """x <- x + mixer(norm1(x)) + ff(norm2(x)); x float32, in place.  The stream's root mean square serves both norms, so one kernel
+        sums the sublayers' outputs (those of two mixers side by side normed first) into it and writes the two operands that the next
+        execution reads."""
+        cfg, ops, eps = self.cfg, self.ops, self.cfg.norm_eps
+        n = len(self.runs)
+
+        def norms(ri):                               # weights of execution ri's two norms (None: nothing reads it)
+            if ri >= n:
+                return None, None
+            return self.layers[self.runs[ri]].norm1, self.layers[self.runs[ri]].norm2 if cfg.mlps[self.runs[ri]] is not None else None
+
+        u1, u2 = ops.join_norms(x, None, None, None, *norms(0), eps, self.act)
+        for ri, li in enumerate(self.runs):
+            m, mlp, lt = cfg.mixers[li], cfg.mlps[li], self.layers[li]
+            y, side = self._mixer(ri, m, lt, F.linear(u1, lt.w_in, lt.b_in), meta), None
+            if isinstance(m, SideBySide) and m.out_norms:
+                side, y = (*y, lt.left.out_norm, lt.right.out_norm, m.mix), None
+            else:
+                y = F.linear(y, lt.w_out)
+            if isinstance(mlp, DenseMlp):
+                y2 = F.linear(ops.act_cols(F.linear(u2, lt.w_ff), 0, mlp.ff, mlp.act, lt.act_params or (0.0, 0.0)), lt.w_down, lt.b_down)
+            elif isinstance(mlp, RoutedExperts):
+                y2 = self._experts(mlp, lt, u2, meta)
+            elif mlp is None:
+                y2 = None
+            else:
+                raise ValueError("the parallel block has no such feed-forward")
+            u1, u2 = ops.join_norms(x, y, y2, side, *norms(ri + 1), eps, self.act)
+            if collect is not None:
+                collect.append(x.clone())
 
     def _prenorm_layers(self, x, meta, collect):
         """x <- x + f(norm(x)) for the mixer and then the feed-forward of every execution, on a stream of ``cfg.streams``
@@ -918,5 +1040,6 @@ class RaggedDecoder:
     def weight_bytes(self):
         ts = [self.embed, self.head, self.final_norm] + [t for t in (self.pair_table, self.w_mix, self.pos_table) if t is not None]
         for lt in self.layers:
-            ts += [t for t in vars(lt).values() if isinstance(t, torch.Tensor)]
+            for part in (lt, lt.left, lt.right):     # (a side-by-side layer's input projections are those of the layer)
+                ts += [t for n, t in vars(part).items() if isinstance(t, torch.Tensor) and (part is lt or n != "w_in")] if part is not None else []
         return sum(t.numel() * t.element_size() for t in ts)

@@ -93,20 +93,31 @@ class _AttnArgs(ctypes.Structure):
                 ("rows", ctypes.c_void_p), ("n_rows", ctypes.c_int), ("tiles", ctypes.c_void_p), ("n_tiles", ctypes.c_int),
                 ("ldv", ctypes.c_int64), ("sink", ctypes.c_int), ("sink_score", ctypes.c_float), ("chunk", ctypes.c_int),
                 ("softcap", ctypes.c_float), ("gate_wide", ctypes.c_int), ("sinks", ctypes.c_void_p),
-                ("slopes", ctypes.c_void_p)]
+                ("slopes", ctypes.c_void_p), ("dist_bias", ctypes.c_void_p), ("n_bias", ctypes.c_int)]
 
 
 class _QkvRowsArgs(ctypes.Structure):
     _fields_ = [("P", ctypes.c_void_p), ("ldp", ctypes.c_int64)] + [(n, ctypes.c_int) for n in ("H", "G", "d", "vd")] + \
                [("qw", ctypes.c_void_p), ("kw", ctypes.c_void_p), ("eps", ctypes.c_float), ("rot", ctypes.c_int),
                 ("cossin", ctypes.c_void_p), ("q_out", ctypes.c_void_p), ("kpages", ctypes.c_void_p), ("vpages", ctypes.c_void_p),
-                ("v_norm", ctypes.c_int), ("first_in", ctypes.c_void_p), ("first_out", ctypes.c_void_p), ("lam", ctypes.c_float)]
+                ("v_norm", ctypes.c_int), ("first_in", ctypes.c_void_p), ("first_out", ctypes.c_void_p), ("lam", ctypes.c_float),
+                ("head_norms", ctypes.c_int), ("temp_every", ctypes.c_int), ("temp_coef", ctypes.c_float)]
 
 
 class _GatedDeltaArgs(ctypes.Structure):
     _fields_ = [("P", ctypes.c_void_p), ("ldp", ctypes.c_int64), ("cw", ctypes.c_void_p), ("taps", ctypes.c_int), ("state", ctypes.c_void_p),
                 ("b0", ctypes.c_int), ("a0", ctypes.c_int), ("arate", ctypes.c_void_p), ("dt_bias", ctypes.c_void_p), ("tiny", ctypes.c_float)] + \
-               [(n, ctypes.c_void_p) for n in ("qf", "kf", "vo", "gb")] + [(n, ctypes.c_int) for n in ("H", "G", "d", "vd", "write_state")]
+               [(n, ctypes.c_void_p) for n in ("wl", "wf", "qf", "kf", "vo", "gb")] + [(n, ctypes.c_int) for n in ("H", "G", "d", "vd", "write_state")]
+
+
+class _SpaceArgs(ctypes.Structure):
+    _fields_ = [("dt", ctypes.c_void_p), ("lddt", ctypes.c_int64)] + [(n, ctypes.c_void_p) for n in ("dt_bias", "rate", "D")] + \
+               [("b0", ctypes.c_int), ("c0", ctypes.c_int)]
+
+
+class _JoinArgs(ctypes.Structure):
+    _fields_ = [(n, ctypes.c_void_p) for n in ("x", "y", "y2", "ya", "yb", "wa", "wb")] + [("mix", ctypes.c_float)] + \
+               [(n, ctypes.c_void_p) for n in ("w1", "w2", "u1", "u2")] + [("D", ctypes.c_int), ("eps", ctypes.c_float)]
 
 
 class _SelScanArgs(ctypes.Structure):
@@ -133,8 +144,11 @@ def lib():
         L.ragged_mlstm_gates.argtypes = [vp, i64, ci, vp, cf, cf, vp, vp, vp, vp, ci, _Batch, ci, vp]
         L.ragged_mlstm_expand.argtypes = [vp, i64, ci, ci, vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
         L.ragged_head_norm_gate.argtypes = [vp, vp, vp, i64, ci, vp, i64, ci, ci, cf, ci, vp, cf, cf, ci, ci, vp]
-        L.ragged_moe_route.argtypes = [vp, i64, vp, vp, vp, i64, ci, ci, ci, ci, ci, cf, ci, ci, ci, ci, vp]
-        L.ragged_embed_rows.argtypes = [vp, vp, vp, vp, cf, vp, i64, ci, ci, vp]
+        L.ragged_moe_route.argtypes = [vp, i64, vp, vp, vp, i64, ci, ci, ci, ci, ci, cf, ci, ci, ci, vp, vp, vp, ci, vp]
+        L.ragged_embed_rows.argtypes = [vp, vp, vp, vp, cf, vp, cf, vp, i64, ci, ci, vp]
+        L.ragged_join_norms.argtypes = [_JoinArgs, i64, ci, vp]
+        L.ragged_gate_group_norm.argtypes = [vp, vp, i64, ci, vp, vp, i64, ci, ci, cf, ci, vp]
+        L.ragged_state_space_scan.argtypes = [_SpaceArgs, vp, i64, ci, vp, vp, ci, ci, ci, _Batch, ci, vp]
         L.ragged_add_norm.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, ci, vp]
         L.ragged_act_cols.argtypes = [vp, i64, ci, vp, i64, ci, ci, cf, cf, ci, vp]
         L.ragged_hc_step.argtypes = [vp, vp, vp, vp, vp, vp, vp, i64, ci, ci, cf, ci, vp]
@@ -142,7 +156,7 @@ def lib():
         L.ragged_delta_gates.argtypes = [vp, i64, ci, ci, ci, vp, vp, vp, cf, cf, vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
         L.ragged_delta_scan.argtypes = [vp, vp, vp, vp, vp, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
         L.ragged_gated_delta_prep.argtypes = [_GatedDeltaArgs, _Batch, ci, vp]
-        L.ragged_gated_delta_scan.argtypes = [vp, vp, vp, ci, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
+        L.ragged_gated_delta_scan.argtypes = [vp, vp, vp, vp, ci, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
         L.ragged_conv_rows.argtypes = [vp, i64, ci, vp, vp, vp, ci, ci, vp, ci, ci, ci, _Batch, ci, ci, vp]
         L.ragged_ln_add.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, vp, ci, vp, _Batch, ci, vp]
         L.ragged_qkv_rows.argtypes = [_QkvRowsArgs, _Batch, ci, vp]
@@ -150,7 +164,7 @@ def lib():
         L.ragged_selective_chain.argtypes = [vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, vp]
         L.ragged_delta_chain_ok.argtypes = [ci]
         L.ragged_delta_chain.argtypes = [vp, vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, vp]
-        L.ragged_glu_pairs.argtypes = [vp, i64, vp, i64, ci, ci, vp]
+        L.ragged_glu_pairs.argtypes = [vp, i64, vp, vp, i64, ci, ci, vp]
         L.ragged_relu2.argtypes = [vp, vp, i64, ci, vp]
         L.ragged_moe_combine.argtypes = [vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
         L.ragged_moe_grouped_ok.argtypes = [ci, ci, ci]
@@ -471,13 +485,16 @@ class HipOps:
         return out
 
     def paged_attn(self, q, kpages, vpages, meta, *, maps, H, G, d, vd, window, keep_first, scale, lam, out_scale, out_norm,
-                   eps, gate=None, gate0=0, sink=None, chunk=0, softcap=0.0, gate_wide=False, sinks=None, slopes=None):
+                   eps, gate=None, gate0=0, sink=None, chunk=0, softcap=0.0, gate_wide=False, sinks=None, slopes=None, dist_bias=None):
         """``vpages`` may be ``kpages`` itself: the values are then the leading ``vd`` channels of the key rows.
         ``chunk`` > 0: a key is visible only inside the query's block of that many positions; ``softcap`` > 0: scores go
         through softcap * tanh(. / softcap); ``gate_wide``: one gate column per output channel instead of one per head;
         ``sinks`` float [H]: every head's own sink score (instead of the one number ``sink``); ``slopes`` float [H]:
-        slopes[h] * (i - j) is taken off the scaled score of query i and key j."""
-        _f32(q, sinks, slopes)
+        slopes[h] * (i - j) is taken off the scaled score of query i and key j; ``dist_bias`` float [H, n]: dist_bias[h, min(i - j,
+        n - 1)] joins it."""
+        _f32(q, sinks, slopes, dist_bias)
+        if dist_bias is not None and (dist_bias.dim() != 2 or dist_bias.shape[0] != H or dist_bias.shape[1] < 1):
+            raise ValueError("one row of distance biases per query head")
         if any(t is not None and t.numel() != H for t in (sinks, slopes)):
             raise ValueError("one sink score / one slope per query head")
         _act(kpages, vpages, gate)
@@ -507,9 +524,11 @@ class HipOps:
             a.sink, a.sinks = 1, sinks.data_ptr()
         if slopes is not None:
             a.slopes = slopes.data_ptr()
+        if dist_bias is not None:
+            a.dist_bias, a.n_bias = dist_bias.data_ptr(), dist_bias.shape[1]
         if kpages.dtype == torch.bfloat16 and self.mfma and maps == 1 and not lib().ragged_paged_attn_mfma_ok(d, vd) \
                 and lib().ragged_paged_attn_mfma_wide_ok(d, vd) and a.ldv % 8 == 0 and not keep_first and not out_norm \
-                and gate is None and not chunk and not softcap and sinks is None and slopes is None:
+                and gate is None and not chunk and not softcap and sinks is None and slopes is None and dist_bias is None:
             # rows too wide for the row-wise kernel's lanes: long portions as tiles of 64 rows of one head, single tokens
             # and short portions with 16 heads of a row side by side, both on the matrix cores
             tiles, n_tiles, rows, n_rows = meta.attn_split(self.mfma_min_rows)
@@ -521,7 +540,7 @@ class HipOps:
                 _ok(lib().ragged_paged_attn_mfma_heads(a, meta.c(), _stream()), "paged_attn_mfma_heads")
             return out
         if kpages.dtype == torch.bfloat16 and self.mfma and lib().ragged_paged_attn_mfma_ok(d, vd) and a.ldv % 8 == 0 \
-                and not (gate_wide and (a.ldg % 4 or gate0 % 4)):
+                and not (gate_wide and (a.ldg % 4 or gate0 % 4)) and not (maps == 2 and dist_bias is not None):
             # long portions on the matrix cores, single tokens and short portions row by row
             tiles, n_tiles, rows, n_rows = meta.attn_split(self.mfma_min_rows)
             if n_tiles:
@@ -601,21 +620,24 @@ class HipOps:
                                       gf.data_ptr(), T, H, d, _DT[P.dtype], _stream()), "mlstm_expand")
         return qf, ff, gf
 
-    def moe_route(self, xa, w_router, groups, keep, top, scale, score="softmax", group_top=1, renorm=False):
+    def moe_route(self, xa, w_router, groups, keep, top, scale, score="softmax", group_top=1, renorm=False, correction=None, w_gate=None):
         """``score``: "softmax" over all experts or "sigmoid" per expert; a group is worth the sum of its ``group_top``
-        best scores; ``renorm``: the chosen scores are divided by their sum (+ 1e-20) before ``scale``."""
+        best scores; ``renorm``: the chosen scores are divided by their sum (+ 1e-20) before ``scale``; ``correction`` float [E] joins
+        the scores for the choice alone.  Returns (expert indices, weights), with ``w_gate`` float [D] also sigmoid(w_gate . x) [T]."""
         _act(xa)
-        _f32(w_router)
+        _f32(w_router, correction, w_gate)
         T, D = xa.shape
         E = w_router.shape[0]
-        if w_router.shape[1] != D:
+        if w_router.shape[1] != D or (correction is not None and correction.numel() != E) or (w_gate is not None and w_gate.numel() != D):
             raise ValueError("router rows do not fit the stream")
         idx = torch.empty(T, top, dtype=torch.int32, device=xa.device)
         wts = torch.empty(T, top, dtype=torch.float32, device=xa.device)
+        gate = torch.empty(T, dtype=torch.float32, device=xa.device) if w_gate is not None else None
         _ok(lib().ragged_moe_route(xa.data_ptr(), xa.stride(0), w_router.data_ptr(), idx.data_ptr(), wts.data_ptr(), T, D, E, groups,
                                    keep, top, scale, {"softmax": 0, "sigmoid": 1}[score], int(group_top), int(bool(renorm)),
-                                   _DT[xa.dtype], _stream()), "moe_route")
-        return idx, wts
+                                   None if correction is None else correction.data_ptr(), None if gate is None else w_gate.data_ptr(),
+                                   None if gate is None else gate.data_ptr(), _DT[xa.dtype], _stream()), "moe_route")
+        return (idx, wts) if gate is None else (idx, wts, gate)
 
     def moe_sorted(self, xa, idx, wts, w_up, w_dn, base, gated=False):
         """The experts of long bfloat16 portions without a word to the host: (row, choice) pairs sorted by expert, every
@@ -688,9 +710,12 @@ class HipOps:
                                   int(bool(gated)), _DT[xa.dtype], _stream()), "moe_rows")
         return y
 
-    def embed_rows(self, ids, table, ids2=None, table2=None, scale=1.0):
-        """float32 [T, width]: scale * table[ids] (+ table2[ids2]), summed in float."""
+    def embed_rows(self, ids, table, ids2=None, table2=None, scale=1.0, norm=None, eps=0.0):
+        """float32 [T, width]: scale * table[ids] (+ table2[ids2]), summed in float; ``norm`` [width]: RMS-normed with that weight."""
         _act(table, table2)
+        _f32(norm)
+        if norm is not None and norm.numel() != table.shape[1]:
+            raise ValueError("norm weight size")
         T, D = ids.numel(), table.shape[1]
         for i, t in ((ids, table), (ids2, table2)):
             if t is not None and (i is None or i.dtype != torch.int64 or not i.is_contiguous() or i.numel() != T
@@ -698,8 +723,9 @@ class HipOps:
                 raise ValueError("row ids / embedding tables do not fit")
         x = torch.empty(T, D, dtype=torch.float32, device=table.device)
         _ok(lib().ragged_embed_rows(ids.data_ptr(), table.data_ptr(), None if table2 is None else ids2.data_ptr(),
-                                    None if table2 is None else table2.data_ptr(), scale, x.data_ptr(), T, D, _DT[table.dtype],
-                                    _stream()), "embed_rows")
+                                    None if table2 is None else table2.data_ptr(), scale,
+                                    None if norm is None else norm.data_ptr(), eps, x.data_ptr(), T, D, _DT[table.dtype], _stream()),
+            "embed_rows")
         return x
 
     def add_norm(self, x, y1, y2, w_next, eps, act):
@@ -719,6 +745,35 @@ class HipOps:
                                   _DT[act], _stream()), "add_norm")
         return xa
 
+    def join_norms(self, x, y, y2, side, w1, w2, eps, act):
+        """x <- x + y + y2 in place on the float32 stream (either may be None); ``side`` = (ya, yb, wa, wb, mix) adds mix *
+        (rms(ya) wa + rms(yb) wb) in place of y.  Returns (rms(x) w1, rms(x) w2) as ``act``, None where there is no weight."""
+        ya, yb, wa, wb, mix = side or (None, None, None, None, 1.0)
+        _f32(x, wa, wb, w1, w2)
+        _act(y, y2, ya, yb)
+        rows, D = x.shape
+        if any(t is not None and (t.shape != x.shape or not t.is_contiguous() or t.dtype != act) for t in (y, y2, ya, yb)) \
+                or any(w is not None and w.numel() != D for w in (wa, wb, w1, w2)) or (y is not None and side) or (w1 is None and w2 is not None):
+            raise ValueError("sublayer outputs / norm weights do not fit the stream")
+        u1, u2 = (None if w is None else torch.empty(rows, D, dtype=act, device=x.device) for w in (w1, w2))
+        ptr = lambda t: None if t is None else t.data_ptr()                    # noqa: E731
+        a = _JoinArgs(*(ptr(t) for t in (x, y, y2, ya, yb, wa, wb)), float(mix), *(ptr(t) for t in (w1, w2, u1, u2)), D, eps)
+        _ok(lib().ragged_join_norms(a, rows, _DT[act], _stream()), "join_norms")
+        return u1, u2
+
+    def gate_group_norm(self, y, P, z0, w, groups, eps, act):
+        """w * groupnorm(y * silu(P[:, z0 ..])) as ``act``: float head outputs y [rows, n] gated, then every one of ``groups`` equal
+        parts of a row divided by its own root mean square."""
+        _f32(y, w)
+        _act(P)
+        rows, n = y.shape
+        if w.numel() != n or n % groups or P.shape[0] != rows or z0 + n > P.shape[1] or P.dtype != act:
+            raise ValueError("gate columns / norm groups do not fit")
+        out = torch.empty(rows, n, dtype=act, device=y.device)
+        _ok(lib().ragged_gate_group_norm(y.data_ptr(), P.data_ptr(), P.stride(0), z0, w.data_ptr(), out.data_ptr(), rows, n, groups, eps,
+                                         _DT[act], _stream()), "gate_group_norm")
+        return out
+
     _ACT_KINDS = {"gelu_erf": 0, "gelu_tanh": 1, "relu2": 2, "xielu": 3, "tanh": 4}
 
     def act_cols(self, P, col0, n, kind, params=(0.0, 0.0)):
@@ -732,14 +787,16 @@ class HipOps:
                                   float(params[1]), _DT[P.dtype], _stream()), "act_cols")
         return out
 
-    def glu_pairs(self, P):
-        """silu(P[:, 0::2]) * P[:, 1::2]: inner channels that come as neighbouring (gate, up) pairs."""
+    def glu_pairs(self, P, row_gate=None):
+        """silu(P[:, 0::2]) * P[:, 1::2]: inner channels that come as neighbouring (gate, up) pairs; ``row_gate`` float [rows] multiplies
+        a row."""
         _act(P)
-        if P.dim() != 2 or P.shape[1] % 2:
+        _f32(row_gate)
+        if P.dim() != 2 or P.shape[1] % 2 or (row_gate is not None and row_gate.numel() != P.shape[0]):
             raise ValueError("(gate, up) pairs expected")
         out = torch.empty(P.shape[0], P.shape[1] // 2, dtype=P.dtype, device=P.device)
         if out.numel():
-            _ok(lib().ragged_glu_pairs(P.data_ptr(), P.stride(0), out.data_ptr(), P.shape[0], P.shape[1] // 2, _DT[P.dtype], _stream()),
+            _ok(lib().ragged_glu_pairs(P.data_ptr(), P.stride(0), None if row_gate is None else row_gate.data_ptr(), out.data_ptr(), P.shape[0], P.shape[1] // 2, _DT[P.dtype], _stream()),
                 "glu_pairs")
         return out
 
@@ -825,10 +882,13 @@ class HipOps:
                                     None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt, st), what)
         return self._delta_passes(scan, state, H, d, vd, meta)
 
-    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta):
+    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta, wf=None):
         """S' = g S, u = beta (v - S'^T k), S <- S' + k u^T, o = S^T q per head (head h reads q / k head h / (H / G)): ``qf``,
-        ``kf`` [T, G d], ``gb`` [T, H, 2] = (g, beta), values V [T, H vd], ``state`` float [slots, H, d, vd]."""
-        _f32(qf, kf, gb, state)
+        ``kf`` [T, G d], ``gb`` [T, H, 2] = (g, beta), values V [T, H vd], ``state`` float [slots, H, d, vd].  ``wf`` [T, H d]: a
+        decay per key channel, S' = diag(w) S."""
+        _f32(qf, kf, gb, state, wf)
+        if wf is not None and wf.shape != (meta.T, H * d):
+            raise ValueError("one decay per head and key channel")
         _act(V)
         if G <= 0 or H % G or qf.shape != (meta.T, G * d) or kf.shape != qf.shape or gb.shape != (meta.T, H, 2) \
                 or V.shape != (meta.T, H * vd) or state.shape[1:] != (H, d, vd) or max(s[0] for s in meta.seqs) >= state.shape[0]:
@@ -836,7 +896,7 @@ class HipOps:
         L, dt, st = lib(), _DT[V.dtype], _stream()
 
         def scan(states, out, cols, values, batch, what):
-            _ok(L.ragged_gated_delta_scan(qf.data_ptr(), kf.data_ptr(), gb.data_ptr(), G, V.data_ptr() if values else None, V.stride(0), 0,
+            _ok(L.ragged_gated_delta_scan(qf.data_ptr(), kf.data_ptr(), None if wf is None else wf.data_ptr(), gb.data_ptr(), G, V.data_ptr() if values else None, V.stride(0), 0,
                                           states.data_ptr(), None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt,
                                           st), what)
         return self._delta_passes(scan, state, H, d, vd, meta)
@@ -881,16 +941,18 @@ class HipOps:
         scan(begin, out, vd, True, chunk_batch(ones), "delta_scan (chunks from their start states)")
         return out
 
-    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta):
+    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta, wl=None):
         """Inputs of ``gated_delta_scan`` from this step's projections, columns q [G d] | k [G d] | v [H vd] of P behind a causal
         convolution (``cw`` [channels, taps], older inputs in ``tail`` [slots, taps - 1, channels]) and silu: (unit q times
         d^-1/2, unit k, values of P's type, (exp(-arate softplus(a + dt_bias)), sigmoid(b)) with a, b = columns a0 .., b0 ..).
-        The tail moves on."""
+        ``wl`` float [T, H d]: decay logits per key channel (dt_bias [H d]); the fifth result is then exp(-arate softplus(wl + dt_bias))
+        and the first of the two gates is 1.  The tail moves on."""
         _act(P, tail)
-        _f32(cw, arate, dt_bias)
+        _f32(cw, arate, dt_bias, wl)
         C = 2 * G * d + H * vd
-        if P.dim() != 2 or P.shape[0] != meta.T or min(b0, a0) < C or max(b0, a0) + H > P.shape[1] or cw.shape != (C, taps) \
-                or arate.numel() != H or dt_bias.numel() != H or H % G:
+        if P.dim() != 2 or P.shape[0] != meta.T or b0 < C or b0 + H > P.shape[1] or cw.shape != (C, taps) or arate.numel() != H or H % G \
+                or dt_bias.numel() != (H if wl is None else H * d) or (wl is None and (a0 < C or a0 + H > P.shape[1])) \
+                or (wl is not None and wl.shape != (meta.T, H * d)):
             raise ValueError("delta-rule columns / taps / gates do not fit")
         self._tail_check(tail, taps, C, P.dtype, meta)
         dev = P.device
@@ -898,13 +960,15 @@ class HipOps:
         kf = torch.empty_like(qf)
         vo = torch.empty(meta.T, H * vd, dtype=P.dtype, device=dev)
         gb = torch.empty(meta.T, H, 2, dtype=torch.float32, device=dev)
+        wf = None if wl is None else torch.empty_like(wl)
         a = _GatedDeltaArgs(P.data_ptr(), P.stride(0), cw.data_ptr(), taps, None if tail is None else tail.data_ptr(), b0, a0,
-                            arate.data_ptr(), dt_bias.data_ptr(), float(tiny), qf.data_ptr(), kf.data_ptr(), vo.data_ptr(), gb.data_ptr(),
+                            arate.data_ptr(), dt_bias.data_ptr(), float(tiny), None if wl is None else wl.data_ptr(),
+                            None if wf is None else wf.data_ptr(), qf.data_ptr(), kf.data_ptr(), vo.data_ptr(), gb.data_ptr(),
                             H, G, d, vd, int(meta.single))
         _ok(lib().ragged_gated_delta_prep(a, meta.c(), _DT[P.dtype], _stream()), "gated_delta_prep")
         if taps > 1 and not meta.single:
             self.conv_state(P, 0, tail, taps, C, meta)
-        return qf, kf, vo, gb
+        return (qf, kf, vo, gb) if wf is None else (qf, kf, vo, gb, wf)
 
     @staticmethod
     def _tail_check(tail, taps, C, dtype, meta):
@@ -952,16 +1016,18 @@ class HipOps:
         return xa
 
     def qkv_rows(self, P, qw, kw, eps, rot, inv_freq, kpages, vpages, meta, *, H, G, d, vd, v_norm=False, first_in=None, lam=0.0,
-                 want_first=False):
+                 want_first=False, head_norms=False, q_temp=None):
         """Columns q [H d] | k [G d] | v [G vd] of P: q and k RMS-normed over the whole projection with a weight per channel, the
-        first ``rot`` channels of every head turned (pairs i, i + rot / 2); values RMS-normed per head (``v_norm``) and mixed with
+        first ``rot`` channels of every head turned (pairs i, i + rot / 2); ``head_norms``: every head normed by itself with a weight of
+        d channels that all heads share; ``q_temp`` = (coef, every): queries times 1 + coef ln(floor((pos + 1) / every) + 1); values RMS-normed per head (``v_norm``) and mixed with
         ``first_in`` [T, G vd] as (1 - lam) v + lam first.  Keys and values go to their pages; returns (q float [T, H d], the
         values as float if ``want_first`` else None)."""
         _act(P, kpages, vpages)
         _f32(qw, kw, inv_freq, first_in)
         _page_check(meta, kpages)
         _page_check(meta, vpages)
-        if P.dim() != 2 or P.shape[0] != meta.T or (H + G) * d + G * vd > P.shape[1] or qw.numel() != H * d or kw.numel() != G * d \
+        if P.dim() != 2 or P.shape[0] != meta.T or (H + G) * d + G * vd > P.shape[1] \
+                or qw.numel() != (d if head_norms else H * d) or kw.numel() != (d if head_norms else G * d) \
                 or kpages.shape[1:] != (G, PAGE, d) or vpages.shape[1:] != (G, PAGE, vd) or kpages.dtype != P.dtype or vpages.dtype != P.dtype \
                 or (first_in is not None and first_in.shape != (meta.T, G * vd)) or (rot and (inv_freq.numel() != rot // 2 or rot > d)):
             raise ValueError("projections / norm weights / cache pages do not fit the head layout")
@@ -970,9 +1036,26 @@ class HipOps:
         a = _QkvRowsArgs(P.data_ptr(), P.stride(0), H, G, d, vd, qw.data_ptr(), kw.data_ptr(), eps, rot,
                          meta.cossin(inv_freq).data_ptr() if rot else None, q.data_ptr(), kpages.data_ptr(), vpages.data_ptr(),
                          int(bool(v_norm)), None if first_in is None else first_in.data_ptr(),
-                         None if first is None else first.data_ptr(), float(lam))
+                         None if first is None else first.data_ptr(), float(lam), int(bool(head_norms)),
+                         int(q_temp[1]) if q_temp else 0, float(q_temp[0]) if q_temp else 0.0)
         _ok(lib().ragged_qkv_rows(a, meta.c(), _DT[P.dtype], _stream()), "qkv_rows")
         return q, first
+
+    def state_space_scan(self, X, b0, c0, P, dt0, dt_bias, rate, D, state, H, G, N, vd, meta):
+        """S <- exp(-rate d) S + d B x^T, y = S^T C + D x per head (head h reads group h / (H / G)), d = softplus(dt + dt_bias): x =
+        columns 0 .. H vd of X, B and C = columns b0 .. and c0 .. (G N each), step logits = columns dt0 .. of P (H), ``state`` float
+        [slots, H, N, vd].  Returns y float [T, H vd]."""
+        _act(X, P)
+        _f32(dt_bias, rate, D, state)
+        if X.shape[0] != meta.T or P.shape[0] != meta.T or X.dtype != P.dtype or H % G or H * vd > X.shape[1] or max(b0, c0) + G * N > X.shape[1] \
+                or dt0 + H > P.shape[1] or any(t.numel() != H for t in (dt_bias, rate, D)) or state.shape[1:] != (H, N, vd) \
+                or max(s[0] for s in meta.seqs) >= state.shape[0]:
+            raise ValueError("recurrent state / scan inputs do not fit")
+        y = torch.empty(meta.T, H * vd, dtype=torch.float32, device=X.device)
+        a = _SpaceArgs(P[:, dt0:].data_ptr(), P.stride(0), dt_bias.data_ptr(), rate.data_ptr(), D.data_ptr(), b0, c0)
+        _ok(lib().ragged_state_space_scan(a, X.data_ptr(), X.stride(0), G, state.data_ptr(), y.data_ptr(), H, N, vd, meta.c(), _DT[X.dtype],
+                                          _stream()), "state_space_scan")
+        return y
 
     selective_chunked_from = 128  # portions of at least this many tokens run the selective scan in chunks
     selective_waves = 4096        # wavefronts of a pass that the chunk length aims at (sixteen per CU)
@@ -1128,7 +1211,7 @@ class TorchOps:
         return (v if w is None else v * w).to(act)
 
     def paged_attn(self, q, kpages, vpages, meta, *, maps, H, G, d, vd, window, keep_first, scale, lam, out_scale, out_norm,
-                   eps, gate=None, gate0=0, sink=None, chunk=0, softcap=0.0, gate_wide=False, sinks=None, slopes=None):
+                   eps, gate=None, gate0=0, sink=None, chunk=0, softcap=0.0, gate_wide=False, sinks=None, slopes=None, dist_bias=None):
         out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=q.device)
         q = q.view(meta.T, H, maps, d)
         for b, (slot, past, n, pg) in enumerate(meta.seqs):
@@ -1150,6 +1233,8 @@ class TorchOps:
                 s = torch.einsum("thd,hld->htl", qs[:, :, mp], k[:, :, mp].repeat_interleave(rep, 0)) * scale
                 if slopes is not None:
                     s = s - slopes.view(H, 1, 1) * (i - j).float()
+                if dist_bias is not None:
+                    s = s + dist_bias[:, (i - j).clamp(0, dist_bias.shape[1] - 1)]
                 if softcap > 0:
                     s = softcap * torch.tanh(s / softcap)
                 s = s.masked_fill(~vis, float("-inf"))
@@ -1210,18 +1295,20 @@ class TorchOps:
         k = P[:, k0:k0 + H * d].float().view(T, H, d)
         return q, a[:, :, None].expand(T, H, d).reshape(T, -1).contiguous(), (b[:, :, None] * k).reshape(T, -1)
 
-    def moe_route(self, xa, w_router, groups, keep, top, scale, score="softmax", group_top=1, renorm=False):
+    def moe_route(self, xa, w_router, groups, keep, top, scale, score="softmax", group_top=1, renorm=False, correction=None, w_gate=None):
         z = xa.float() @ w_router.t()
         s = torch.sigmoid(z) if score == "sigmoid" else torch.softmax(z, -1)
         E = s.shape[1]
-        best = s.view(-1, groups, E // groups).topk(min(group_top, E // groups), -1).values.sum(-1)
+        c = s if correction is None else s + correction
+        best = c.view(-1, groups, E // groups).topk(min(group_top, E // groups), -1).values.sum(-1)
         kept = torch.zeros_like(best, dtype=torch.bool)
         kept.scatter_(1, best.topk(keep, -1).indices, True)
-        idx = s.masked_fill(~kept.repeat_interleave(E // groups, 1), -1.0).topk(top, -1).indices
+        idx = c.masked_fill(~kept.repeat_interleave(E // groups, 1), float("-inf")).topk(top, -1).indices
         w = s.gather(1, idx)
         if renorm:
             w = w / (w.sum(-1, keepdim=True) + 1e-20)
-        return idx.to(torch.int32), w * scale
+        gate = () if w_gate is None else (torch.sigmoid(xa.float() @ w_gate),)
+        return (idx.to(torch.int32), w * scale, *gate)
 
     def moe_sorted(self, xa, idx, wts, w_up, w_dn, base, gated=False):
         return None                                             # (the host statements run the experts one by one)
@@ -1242,9 +1329,24 @@ class TorchOps:
                 y[t] += wts[t, j] * (w_dn[e].float() @ a.float())
         return y.to(xa.dtype)
 
-    def embed_rows(self, ids, table, ids2=None, table2=None, scale=1.0):
+    def embed_rows(self, ids, table, ids2=None, table2=None, scale=1.0, norm=None, eps=0.0):
         x = table[ids].float() * scale
-        return x if table2 is None else x + table2[ids2].float()
+        x = x if table2 is None else x + table2[ids2].float()
+        return x if norm is None else x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * norm
+
+    def join_norms(self, x, y, y2, side, w1, w2, eps, act):
+        rms = lambda v: v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)       # noqa: E731
+        if side:
+            ya, yb, wa, wb, mix = side
+            x += mix * (rms(ya.float()) * wa + rms(yb.float()) * wb)
+        for t in (y, y2):
+            if t is not None:
+                x += t.float()
+        return tuple(None if w is None else (rms(x) * w).to(act) for w in (w1, w2))
+
+    def gate_group_norm(self, y, P, z0, w, groups, eps, act):
+        v = (y * F.silu(P[:, z0:z0 + y.shape[1]].float())).view(y.shape[0], groups, -1)
+        return ((v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)).reshape(y.shape) * w).to(act)
 
     def add_norm(self, x, y1, y2, w_next, eps, act):
         if y1 is not None:
@@ -1267,8 +1369,9 @@ class TorchOps:
             v = torch.relu(z).pow(2)
         return v.to(P.dtype)
 
-    def glu_pairs(self, P):
-        return (F.silu(P[:, 0::2].float()) * P[:, 1::2].float()).to(P.dtype)
+    def glu_pairs(self, P, row_gate=None):
+        v = F.silu(P[:, 0::2].float()) * P[:, 1::2].float()
+        return (v if row_gate is None else v * row_gate[:, None]).to(P.dtype)
 
     def hc_step(self, X, y, prev, nxt, w_next, eps, act, want_u=False):
         S = X.shape[1]
@@ -1305,23 +1408,28 @@ class TorchOps:
             state[slot] = S
         return out
 
-    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta):
+    def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta, wl=None):
         C, T = 2 * G * d + H * vd, meta.T
         u = F.silu(self._segment(P, 0, meta, cw, taps, C, 0, tail, C))
         if taps > 1:
             self.conv_state(P, 0, tail, taps, C, meta)
         unit = lambda v: (v / torch.sqrt(v.pow(2).sum(-1, keepdim=True) + tiny)).reshape(T, G * d)      # noqa: E731
-        g = torch.exp(-arate * F.softplus(P[:, a0:a0 + H].float() + dt_bias, threshold=80.0))
+        wf = ()
+        if wl is None:
+            g = torch.exp(-arate * F.softplus(P[:, a0:a0 + H].float() + dt_bias, threshold=80.0))
+        else:
+            g = torch.ones(T, H)
+            wf = (torch.exp(-arate.repeat_interleave(d) * F.softplus(wl + dt_bias, threshold=80.0)),)
         return unit(u[:, :G * d].reshape(T, G, d)) * d ** -0.5, unit(u[:, G * d:2 * G * d].reshape(T, G, d)), u[:, 2 * G * d:].to(P.dtype), \
-            torch.stack([g, torch.sigmoid(P[:, b0:b0 + H].float())], -1)
+            torch.stack([g, torch.sigmoid(P[:, b0:b0 + H].float())], -1), *wf
 
-    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta):
+    def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta, wf=None):
         out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=V.device)
         for b, (slot, past, n, _) in enumerate(meta.seqs):
             S = state[slot].clone() if past > 0 else torch.zeros_like(state[slot])
             for t in range(meta.start[b], meta.start[b] + n):
                 q, k = (a[t].view(G, d, 1).repeat_interleave(H // G, 0) for a in (qf, kf))
-                S = gb[t, :, 0].view(H, 1, 1) * S
+                S = gb[t, :, 0].view(H, 1, 1) * S if wf is None else wf[t].view(H, d, 1) * S
                 S = S + k * (gb[t, :, 1].view(H, 1, 1) * (V[t].float().view(H, 1, vd) - (S * k).sum(1, keepdim=True)))
                 out[t] = (S * q).sum(1).reshape(-1)
             state[slot] = S
@@ -1348,11 +1456,17 @@ class TorchOps:
         return x.to(act) if want else None
 
     def qkv_rows(self, P, qw, kw, eps, rot, inv_freq, kpages, vpages, meta, *, H, G, d, vd, v_norm=False, first_in=None, lam=0.0,
-                 want_first=False):
+                 want_first=False, head_norms=False, q_temp=None):
         u = P.float()
         nq, nk = H * d, G * d
         rms = lambda v: v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)       # noqa: E731
-        qk = torch.cat([rms(u[:, :nq]) * qw, rms(u[:, nq:nq + nk]) * kw], 1).contiguous()
+        if head_norms:
+            qk = torch.cat([(rms(u[:, :nq].reshape(-1, H, d)) * qw).reshape(-1, nq), (rms(u[:, nq:nq + nk].reshape(-1, G, d)) * kw).reshape(-1, nk)], 1)
+        else:
+            qk = torch.cat([rms(u[:, :nq]) * qw, rms(u[:, nq:nq + nk]) * kw], 1).contiguous()
+        if q_temp:
+            at = torch.div(meta.tok_pos.long() + 1, int(q_temp[1]), rounding_mode="floor").float() + 1.0
+            qk[:, :nq] *= (1.0 + q_temp[0] * torch.log(at))[:, None]
         none = dict(cw=None, taps=0, C=0, ch0=0, state=None, normw=None, eps=eps)
         q = torch.empty(meta.T, nq, dtype=torch.float32)
         k = torch.empty(meta.T, nk, dtype=torch.float32)
@@ -1365,6 +1479,19 @@ class TorchOps:
         for rows, n, pages in ((k, d, kpages), (v.contiguous(), vd, vpages)):
             self.conv_head(rows, 0, meta, ngroups=G, gsize=n, rot=0, inv_freq=None, pages=pages, **none)
         return q, (v if want_first else None)
+
+    def state_space_scan(self, X, b0, c0, P, dt0, dt_bias, rate, D, state, H, G, N, vd, meta):
+        out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=X.device)
+        step = F.softplus(P[:, dt0:dt0 + H].float() + dt_bias, threshold=80.0)
+        for b, (slot, past, n, _) in enumerate(meta.seqs):
+            S = state[slot].clone() if past > 0 else torch.zeros_like(state[slot])
+            for t in range(meta.start[b], meta.start[b] + n):
+                x = X[t, :H * vd].float().view(H, 1, vd)
+                B, C = (X[t, c:c + G * N].float().view(G, N, 1).repeat_interleave(H // G, 0) for c in (b0, c0))
+                S = torch.exp(-rate * step[t]).view(H, 1, 1) * S + step[t].view(H, 1, 1) * B * x
+                out[t] = ((S * C).sum(1) + D.view(H, 1) * x[:, 0]).reshape(-1)
+            state[slot] = S
+        return out
 
     def selective_scan(self, x, dt, dt_bias, M, b0, c0, A, D, P, z0, state, meta):
         C, N = A.shape
