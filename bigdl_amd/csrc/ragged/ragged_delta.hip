@@ -8,7 +8,7 @@
 // the same scan with two arrays and two scalars per token instead of five arrays, or with three where g has a number per key
 // channel.  The state space recurrence (Mamba-2) is the one without the forgetting term,
 //     S <- exp(-a d) S + d B x^T,   y = S^T C + D x,     d = softplus(step logit + bias) per head.
-#include "ragged_common.h"
+#include "ragged_space.h"
 
 using namespace ragged;
 
@@ -248,7 +248,8 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
 // arrays).  The five arrays of a block of TB tokens are brought into LDS by the whole workgroup with coalesced loads
 // while the previous block is scanned (register look-ahead, two LDS buffers) and read back as 16-byte broadcasts.
 // Grid: (column blocks, heads, sequences).  `values` = 0: v is taken as 0 (the state only decays and forgets: from an
-// identity state this yields a chunk's transition matrix).
+// identity state this yields a chunk's transition matrix).  `trans`: both at once, sequences grid.z / 2 .. scan the same tokens
+// without values from the d columns of `trans` (a state array like `state`).
 // MODE: which recurrence.
 //   general  five arrays, as above.
 //   gated    q and k of G heads (head h reads head h / (H / G)); `gb` holds every token's decay and write strength per head, and the
@@ -257,15 +258,6 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
 //   space    the state space recurrence: q and k are the rows C and B of G groups, columns c0 .. and b0 .. of P (type T); a token's
 //            decay and step size per head come from its step logit (`ss`), the read-out takes D v on top.
 enum DeltaMode { DL_GENERAL, DL_GATED, DL_CHANNEL, DL_SPACE };
-
-struct SpaceArgs {
-  const void* dt;        // step logits: row t, column h of a [rows, lddt] matrix of type T
-  int64_t lddt;
-  const float* dt_bias;  // [H]
-  const float* rate;     // [H]
-  const float* D;        // [H]
-  int b0, c0;
-};
 
 constexpr int DL_DR = 32;
 constexpr int DL_SEG = DL_DR + 4;   // LDS floats per lane group and token (padding shifts the banks between groups)
@@ -277,14 +269,21 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
                                                          const float* __restrict__ kf, const float* __restrict__ gb, int G,
                                                          const T* __restrict__ P, int64_t ldp, int v0,
                                                          float* __restrict__ state, float* __restrict__ out, int H, int d, int vd,
-                                                         int R, int TB, int values, SpaceArgs ss, Batch bt) {
+                                                         float* __restrict__ trans, int R, int TB, int values, SpaceArgs ss, Batch bt) {
   constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2, KI = MODE == DL_GENERAL ? 4 : 1;    // arrays, k's place among them
   constexpr bool GB = MODE != DL_GENERAL;                    // two scalars per token
   constexpr int NT = 64 * NW, DL_PRE = NA * DL_TBR * DL_DR / NT;
   extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k (r, k, w): [TB][R][SEG] each, v[TB][wcols], (g, beta)[TB] }
-  const int b = blockIdx.z, h = blockIdx.y, tid = threadIdx.x;
+  int b = blockIdx.z;
+  bool fresh = true;                                         // sequences without a past start from zero
+  if (trans) {
+    const int half = gridDim.z >> 1;
+    if (b >= half) { b -= half; state = trans; vd = d; values = 0; fresh = false; }
+  }
+  const int h = blockIdx.y, tid = threadIdx.x;
   const int wave = tid >> 6, lane = tid & 63;
   const int cols = 64 / R, wcols = NW * cols;
+  if ((int)blockIdx.x * wcols >= vd) return;                 // (the whole workgroup: no barrier is left waiting)
   const int r = lane % R, lc = wave * cols + lane / R;     // column inside the workgroup's block
   const int col = blockIdx.x * wcols + lc;
   const int start = bt.seq_start[b], n = bt.seq_start[b + 1] - start, past = bt.seq_past[b], slot = bt.seq_slot[b];
@@ -303,7 +302,7 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
     for (int k = 0; k < DL_DR; ++k) {
       const int row = row0 + k;
       const float v = sp[(int64_t)(row < d ? row : d - 1) * vd + cc];    // no condition around the load
-      S[k] = (past > 0 && colok && row < d) ? v : 0.f;
+      S[k] = ((past > 0 || !fresh) && colok && row < d) ? v : 0.f;
     }
   }
   float pre[DL_PRE], prev[4], preg = 0.f;
@@ -402,6 +401,18 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
         dot = group_sum((acc[0] + acc[1]) + (acc[2] + acc[3]), R);
         acc[0] = acc[1] = acc[2] = acc[3] = 0.f;
       }
+      if (MODE == DL_CHANNEL && !out) {                      // (only the end states are wanted)
+        const float c = buf[NA * qsz + TB * wcols + 2 * tk + 1] * (v - dot);
+#pragma unroll
+        for (int k = 0; k < DL_DR / 4; ++k) {
+          const float4 kk = k4[k];
+          S[4 * k] += kk.x * c;
+          S[4 * k + 1] += kk.y * c;
+          S[4 * k + 2] += kk.z * c;
+          S[4 * k + 3] += kk.w * c;
+        }
+        continue;
+      }
       if (MODE == DL_CHANNEL) {
         const float c = buf[NA * qsz + TB * wcols + 2 * tk + 1] * (v - dot);
 #pragma unroll
@@ -452,42 +463,45 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
 
 template <int MODE>
 static int launch_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const float* gb, int G,
-                             const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, SpaceArgs ss,
-                             Batch bt, int dtype, hipStream_t st) {
+                             const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, float* trans,
+                             SpaceArgs ss, Batch bt, int dtype, hipStream_t st) {
   constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2;
   if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 32 || (values && !P)) return -1;
+  if (trans && (out || !values || bt.B > 32767)) return -1;
   int R = 1;
   while (R * DL_DR < d) R <<= 1;
-  const int nw = vd <= 2 * (64 / R) ? 2 : 4;                // wavefronts of a workgroup: no more than the columns ask for
+  const int cols = trans && d > vd ? d : vd;
+  const int nw = cols <= 2 * (64 / R) ? 2 : 4;              // wavefronts of a workgroup: no more than the columns ask for
   const int wcols = nw * (64 / R);
   int TB = DL_TBR / R < 16 ? DL_TBR / R : 16;
   if (TB * wcols > 4 * 64 * nw) TB = 4 * 64 * nw / wcols;   // the value look-ahead holds 4 floats per thread
   if (TB < 1) return -1;
   // (2 TB <= 32 threads bring a token's two scalars; TB wcols and a buffer's parts are multiples of 16 bytes)
   const size_t sm = 2 * (size_t)(NA * TB * R * DL_SEG + TB * wcols + (MODE != DL_GENERAL ? (2 * TB + 3) & ~3 : 0)) * sizeof(float);
-  const dim3 grid((vd + wcols - 1) / wcols, H, bt.B);
+  const dim3 grid((cols + wcols - 1) / wcols, H, trans ? 2 * bt.B : bt.B);
   RAGGED_DISPATCH(dtype,
     if (nw == 2) hipLaunchKernelGGL((delta_scan_kernel<T, 2, MODE>), grid, dim3(128), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp,
-                                    v0, state, out, H, d, vd, R, TB, values, ss, bt);
+                                    v0, state, out, H, d, vd, trans, R, TB, values, ss, bt);
     else hipLaunchKernelGGL((delta_scan_kernel<T, 4, MODE>), grid, dim3(256), sm, st, rf, wf, nf, bf, kf, gb, G, (const T*)P, ldp, v0,
-                            state, out, H, d, vd, R, TB, values, ss, bt))
+                            state, out, H, d, vd, trans, R, TB, values, ss, bt))
   return RAGGED_LAUNCH_OK();
 }
 
-// out may be null (only the end states are wanted); values = 0: the value columns of P are not read and count as 0
+// out may be null (only the end states are wanted); values = 0: the value columns of P are not read and count as 0; trans (with
+// values, without out): the chunks' transition matrices in the same launch
 extern "C" int ragged_delta_scan(const float* rf, const float* wf, const float* nf, const float* bf, const float* kf, const void* P,
-                                 int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, Batch bt,
+                                 int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, float* trans, Batch bt,
                                  int dtype, hipStream_t st) {
-  return launch_delta_scan<DL_GENERAL>(rf, wf, nf, bf, kf, nullptr, H, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt, dtype, st);
+  return launch_delta_scan<DL_GENERAL>(rf, wf, nf, bf, kf, nullptr, H, P, ldp, v0, state, out, H, d, vd, values, trans, SpaceArgs{}, bt, dtype, st);
 }
 
 // the gated rule: qf, kf [rows, G d], gb [rows, H, 2]; wf [rows, H d] or null: a decay per key channel
 extern "C" int ragged_gated_delta_scan(const float* qf, const float* kf, const float* wf, const float* gb, int G, const void* P, int64_t ldp, int v0,
-                                       float* state, float* out, int H, int d, int vd, int values, Batch bt, int dtype, hipStream_t st) {
+                                       float* state, float* out, int H, int d, int vd, int values, float* trans, Batch bt, int dtype, hipStream_t st) {
   if (G <= 0 || H % G || !gb) return -1;
-  if (wf) return launch_delta_scan<DL_CHANNEL>(qf, wf, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt,
+  if (wf) return launch_delta_scan<DL_CHANNEL>(qf, wf, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, trans, SpaceArgs{}, bt,
                                                dtype, st);
-  return launch_delta_scan<DL_GATED>(qf, nullptr, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, SpaceArgs{}, bt, dtype, st);
+  return launch_delta_scan<DL_GATED>(qf, nullptr, nullptr, nullptr, kf, gb, G, P, ldp, v0, state, out, H, d, vd, values, trans, SpaceArgs{}, bt, dtype, st);
 }
 
 // the state space recurrence: X [rows, ldx] of type T holds x (columns 0 .. H vd), B and C (columns b0 .., c0 .., G d each)
@@ -495,7 +509,7 @@ extern "C" int ragged_state_space_scan(SpaceArgs ss, const void* X, int64_t ldx,
                                        Batch bt, int dtype, hipStream_t st) {
   if (G <= 0 || H % G || !ss.dt || !ss.dt_bias || !ss.rate || !ss.D || ss.lddt < H || ss.b0 < 0 || ss.c0 < 0) return -1;
   if (ldx < (int64_t)H * vd || ldx < ss.b0 + (int64_t)G * d || ldx < ss.c0 + (int64_t)G * d || !out) return -1;
-  return launch_delta_scan<DL_SPACE>(nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, G, X, ldx, 0, state, out, H, d, vd, 1, ss, bt, dtype, st);
+  return launch_delta_scan<DL_SPACE>(nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, G, X, ldx, 0, state, out, H, d, vd, 1, nullptr, ss, bt, dtype, st);
 }
 
 // ---------------------------------------------------------------------------------------------------------------

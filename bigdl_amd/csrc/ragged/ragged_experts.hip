@@ -32,10 +32,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
   __syncthreads();
   // two experts per wavefront and pass, 16 bytes of each router row per lane: eight loads in flight
   const bool v4 = (D & 3) == 0;
-  for (int e0 = 2 * wave; e0 < E; e0 += 8) {
-    const int e1 = e0 + 1 < E ? e0 + 1 : e0;
-    const float* w0 = wr + (int64_t)e0 * D;
-    const float* w1 = wr + (int64_t)e1 * D;
+  const int rows = wg ? E + 1 : E;                          // (the row of the shared expert's gate comes last)
+  for (int e0 = 2 * wave; e0 < rows; e0 += 8) {
+    const int e1 = e0 + 1 < rows ? e0 + 1 : e0;
+    const float* w0 = e0 < E ? wr + (int64_t)e0 * D : wg;
+    const float* w1 = e1 < E ? wr + (int64_t)e1 * D : wg;
     float a0 = 0.f, a1 = 0.f;
     if (v4) {
       for (int c = 4 * lane; c < D; c += 1024) {
@@ -59,15 +60,13 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
     }
     a0 = wave_sum(a0);
     a1 = wave_sum(a1);
-    if (lane == 0) { z[e0] = a0; z[e1] = a1; }
+    if (lane == 0) {
+      if (e0 < E) z[e0] = a0;
+      if (e1 < E) z[e1] = a1;
+      if (e1 == E) gate_out[t] = 1.0f / (1.0f + expf(-a1));       // (an odd count repeats its last row)
+    }
   }
   __syncthreads();
-  if (wg && wave == 3) {
-    float g = 0.f;
-    for (int c = lane; c < D; c += 64) g += wg[c] * xs[c];
-    g = wave_sum(g);
-    if (lane == 0) gate_out[t] = 1.0f / (1.0f + expf(-g));
-  }
   if (wave != 0) return;
   constexpr float NONE = -INFINITY;
   float s[MOE_SLOTS];

@@ -1,0 +1,13 @@
+// Argument block shared by the two kernels of the state space recurrence (token by token in ragged_delta.hip, long bfloat16
+// portions on the matrix cores in ragged_space.hip).
+#pragma once
+#include "ragged_common.h"
+
+struct SpaceArgs {
+  const void* dt;        // step logits: row t, column h of a [rows, lddt] matrix of type T
+  int64_t lddt;
+  const float* dt_bias;  // [H]
+  const float* rate;     // [H]
+  const float* D;        // [H]
+  int b0, c0;            // columns of the inputs' matrix where B and C begin
+};

@@ -148,15 +148,17 @@ def lib():
         L.ragged_embed_rows.argtypes = [vp, vp, vp, vp, cf, vp, cf, vp, i64, ci, ci, vp]
         L.ragged_join_norms.argtypes = [_JoinArgs, i64, ci, vp]
         L.ragged_gate_group_norm.argtypes = [vp, vp, i64, ci, vp, vp, i64, ci, ci, cf, ci, vp]
+        L.ragged_state_space_mfma_ok.argtypes = [ci]
+        L.ragged_state_space_mfma.argtypes = [_SpaceArgs, vp, i64, ci, vp, vp, ci, ci, ci, _Batch, vp]
         L.ragged_state_space_scan.argtypes = [_SpaceArgs, vp, i64, ci, vp, vp, ci, ci, ci, _Batch, ci, vp]
         L.ragged_add_norm.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, ci, vp]
         L.ragged_act_cols.argtypes = [vp, i64, ci, vp, i64, ci, ci, cf, cf, ci, vp]
         L.ragged_hc_step.argtypes = [vp, vp, vp, vp, vp, vp, vp, i64, ci, ci, cf, ci, vp]
         L.ragged_gate_cols.argtypes = [vp, vp, i64, ci, vp, i64, ci, cf, ci, vp]
         L.ragged_delta_gates.argtypes = [vp, i64, ci, ci, ci, vp, vp, vp, cf, cf, vp, vp, vp, vp, vp, i64, ci, ci, ci, vp]
-        L.ragged_delta_scan.argtypes = [vp, vp, vp, vp, vp, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
+        L.ragged_delta_scan.argtypes = [vp, vp, vp, vp, vp, vp, i64, ci, vp, vp, ci, ci, ci, ci, vp, _Batch, ci, vp]
         L.ragged_gated_delta_prep.argtypes = [_GatedDeltaArgs, _Batch, ci, vp]
-        L.ragged_gated_delta_scan.argtypes = [vp, vp, vp, vp, ci, vp, i64, ci, vp, vp, ci, ci, ci, ci, _Batch, ci, vp]
+        L.ragged_gated_delta_scan.argtypes = [vp, vp, vp, vp, ci, vp, i64, ci, vp, vp, ci, ci, ci, ci, vp, _Batch, ci, vp]
         L.ragged_conv_rows.argtypes = [vp, i64, ci, vp, vp, vp, ci, ci, vp, ci, ci, ci, _Batch, ci, ci, vp]
         L.ragged_ln_add.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, vp, ci, vp, _Batch, ci, vp]
         L.ragged_qkv_rows.argtypes = [_QkvRowsArgs, _Batch, ci, vp]
@@ -877,9 +879,9 @@ class HipOps:
         L, dt, st = lib(), _DT[P.dtype], _stream()
         ptrs = [a.data_ptr() for a in arrays]
 
-        def scan(states, out, cols, values, batch, what):
-            _ok(L.ragged_delta_scan(*ptrs, P.data_ptr() if values else None, P.stride(0), v0, states.data_ptr(),
-                                    None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt, st), what)
+        def scan(states, out, trans, batch, what):
+            _ok(L.ragged_delta_scan(*ptrs, P.data_ptr(), P.stride(0), v0, states.data_ptr(), None if out is None else out.data_ptr(), H, d,
+                                    vd, 1, None if trans is None else trans.data_ptr(), batch, dt, st), what)
         return self._delta_passes(scan, state, H, d, vd, meta)
 
     def gated_delta_scan(self, qf, kf, gb, G, V, state, H, d, vd, meta, wf=None):
@@ -895,23 +897,23 @@ class HipOps:
             raise ValueError("recurrent state / scan arrays do not fit")
         L, dt, st = lib(), _DT[V.dtype], _stream()
 
-        def scan(states, out, cols, values, batch, what):
-            _ok(L.ragged_gated_delta_scan(qf.data_ptr(), kf.data_ptr(), None if wf is None else wf.data_ptr(), gb.data_ptr(), G, V.data_ptr() if values else None, V.stride(0), 0,
-                                          states.data_ptr(), None if out is None else out.data_ptr(), H, d, cols, int(values), batch, dt,
-                                          st), what)
+        def scan(states, out, trans, batch, what):
+            _ok(L.ragged_gated_delta_scan(qf.data_ptr(), kf.data_ptr(), None if wf is None else wf.data_ptr(), gb.data_ptr(), G, V.data_ptr(),
+                                          V.stride(0), 0, states.data_ptr(), None if out is None else out.data_ptr(), H, d, vd, 1,
+                                          None if trans is None else trans.data_ptr(), batch, dt, st), what)
         return self._delta_passes(scan, state, H, d, vd, meta)
 
     def _delta_passes(self, scan, state, H, d, vd, meta):
-        """``scan(states, out or None, columns, with values, batch, name)``: one pass of either delta rule"""
+        """``scan(states, out or None, transition matrices or None, batch, name)``: one pass of either delta rule"""
         L, st, device = lib(), _stream(), state.device
         out = torch.empty(meta.T, H * vd, dtype=torch.float32, device=device)
         longest = max(n for _, _, n, _ in meta.seqs)
         if longest < self.delta_chunked_from:
-            scan(state, out, vd, True, meta.c(), "delta_scan")
+            scan(state, out, None, meta.c(), "delta_scan")
             return out
         # Long portions: chunks side by side.  A chunk maps its start state linearly, S_end = A S_start + L: L is the chunk
-        # scanned from zero, A (d x d per head) the chunk scanned without inputs from the identity.  The chunk-start states
-        # follow one after the other from those, and the chunks are scanned again from them for the outputs.
+        # scanned from zero, A (d x d per head) the chunk scanned without inputs from the identity (one launch makes both).  The
+        # chunk-start states follow one after the other from those, and the chunks are scanned again from them for the outputs.
         nc, cstart, zeros, ones, cid, cfirst, last = meta.chunks(self._delta_chunk_length(meta, H, d, vd))
         local = torch.empty(nc, H, d, vd, dtype=torch.float32, device=device)
         trans = torch.eye(d, dtype=torch.float32, device=device).repeat(nc, H, 1, 1)
@@ -919,8 +921,7 @@ class HipOps:
 
         def chunk_batch(past):
             return _Batch(None, None, cstart.data_ptr(), past.data_ptr(), cid.data_ptr(), None, meta.T, nc, 0)
-        scan(local, None, vd, True, chunk_batch(zeros), "delta_scan (chunks from zero)")
-        scan(trans, None, d, False, chunk_batch(ones), "delta_scan (transition matrices)")
+        scan(local, None, trans, chunk_batch(zeros), "delta_scan (chunks from zero, transition matrices)")
         if self.delta_chain and L.ragged_delta_chain_ok(d):
             _ok(L.ragged_delta_chain(state.data_ptr(), local.data_ptr(), trans.data_ptr(), begin.data_ptr(), cfirst.data_ptr(),
                                      meta.seq_past.data_ptr(), meta.seq_slot.data_ptr(), meta.B, H, d, vd, st), "delta_chain")
@@ -938,7 +939,7 @@ class HipOps:
                 begin[cs] = S[bi]
                 S[bi] = torch.matmul(trans[cs], S[bi]) + local[cs]
             state[slots] = S
-        scan(begin, out, vd, True, chunk_batch(ones), "delta_scan (chunks from their start states)")
+        scan(begin, out, None, chunk_batch(ones), "delta_scan (chunks from their start states)")
         return out
 
     def gated_delta_prep(self, P, cw, taps, tail, b0, a0, arate, dt_bias, tiny, H, G, d, vd, meta, wl=None):
@@ -1041,6 +1042,8 @@ class HipOps:
         _ok(lib().ragged_qkv_rows(a, meta.c(), _DT[P.dtype], _stream()), "qkv_rows")
         return q, first
 
+    space_blocks_from = 16    # bfloat16 portions of at least this many tokens run the state space recurrence in blocks of 64
+
     def state_space_scan(self, X, b0, c0, P, dt0, dt_bias, rate, D, state, H, G, N, vd, meta):
         """S <- exp(-rate d) S + d B x^T, y = S^T C + D x per head (head h reads group h / (H / G)), d = softplus(dt + dt_bias): x =
         columns 0 .. H vd of X, B and C = columns b0 .. and c0 .. (G N each), step logits = columns dt0 .. of P (H), ``state`` float
@@ -1053,6 +1056,11 @@ class HipOps:
             raise ValueError("recurrent state / scan inputs do not fit")
         y = torch.empty(meta.T, H * vd, dtype=torch.float32, device=X.device)
         a = _SpaceArgs(P[:, dt0:].data_ptr(), P.stride(0), dt_bias.data_ptr(), rate.data_ptr(), D.data_ptr(), b0, c0)
+        if X.dtype == torch.bfloat16 and max(n for _, _, n, _ in meta.seqs) >= self.space_blocks_from and lib().ragged_state_space_mfma_ok(N) \
+                and not (b0 % 8 or c0 % 8 or X.stride(0) % 8 or X.data_ptr() % 16):
+            _ok(lib().ragged_state_space_mfma(a, X.data_ptr(), X.stride(0), G, state.data_ptr(), y.data_ptr(), H, N, vd, meta.c(), _stream()),
+                "state_space_mfma")
+            return y
         _ok(lib().ragged_state_space_scan(a, X.data_ptr(), X.stride(0), G, state.data_ptr(), y.data_ptr(), H, N, vd, meta.c(), _DT[X.dtype],
                                           _stream()), "state_space_scan")
         return y
