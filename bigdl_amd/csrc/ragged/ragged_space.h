@@ -10,4 +10,6 @@ struct SpaceArgs {
   const float* rate;     // [H]
   const float* D;        // [H]
   int b0, c0;            // columns of the inputs' matrix where B and C begin
+  float* sum_log;        // [B, H] or null (matrix-core kernel): the sum of a sequence's log decays
+  int keep_end;          // 1: the last state goes back to the state array (always so token by token)
 };

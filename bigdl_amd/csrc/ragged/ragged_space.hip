@@ -17,6 +17,8 @@
 //  * rows of B and C, and B transposed, are staged in LDS by the whole workgroup from registers requested one block ahead; the score
 //    tiles are shared out over the wavefronts (wavefront w: the 16 tokens 16 w ..) and exchanged through LDS.
 // Tokens behind a portion's end take d = 0: they decay nothing and write nothing.
+// A long portion is cut into segments that are walked side by side: first from zero for their end states alone (`out` null: no C,
+// no scores), then, once space_chain_kernel has turned those into start states, for the outputs.
 #include "ragged_space.h"
 
 using namespace ragged;
@@ -70,6 +72,8 @@ __global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, con
   const int start = bt.seq_start[b], n = bt.seq_start[b + 1] - start, past = bt.seq_past[b], slot = bt.seq_slot[b];
   const int p = blockIdx.x * 64 + 16 * wave + lq, pc = p < vd ? p : vd - 1;
   const float rate = ss.rate[h], dtb = ss.dt_bias[h], skip = ss.D[h];
+  const bool outs = out != nullptr;
+  double total = 0.0;
   float* sp = state + ((int64_t)slot * H + h) * N * vd;
   f32x4 S[NT];
 #pragma unroll
@@ -90,7 +94,7 @@ __global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, con
     for (int it = 0; it < KS; ++it) {
       const int e0 = 8 * (4 * it + wave);
       const bool in = e0 < N;                                // (N is a multiple of 8)
-      creg[it].q = in ? *reinterpret_cast<const uint4*>(src + ss.c0 + e0) : uint4{0, 0, 0, 0};
+      creg[it].q = in && outs ? *reinterpret_cast<const uint4*>(src + ss.c0 + e0) : uint4{0, 0, 0, 0};
       breg[it].q = in ? *reinterpret_cast<const uint4*>(src + ss.b0 + e0) : uint4{0, 0, 0, 0};
     }
     dtn = to_f(((const bf16*)ss.dt)[(int64_t)(start + row) * ss.lddt + h]);
@@ -115,8 +119,10 @@ __global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, con
 #pragma unroll
     for (int it = 0; it < KS; ++it) {
       const int e0 = 8 * (4 * it + wave);
-      *reinterpret_cast<uint4*>(Cs + lane * LDN + e0) = creg[it].q;
-      *reinterpret_cast<uint4*>(Bs + lane * LDN + e0) = breg[it].q;
+      if (outs) {
+        *reinterpret_cast<uint4*>(Cs + lane * LDN + e0) = creg[it].q;
+        *reinterpret_cast<uint4*>(Bs + lane * LDN + e0) = breg[it].q;
+      }
 #pragma unroll
       for (int u = 0; u < 8; ++u) BT[(e0 + u) * SP_LDT + lane] = breg[it].h[u];
     }
@@ -135,92 +141,95 @@ __global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, con
     cum[lane] = run_hi;
     cuml[lane] = run_lo;
     dts[lane] = d;
+    total += run;                                            // (of lane 63: the whole block)
     const float last = lane_value(run_hi, 63), last_lo = lane_value(run_lo, 63);
     __syncthreads();
     if (c0 + SP_Q < n) fetch(c0 + SP_Q);                     // in flight during this block's arithmetic
 
-    // ---- scores of this wavefront's 16 tokens t against the tokens s <= t, decayed, as two-term operands
-    {
-      const int t = 16 * wave + lq;
-      const float ct = cum[t], ctl = cuml[t];
-      Frag cf[KS];
+    if (outs) {
+      // ---- scores of this wavefront's 16 tokens t against the tokens s <= t, decayed, as two-term operands
+      {
+        const int t = 16 * wave + lq;
+        const float ct = cum[t], ctl = cuml[t];
+        Frag cf[KS];
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) cf[ks] = pieces(Cs + t * LDN, ks);
+        for (int ks = 0; ks < KS; ++ks) cf[ks] = pieces(Cs + t * LDN, ks);
 #pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        if (2 * k > wave) continue;                          // (no token of these 32 lies at or before t)
-        Frag hi, lo;
+        for (int k = 0; k < 2; ++k) {
+          if (2 * k > wave) continue;                          // (no token of these 32 lies at or before t)
+          Frag hi, lo;
 #pragma unroll
-        for (int half = 0; half < 2; ++half) {
-          const int st = 2 * k + half;
-          f32x4 m = f32x4{0.f, 0.f, 0.f, 0.f};
-          if (st <= wave) {
+          for (int half = 0; half < 2; ++half) {
+            const int st = 2 * k + half;
+            f32x4 m = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (st <= wave) {
 #pragma unroll
-            for (int ks = 0; ks < KS; ++ks)
-              m = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pieces(Bs + (16 * st + lq) * LDN, ks).v, cf[ks].v, m, 0, 0, 0);
-            const int s0 = 16 * st + 4 * g4;
-            const float4 cs = *reinterpret_cast<const float4*>(cum + s0), cl = *reinterpret_cast<const float4*>(cuml + s0);
-            const float4 ds = *reinterpret_cast<const float4*>(dts + s0);
-            const float cv[4] = {cs.x, cs.y, cs.z, cs.w}, lv[4] = {cl.x, cl.y, cl.z, cl.w}, dv[4] = {ds.x, ds.y, ds.z, ds.w};
+              for (int ks = 0; ks < KS; ++ks)
+                m = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pieces(Bs + (16 * st + lq) * LDN, ks).v, cf[ks].v, m, 0, 0, 0);
+              const int s0 = 16 * st + 4 * g4;
+              const float4 cs = *reinterpret_cast<const float4*>(cum + s0), cl = *reinterpret_cast<const float4*>(cuml + s0);
+              const float4 ds = *reinterpret_cast<const float4*>(dts + s0);
+              const float cv[4] = {cs.x, cs.y, cs.z, cs.w}, lv[4] = {cl.x, cl.y, cl.z, cl.w}, dv[4] = {ds.x, ds.y, ds.z, ds.w};
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
-              const int s = s0 + i;
-              const float v = m[i] * __expf((ct - cv[i]) + (ctl - lv[i])) * dv[i];
-              m[i] = s < t ? v : s == t ? v + skip : 0.f;
+              for (int i = 0; i < 4; ++i) {
+                const int s = s0 + i;
+                const float v = m[i] * __expf((ct - cv[i]) + (ctl - lv[i])) * dv[i];
+                m[i] = s < t ? v : s == t ? v + skip : 0.f;
+              }
             }
+            split_pair(m[0], m[1], hi, lo, 2 * half);
+            split_pair(m[2], m[3], hi, lo, 2 * half + 1);
           }
-          split_pair(m[0], m[1], hi, lo, 2 * half);
-          split_pair(m[2], m[3], hi, lo, 2 * half + 1);
-        }
-        Mf[((wave * 2 + k) * 2) * 64 + lane] = hi.q;
-        Mf[((wave * 2 + k) * 2 + 1) * 64 + lane] = lo.q;
-      }
-    }
-    // ---- what the block's start state adds to every token's output: y^T[p][t], lane = token t
-    f32x4 Y[4];
-#pragma unroll
-    for (int tt = 0; tt < 4; ++tt) Y[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (past > 0 || c0 > 0) {
-#pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        Frag hi, lo;
-#pragma unroll
-        for (int half = 0; half < 2; ++half) {
-          split_pair(S[2 * ks + half][0], S[2 * ks + half][1], hi, lo, 2 * half);
-          split_pair(S[2 * ks + half][2], S[2 * ks + half][3], hi, lo, 2 * half + 1);
-        }
-#pragma unroll
-        for (int tt = 0; tt < 4; ++tt) {
-          const Frag cf = pieces(Cs + (16 * tt + lq) * LDN, ks);
-          Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi.v, cf.v, Y[tt], 0, 0, 0);
-          Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo.v, cf.v, Y[tt], 0, 0, 0);
+          Mf[((wave * 2 + k) * 2) * 64 + lane] = hi.q;
+          Mf[((wave * 2 + k) * 2 + 1) * 64 + lane] = lo.q;
         }
       }
+      // ---- what the block's start state adds to every token's output: y^T[p][t], lane = token t
+      f32x4 Y[4];
 #pragma unroll
-      for (int tt = 0; tt < 4; ++tt) Y[tt] *= expf(cum[16 * tt + lq]);
-    }
-    __syncthreads();                                         // every wavefront's scores are there
-    // ---- the block's own tokens
+      for (int tt = 0; tt < 4; ++tt) Y[tt] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (past > 0 || c0 > 0) {
 #pragma unroll
-    for (int tt = 0; tt < 4; ++tt) {
+        for (int ks = 0; ks < KS; ++ks) {
+          Frag hi, lo;
 #pragma unroll
-      for (int k = 0; k < 2; ++k) {
-        if (2 * k > tt) continue;
-        Frag hi, lo;
-        hi.q = Mf[((tt * 2 + k) * 2) * 64 + lane];
-        lo.q = Mf[((tt * 2 + k) * 2 + 1) * 64 + lane];
-        Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xs[k].v, hi.v, Y[tt], 0, 0, 0);
-        Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xs[k].v, lo.v, Y[tt], 0, 0, 0);
+          for (int half = 0; half < 2; ++half) {
+            split_pair(S[2 * ks + half][0], S[2 * ks + half][1], hi, lo, 2 * half);
+            split_pair(S[2 * ks + half][2], S[2 * ks + half][3], hi, lo, 2 * half + 1);
+          }
+#pragma unroll
+          for (int tt = 0; tt < 4; ++tt) {
+            const Frag cf = pieces(Cs + (16 * tt + lq) * LDN, ks);
+            Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(hi.v, cf.v, Y[tt], 0, 0, 0);
+            Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(lo.v, cf.v, Y[tt], 0, 0, 0);
+          }
+        }
+#pragma unroll
+        for (int tt = 0; tt < 4; ++tt) Y[tt] *= expf(cum[16 * tt + lq]);
       }
-      const int t = 16 * tt + lq, p0 = blockIdx.x * 64 + 16 * wave + 4 * g4;
-      if (t < nt) {
-        float* o = out + (int64_t)(start + c0 + t) * (H * vd) + h * vd + p0;
-        if ((vd & 3) == 0) {
-          if (p0 < vd) *reinterpret_cast<float4*>(o) = float4{Y[tt][0], Y[tt][1], Y[tt][2], Y[tt][3]};
-        } else {
+      __syncthreads();                                         // every wavefront's scores are there
+      // ---- the block's own tokens
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (p0 + i < vd) o[i] = Y[tt][i];
+      for (int tt = 0; tt < 4; ++tt) {
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+          if (2 * k > tt) continue;
+          Frag hi, lo;
+          hi.q = Mf[((tt * 2 + k) * 2) * 64 + lane];
+          lo.q = Mf[((tt * 2 + k) * 2 + 1) * 64 + lane];
+          Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xs[k].v, hi.v, Y[tt], 0, 0, 0);
+          Y[tt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xs[k].v, lo.v, Y[tt], 0, 0, 0);
+        }
+        const int t = 16 * tt + lq, p0 = blockIdx.x * 64 + 16 * wave + 4 * g4;
+        if (t < nt) {
+          float* o = out + (int64_t)(start + c0 + t) * (H * vd) + h * vd + p0;
+          if ((vd & 3) == 0) {
+            if (p0 < vd) *reinterpret_cast<float4*>(o) = float4{Y[tt][0], Y[tt][1], Y[tt][2], Y[tt][3]};
+          } else {
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+              if (p0 + i < vd) o[i] = Y[tt][i];
+          }
         }
       }
     }
@@ -252,7 +261,8 @@ __global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, con
       }
     }
   }
-  if (p >= vd) return;
+  if (ss.sum_log && blockIdx.x == 0 && threadIdx.x == 63) ss.sum_log[(int64_t)b * H + h] = (float)total;
+  if (p >= vd || !ss.keep_end) return;
 #pragma unroll
   for (int t = 0; t < NT; ++t)
 #pragma unroll
@@ -281,7 +291,7 @@ static int launch_space(SpaceArgs ss, const void* X, int64_t ldx, int G, float* 
 extern "C" int ragged_state_space_mfma(SpaceArgs ss, const void* X, int64_t ldx, int G, float* state, float* out, int H, int N, int vd,
                                        Batch bt, hipStream_t st) {
   if (bt.B <= 0 || bt.B > 65535 || H <= 0 || H > 65535 || vd <= 0 || G <= 0 || H % G || !ragged_state_space_mfma_ok(N)) return -1;
-  if (!ss.dt || !ss.dt_bias || !ss.rate || !ss.D || ss.lddt < H || ss.b0 < 0 || ss.c0 < 0 || !X || !state || !out) return -1;
+  if (!ss.dt || !ss.dt_bias || !ss.rate || !ss.D || ss.lddt < H || ss.b0 < 0 || ss.c0 < 0 || !X || !state || (!out && !ss.keep_end)) return -1;
   if (ss.b0 % 8 || ss.c0 % 8 || ldx % 8 || (uintptr_t)X % 16 || (uintptr_t)out % 16) return -1;
   if (ldx < (int64_t)H * vd || ldx < ss.b0 + (int64_t)G * N || ldx < ss.c0 + (int64_t)G * N) return -1;
 #define SP_CASE(KS) return launch_space<KS>(ss, X, ldx, G, state, out, H, N, vd, bt, st)
@@ -291,4 +301,62 @@ extern "C" int ragged_state_space_mfma(SpaceArgs ss, const void* X, int64_t ldx,
   if (N <= 128) SP_CASE(4);
   SP_CASE(8);
 #undef SP_CASE
+}
+
+// The walk over a sequence's segments: one thread per four neighbouring state elements replaces a segment's local end state in
+// `segs` [segments, H, N, vd] by its start state and leaves the last state in the sequence's slot.  A segment's decay is one number per
+// head, exp(sum_log[segment, h]).  cfirst[b] .. cfirst[b + 1] - 1 are b's segments.  V: elements per thread (a head has V * k).
+template <int V>
+__global__ __launch_bounds__(256) void space_chain_kernel(float* __restrict__ state, float* __restrict__ segs, const float* __restrict__ sum_log,
+                                                          const int* __restrict__ cfirst, const int* __restrict__ seq_past,
+                                                          const int* __restrict__ seq_slot, int H, int per_head) {
+  const int b = blockIdx.y;
+  const int64_t E = (int64_t)H * per_head, e = ((int64_t)blockIdx.x * 256 + threadIdx.x) * V;
+  if (e >= E) return;
+  const int h = (int)(e / per_head);
+  float* sp = state + (int64_t)seq_slot[b] * E + e;
+  float S[V];
+#pragma unroll
+  for (int i = 0; i < V; ++i) S[i] = seq_past[b] > 0 ? sp[i] : 0.f;
+  const int c1 = cfirst[b + 1];
+  for (int c0 = cfirst[b]; c0 < c1; c0 += 4) {
+    float loc[4][V], dec[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = c0 + u < c1 ? c0 + u : c1 - 1;
+      if (V == 4) {
+        const float4 q = *reinterpret_cast<const float4*>(segs + (int64_t)c * E + e);
+        loc[u][0] = q.x; loc[u][1 % V] = q.y; loc[u][2 % V] = q.z; loc[u][3 % V] = q.w;
+      } else {
+        loc[u][0] = segs[(int64_t)c * E + e];
+      }
+      dec[u] = sum_log[(int64_t)c * H + h];
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      if (c0 + u >= c1) break;
+      float* o = segs + (int64_t)(c0 + u) * E + e;
+      const float f = expf(dec[u]);
+      if (V == 4) *reinterpret_cast<float4*>(o) = float4{S[0], S[1 % V], S[2 % V], S[3 % V]};
+      else o[0] = S[0];
+#pragma unroll
+      for (int i = 0; i < V; ++i) S[i] = f * S[i] + loc[u][i];
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < V; ++i) sp[i] = S[i];
+}
+
+extern "C" int ragged_space_chain(float* state, float* segs, const float* sum_log, const int* cfirst, const int* seq_past, const int* seq_slot,
+                                  int B, int H, int N, int vd, hipStream_t st) {
+  if (B <= 0 || B > 65535 || H <= 0 || N <= 0 || vd <= 0 || !state || !segs || !sum_log) return -1;
+  const int64_t per_head = (int64_t)N * vd, E = per_head * H;
+  if (per_head > 0x7fffffff) return -1;
+  if (per_head % 4 == 0)
+    hipLaunchKernelGGL(space_chain_kernel<4>, dim3((unsigned)((E / 4 + 255) / 256), B), dim3(256), 0, st, state, segs, sum_log, cfirst, seq_past,
+                       seq_slot, H, (int)per_head);
+  else
+    hipLaunchKernelGGL(space_chain_kernel<1>, dim3((unsigned)((E + 255) / 256), B), dim3(256), 0, st, state, segs, sum_log, cfirst, seq_past,
+                       seq_slot, H, (int)per_head);
+  return RAGGED_LAUNCH_OK();
 }

@@ -112,7 +112,7 @@ class _GatedDeltaArgs(ctypes.Structure):
 
 class _SpaceArgs(ctypes.Structure):
     _fields_ = [("dt", ctypes.c_void_p), ("lddt", ctypes.c_int64)] + [(n, ctypes.c_void_p) for n in ("dt_bias", "rate", "D")] + \
-               [("b0", ctypes.c_int), ("c0", ctypes.c_int)]
+               [("b0", ctypes.c_int), ("c0", ctypes.c_int), ("sum_log", ctypes.c_void_p), ("keep_end", ctypes.c_int)]
 
 
 class _JoinArgs(ctypes.Structure):
@@ -150,6 +150,7 @@ def lib():
         L.ragged_gate_group_norm.argtypes = [vp, vp, i64, ci, vp, vp, i64, ci, ci, cf, ci, vp]
         L.ragged_state_space_mfma_ok.argtypes = [ci]
         L.ragged_state_space_mfma.argtypes = [_SpaceArgs, vp, i64, ci, vp, vp, ci, ci, ci, _Batch, vp]
+        L.ragged_space_chain.argtypes = [vp, vp, vp, vp, vp, vp, ci, ci, ci, ci, vp]
         L.ragged_state_space_scan.argtypes = [_SpaceArgs, vp, i64, ci, vp, vp, ci, ci, ci, _Batch, ci, vp]
         L.ragged_add_norm.argtypes = [vp, vp, vp, vp, vp, i64, ci, cf, ci, vp]
         L.ragged_act_cols.argtypes = [vp, i64, ci, vp, i64, ci, ci, cf, cf, ci, vp]
@@ -1043,6 +1044,12 @@ class HipOps:
         return q, first
 
     space_blocks_from = 16    # bfloat16 portions of at least this many tokens run the state space recurrence in blocks of 64
+    space_groups = 512        # workgroups that a walk over segments aims at (two per CU)
+
+    def _space_segment(self, meta, blocks):
+        """tokens per segment of long portions: as many segments as fill the device, none shorter than four blocks of 64"""
+        per = -(-meta.T * blocks // self.space_groups)
+        return max(256, -(-per // 64) * 64)
 
     def state_space_scan(self, X, b0, c0, P, dt0, dt_bias, rate, D, state, H, G, N, vd, meta):
         """S <- exp(-rate d) S + d B x^T, y = S^T C + D x per head (head h reads group h / (H / G)), d = softplus(dt + dt_bias): x =
@@ -1055,11 +1062,30 @@ class HipOps:
                 or max(s[0] for s in meta.seqs) >= state.shape[0]:
             raise ValueError("recurrent state / scan inputs do not fit")
         y = torch.empty(meta.T, H * vd, dtype=torch.float32, device=X.device)
-        a = _SpaceArgs(P[:, dt0:].data_ptr(), P.stride(0), dt_bias.data_ptr(), rate.data_ptr(), D.data_ptr(), b0, c0)
-        if X.dtype == torch.bfloat16 and max(n for _, _, n, _ in meta.seqs) >= self.space_blocks_from and lib().ragged_state_space_mfma_ok(N) \
+        L, st = lib(), _stream()
+        a = _SpaceArgs(P[:, dt0:].data_ptr(), P.stride(0), dt_bias.data_ptr(), rate.data_ptr(), D.data_ptr(), b0, c0, None, 1)
+        longest = max(n for _, _, n, _ in meta.seqs)
+        if X.dtype == torch.bfloat16 and longest >= self.space_blocks_from and L.ragged_state_space_mfma_ok(N) \
                 and not (b0 % 8 or c0 % 8 or X.stride(0) % 8 or X.data_ptr() % 16):
-            _ok(lib().ragged_state_space_mfma(a, X.data_ptr(), X.stride(0), G, state.data_ptr(), y.data_ptr(), H, N, vd, meta.c(), _stream()),
-                "state_space_mfma")
+            def walk(states, out, batch, what):
+                _ok(L.ragged_state_space_mfma(a, X.data_ptr(), X.stride(0), G, states.data_ptr(), None if out is None else out.data_ptr(), H, N, vd,
+                                              batch, st), what)
+            length = self._space_segment(meta, H * -(-vd // 64))
+            if longest <= length:
+                walk(state, y, meta.c(), "state_space_mfma")
+                return y
+            nc, cstart, zeros, ones, cid, cfirst, _ = meta.chunks(length)
+            segs = torch.empty(nc, H, N, vd, dtype=torch.float32, device=X.device)
+            sums = torch.empty(nc, H, dtype=torch.float32, device=X.device)
+
+            def segment_batch(past):
+                return _Batch(None, None, cstart.data_ptr(), past.data_ptr(), cid.data_ptr(), None, meta.T, nc, 0)
+            a.sum_log = sums.data_ptr()
+            walk(segs, None, segment_batch(zeros), "state_space_mfma (segments from zero)")
+            _ok(L.ragged_space_chain(state.data_ptr(), segs.data_ptr(), sums.data_ptr(), cfirst.data_ptr(), meta.seq_past.data_ptr(),
+                                     meta.seq_slot.data_ptr(), meta.B, H, N, vd, st), "space_chain")
+            a.sum_log, a.keep_end = None, 0
+            walk(segs, y, segment_batch(ones), "state_space_mfma (segments from their start states)")
             return y
         _ok(lib().ragged_state_space_scan(a, X.data_ptr(), X.stride(0), G, state.data_ptr(), y.data_ptr(), H, N, vd, meta.c(), _DT[X.dtype],
                                           _stream()), "state_space_scan")

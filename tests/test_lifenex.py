@@ -512,7 +512,7 @@ def _space_inputs(H, G, N, e, T, g, dtype):
 def test_state_space_scan_across_portions_and_in_a_used_slot(device, dtype, H, G, N, e):
     """the scan op alone against the token-by-token statement on the same (rounded) inputs: portions of 1, 2 and many tokens, a second
     sequence in a slot that the first has left, portions beside each other.  Steps are small, so that the first tokens still weigh
-    at the end.  bfloat16: long portions run in blocks of 64 on the matrix cores."""
+    at the end.  bfloat16: long portions run in blocks of 64 on the matrix cores, the longest in segments side by side."""
     g = torch.Generator().manual_seed(31)
     ops, T = R.ops_for(device), 330
     X, P, dtb, rate, D = _space_inputs(H, G, N, e, T, g, dtype)
@@ -539,7 +539,7 @@ def test_state_space_scan_across_portions_and_in_a_used_slot(device, dtype, H, G
     pool = PagedStatePool({0: [("matrix", H, N, e)]}, 64, 2, dtype, device)
     want, other = statement(0, T), statement(100, 160)
     scale, tol = float(want.abs().max()), 2e-5 if dtype == torch.float32 or device == "cpu" else 1e-4
-    for cuts in ([0, 1, 3, 40, 41, 43, 330], [0, 200, 201, 330], [0, 64, 192, 330]):
+    for cuts in ([0, 1, 3, 40, 41, 43, 330], [0, 200, 201, 330], [0, 64, 192, 330], [0, 330], [0, 5, 330]):
         slot = pool.admit()
         got = torch.cat([scan(pool, [(slot, lo, hi)]) for lo, hi in zip(cuts, cuts[1:])])
         close(got / scale, want / scale, tol)
@@ -548,7 +548,7 @@ def test_state_space_scan_across_portions_and_in_a_used_slot(device, dtype, H, G
         close(scan(pool, [(slot, 100, 160)]) / scale, other / scale, tol)
         pool.release(slot)
     a, b = pool.admit(), pool.admit()
-    got = torch.cat([scan(pool, [(a, 0, 70), (b, 100, 101)])[:70], scan(pool, [(b, 101, 160), (a, 70, 330)])[59:]])
+    got = torch.cat([scan(pool, [(a, 0, 40), (b, 100, 101)])[:40], scan(pool, [(b, 101, 160), (a, 40, 330)])[59:]])
     close(got / scale, want / scale, tol)
 
 
