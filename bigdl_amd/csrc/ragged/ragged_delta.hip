@@ -264,7 +264,7 @@ constexpr int DL_SEG = DL_DR + 4;   // LDS floats per lane group and token (padd
 constexpr int DL_TBR = 32;          // TB * R <= this
 
 template <typename T, int NW, int MODE>
-__global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __restrict__ rf, const float* __restrict__ wf,
+__global__ __launch_bounds__(64 * NW, 2) void delta_scan_kernel(const float* __restrict__ rf, const float* __restrict__ wf,
                                                          const float* __restrict__ nf, const float* __restrict__ bf,
                                                          const float* __restrict__ kf, const float* __restrict__ gb, int G,
                                                          const T* __restrict__ P, int64_t ldp, int v0,
@@ -272,7 +272,7 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
                                                          float* __restrict__ trans, int R, int TB, int values, SpaceArgs ss, Batch bt) {
   constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2, KI = MODE == DL_GENERAL ? 4 : 1;    // arrays, k's place among them
   constexpr bool GB = MODE != DL_GENERAL;                    // two scalars per token
-  constexpr int NT = 64 * NW, DL_PRE = NA * DL_TBR * DL_DR / NT;
+  constexpr int NT = 64 * NW, PRE = DL_TBR * DL_DR / NT;     // threads; elements of an array's block per thread
   extern __shared__ __attribute__((aligned(16))) float smem[];   // 2 x { r, w, n, b, k (r, k, w): [TB][R][SEG] each, v[TB][wcols], (g, beta)[TB] }
   int b = blockIdx.z;
   bool fresh = true;                                         // sequences without a past start from zero
@@ -301,72 +301,76 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
 #pragma unroll
     for (int k = 0; k < DL_DR; ++k) {
       const int row = row0 + k;
-      const float v = sp[(int64_t)(row < d ? row : d - 1) * vd + cc];    // no condition around the load
+      const float v = sp[(unsigned)((row < d ? row : d - 1) * vd + cc)];    // no condition around the load
       S[k] = ((past > 0 || !fresh) && colok && row < d) ? v : 0.f;
     }
   }
-  float pre[DL_PRE], prev[4], preg = 0.f;
-  // element e of a block = (token tk, array, row): tokens are the slowest index, so a block of few tokens (a single
-  // decoded one) ends the loops early; R * 32 is a power of two (lr = its logarithm) and NA a constant, so no step divides
-  const int lr = 31 - __clz(R * DL_DR), rows = R * DL_DR;
+  // A block's element e = (token tk, row): a token has R * 32 rows and a workgroup 2^lw columns, both powers of two, so no step
+  // divides; tokens are the slow index, so a block of few tokens (a single decoded one) ends the loops early.  Every address is a
+  // base that the workgroup shares plus a short offset.
+  const int lr = 31 - __clz(R * DL_DR), rows = 1 << lr, lw = 31 - __clz(wcols);
+  float pre[NA][PRE], prev[4], preg = 0.f;
   auto fetch = [&](int i0) {                               // block of tokens i0 .. i0 + TB - 1 into registers
-    const int live = (n - i0 < TB ? n - i0 : TB) * NA * rows;
+    const int nt = n - i0 < TB ? n - i0 : TB;
+    const int64_t t0 = start + i0;
+    const T* prow = P + t0 * ldp;
 #pragma unroll
-    for (int u = 0; u < DL_PRE; ++u) {
-      if (NT * u >= live) break;
-      const int e = tid + NT * u;
-      const int ta = e >> lr, row = e & (rows - 1);
-      const int tk = ta / NA, which = ta - tk * NA;
-      float v = NA == 5 && which == 1 ? 1.f : 0.f;         // padding: w = 1, everything else 0
-      if (e < live && row < d) {
-        const int64_t t = start + i0 + tk;
+    for (int u = 0; u < PRE; ++u) {
+      if (NT * u >= nt << lr) break;
+      const int e = tid + NT * u, tk = e >> lr, row = e & (rows - 1);
+      const bool ok = tk < nt && row < d;
+#pragma unroll
+      for (int a = 0; a < NA; ++a) {
+        float v;
         if (MODE == DL_SPACE) {
-          v = to_f(P[t * ldp + (which == 0 ? ss.c0 : ss.b0) + hd0 + row]);
-        } else if (MODE == DL_CHANNEL && which == 2) {
-          v = wf[t * (H * d) + h * d + row];
+          v = to_f((prow + (a == 0 ? ss.c0 : ss.b0) + hd0)[ok ? (unsigned)(tk * (int)ldp + row) : 0u]);
         } else {
-          const float* src = which == 0 ? rf : GB ? kf : which == 1 ? wf : which == 2 ? nf : which == 3 ? bf : kf;
-          v = src[t * HD + hd0 + row];
+          const float* src = a == 0 ? rf : MODE == DL_CHANNEL && a == 2 ? wf : GB ? kf : a == 1 ? wf : a == 2 ? nf : a == 3 ? bf : kf;
+          const int stride = MODE == DL_CHANNEL && a == 2 ? H * d : HD, first = MODE == DL_CHANNEL && a == 2 ? h * d : hd0;
+          v = (src + t0 * stride + first)[ok ? (unsigned)(tk * stride + row) : 0u];
         }
+        pre[a][u] = ok ? v : MODE == DL_GENERAL && a == 1 ? 1.f : 0.f;       // padding: w = 1, everything else 0
       }
-      pre[u] = v;
     }
-    if (GB && tid < 2 * TB && i0 + (tid >> 1) < n) {
-      const int64_t t = start + i0 + (tid >> 1);
+    if (GB && tid < 2 * TB && tid >> 1 < nt) {
       if (MODE == DL_SPACE) {
-        const float step = softplusf_(to_f(((const T*)ss.dt)[t * ss.lddt + h]) + dtb);
+        const float step = softplusf_(to_f(((const T*)ss.dt)[(t0 + (tid >> 1)) * ss.lddt + h]) + dtb);
         preg = (tid & 1) ? step : expf(-rate * step);
       } else {
-        preg = gb[(t * H + h) * 2 + (tid & 1)];
+        preg = gb[((t0 + (tid >> 1)) * H + h) * 2 + (tid & 1)];
       }
+    }
+    if (!values) {
+#pragma unroll
+      for (int u = 0; u < 4; ++u) prev[u] = 0.f;
+      return;
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      const int e = tid + NT * u;
-      float v = 0.f;
-      if (e < TB * wcols && values) {
-        const int tk = e / wcols, c = blockIdx.x * wcols + e % wcols;
-        if (i0 + tk < n && c < vd) v = to_f(P[(int64_t)(start + i0 + tk) * ldp + v0 + h * vd + c]);
-      }
-      prev[u] = v;
+      if (NT * u >= nt << lw) break;
+      const int e = tid + NT * u, tk = e >> lw, c = blockIdx.x * wcols + (e & (wcols - 1));
+      const bool ok = tk < nt && c < vd;
+      const float v = to_f((prow + v0 + h * vd)[ok ? (unsigned)(tk * (int)ldp + c) : 0u]);
+      prev[u] = ok ? v : 0.f;
     }
   };
   auto stash = [&](float* buf, int i0) {
-    const int live = (n - i0 < TB ? n - i0 : TB) * NA * rows;
+    const int nt = n - i0 < TB ? n - i0 : TB;
 #pragma unroll
-    for (int u = 0; u < DL_PRE; ++u) {
-      if (NT * u >= live) break;
-      const int e = tid + NT * u;
-      if (e < live) {
-        const int ta = e >> lr, row = e & (rows - 1);
-        const int tk = ta / NA, which = ta - tk * NA;
-        buf[which * qsz + (tk * R + (row >> 5)) * DL_SEG + (row & 31)] = pre[u];
+    for (int u = 0; u < PRE; ++u) {
+      if (NT * u >= nt << lr) break;
+      const int e = tid + NT * u, tk = e >> lr, row = e & (rows - 1);
+      if (tk < nt) {
+        float* dst = buf + (tk * R + (row >> 5)) * DL_SEG + (row & 31);
+#pragma unroll
+        for (int a = 0; a < NA; ++a) dst[a * qsz] = pre[a][u];
       }
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
+      if (NT * u >= nt << lw) break;
       const int e = tid + NT * u;
-      if (e < TB * wcols) buf[NA * qsz + e] = prev[u];
+      if (e >> lw < nt) buf[NA * qsz + e] = prev[u];
     }
     if (GB && tid < 2 * TB) buf[NA * qsz + TB * wcols + tid] = preg;
   };
@@ -457,7 +461,7 @@ __global__ __launch_bounds__(64 * NW) void delta_scan_kernel(const float* __rest
 #pragma unroll
   for (int k = 0; k < DL_DR; ++k) {
     const int row = row0 + k;
-    if (colok && row < d) sp[(int64_t)row * vd + col] = S[k];
+    if (colok && row < d) sp[(unsigned)(row * vd + col)] = S[k];
   }
 }
 
@@ -467,6 +471,7 @@ static int launch_delta_scan(const float* rf, const float* wf, const float* nf, 
                              SpaceArgs ss, Batch bt, int dtype, hipStream_t st) {
   constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2;
   if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 32 || (values && !P)) return -1;
+  if (ldp > 1 << 24 || (int64_t)d * vd > 1 << 30 || (int64_t)H * d > 1 << 24) return -1;         // (offsets inside a block and a state are 32-bit)
   if (trans && (out || !values || bt.B > 32767)) return -1;
   int R = 1;
   while (R * DL_DR < d) R <<= 1;

@@ -15,9 +15,9 @@ constexpr int MOE_SLOTS = MOE_MAX_E / 64;
 // first, with weight s * scale, or (renorm) s / (sum of the chosen s + 1e-20) * scale.  Ties go to the lower lane.
 // `corr` [E] or null: what is compared, for groups and experts alike, is s + corr (of either sign); the weights are made of s.
 // `wg` [D] or null: one more router row, gate_out[t] = sigmoid(wg . x) (how much of a shared expert a row takes).
-// One workgroup of four wavefronts per row: the wavefronts share the router's rows, wavefront 0 chooses.
-template <typename T>
-__global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x, int64_t ldx, const float* __restrict__ wr,
+// One workgroup per row: its NW wavefronts (four, or sixteen where there are few rows) share the router's rows, wavefront 0 chooses.
+template <typename T, int NW>
+__global__ __launch_bounds__(64 * NW) void moe_route_kernel(const T* __restrict__ x, int64_t ldx, const float* __restrict__ wr,
                                                         int* __restrict__ idx, float* __restrict__ wts, int D, int E, int groups,
                                                         int keep, int top, float scale, int score_fn, int group_top, int renorm,
                                                         const float* __restrict__ corr, const float* __restrict__ wg,
@@ -28,12 +28,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const T* __restrict__ x,
   extern __shared__ __attribute__((aligned(16))) float xs[];       // the row as floats
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const T* xr = x + (int64_t)t * ldx;
-  for (int c = threadIdx.x; c < D; c += 256) xs[c] = to_f(xr[c]);
+  for (int c = threadIdx.x; c < D; c += 64 * NW) xs[c] = to_f(xr[c]);
   __syncthreads();
   // two experts per wavefront and pass, 16 bytes of each router row per lane: eight loads in flight
   const bool v4 = (D & 3) == 0;
   const int rows = wg ? E + 1 : E;                          // (the row of the shared expert's gate comes last)
-  for (int e0 = 2 * wave; e0 < rows; e0 += 8) {
+  for (int e0 = 2 * wave; e0 < rows; e0 += 2 * NW) {
     const int e1 = e0 + 1 < rows ? e0 + 1 : e0;
     const float* w0 = e0 < E ? wr + (int64_t)e0 * D : wg;
     const float* w1 = e1 < E ? wr + (int64_t)e1 * D : wg;
@@ -165,8 +165,10 @@ extern "C" int ragged_moe_route(const void* x, int64_t ldx, const float* wr, int
   if (score_fn < 0 || score_fn > 1 || group_top < 1 || group_top > 2 || (renorm && top > 64)) return -1;
   if (rows <= 0 || rows > 0x7fffffff || D <= 0 || D > 12288 || E <= 0 || E > MOE_MAX_E || groups <= 0 || groups > 64 || E % groups) return -1;
   if (keep <= 0 || keep > groups || top <= 0 || top > keep * (E / groups)) return -1;
-  RAGGED_DISPATCH(dtype, hipLaunchKernelGGL((moe_route_kernel<T>), dim3((unsigned)rows), dim3(256), D * sizeof(float), st, (const T*)x, ldx, wr, idx,
-                                            wts, D, E, groups, keep, top, scale, score_fn, group_top, renorm, corr, wg, gate_out))
+#define RT_CASE(NW) hipLaunchKernelGGL((moe_route_kernel<T, NW>), dim3((unsigned)rows), dim3(64 * NW), D * sizeof(float), st, (const T*)x, ldx, wr, idx, \
+                                       wts, D, E, groups, keep, top, scale, score_fn, group_top, renorm, corr, wg, gate_out)
+  RAGGED_DISPATCH(dtype, if (rows <= 256) RT_CASE(16); else RT_CASE(4))
+#undef RT_CASE
   return RAGGED_LAUNCH_OK();
 }
 

@@ -54,7 +54,7 @@ template <int KS> struct SpaceLds {
 
 // KS: 32-row steps of the state, N <= 32 KS (rows past N are zeros)
 template <int KS>
-__global__ __launch_bounds__(256) void state_space_mfma_kernel(SpaceArgs ss, const bf16* __restrict__ X, int64_t ldx, int G,
+__global__ __launch_bounds__(256, KS <= 4 ? 2 : 1) void state_space_mfma_kernel(SpaceArgs ss, const bf16* __restrict__ X, int64_t ldx, int G,
                                                                float* __restrict__ state, float* __restrict__ out, int H, int N, int vd,
                                                                Batch bt) {
   typedef SpaceLds<KS> L;
