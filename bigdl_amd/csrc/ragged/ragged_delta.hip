@@ -241,8 +241,8 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
 
 // ---------------------------------------------------------------------------------------------------------------
 // The scan.  Columns of S are independent: column j follows s <- w * s - b (n . s) + k v_j, and its output is r . s.
-// A wavefront owns 64 / R columns; R neighbouring lanes share a column, lane r of them holds rows 32 r .. 32 r + 31 in
-// registers (R = d / 32 rounded up to a power of two; rows past d carry w = 1 and zeros and stay zero), so a token costs
+// A wavefront owns 64 / R columns; R neighbouring lanes share a column, lane r of them holds rows 16 r .. 16 r + 15 in
+// registers (R = d / 16 rounded up to a power of two; rows past d carry w = 1 and zeros and stay zero), so a token costs
 // two cross-lane sums of R partial products (DPP moves): n . s before the update, r . s after it.  A workgroup is NW such
 // wavefronts (as many as the state has columns for, at most four: a wavefront without columns would still read all five
 // arrays).  The five arrays of a block of TB tokens are brought into LDS by the whole workgroup with coalesced loads
@@ -259,9 +259,9 @@ extern "C" int ragged_gated_delta_prep(GatedDeltaArgs a, Batch bt, int dtype, hi
 //            decay and step size per head come from its step logit (`ss`), the read-out takes D v on top.
 enum DeltaMode { DL_GENERAL, DL_GATED, DL_CHANNEL, DL_SPACE };
 
-constexpr int DL_DR = 32;
+constexpr int DL_DR = 16;
 constexpr int DL_SEG = DL_DR + 4;   // LDS floats per lane group and token (padding shifts the banks between groups)
-constexpr int DL_TBR = 32;          // TB * R <= this
+constexpr int DL_TBR = 64;          // TB * R <= this
 
 template <typename T, int NW, int MODE>
 __global__ __launch_bounds__(64 * NW, 2) void delta_scan_kernel(const float* __restrict__ rf, const float* __restrict__ wf,
@@ -305,7 +305,7 @@ __global__ __launch_bounds__(64 * NW, 2) void delta_scan_kernel(const float* __r
       S[k] = ((past > 0 || !fresh) && colok && row < d) ? v : 0.f;
     }
   }
-  // A block's element e = (token tk, row): a token has R * 32 rows and a workgroup 2^lw columns, both powers of two, so no step
+  // A block's element e = (token tk, row): a token has R * 16 rows and a workgroup 2^lw columns, both powers of two, so no step
   // divides; tokens are the slow index, so a block of few tokens (a single decoded one) ends the loops early.  Every address is a
   // base that the workgroup shares plus a short offset.
   const int lr = 31 - __clz(R * DL_DR), rows = 1 << lr, lw = 31 - __clz(wcols);
@@ -361,7 +361,7 @@ __global__ __launch_bounds__(64 * NW, 2) void delta_scan_kernel(const float* __r
       if (NT * u >= nt << lr) break;
       const int e = tid + NT * u, tk = e >> lr, row = e & (rows - 1);
       if (tk < nt) {
-        float* dst = buf + (tk * R + (row >> 5)) * DL_SEG + (row & 31);
+        float* dst = buf + (tk * R + row / DL_DR) * DL_SEG + row % DL_DR;
 #pragma unroll
         for (int a = 0; a < NA; ++a) dst[a * qsz] = pre[a][u];
       }
@@ -470,7 +470,7 @@ static int launch_delta_scan(const float* rf, const float* wf, const float* nf, 
                              const void* P, int64_t ldp, int v0, float* state, float* out, int H, int d, int vd, int values, float* trans,
                              SpaceArgs ss, Batch bt, int dtype, hipStream_t st) {
   constexpr int NA = MODE == DL_GENERAL ? 5 : MODE == DL_CHANNEL ? 3 : 2;
-  if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 32 || (values && !P)) return -1;
+  if (bt.B <= 0 || H <= 0 || d <= 0 || vd <= 0 || d > DL_DR * 64 || (values && !P)) return -1;
   if (ldp > 1 << 24 || (int64_t)d * vd > 1 << 30 || (int64_t)H * d > 1 << 24) return -1;         // (offsets inside a block and a state are 32-bit)
   if (trans && (out || !values || bt.B > 32767)) return -1;
   int R = 1;

@@ -853,18 +853,20 @@ class HipOps:
     delta_chunked_from = 192  # portions of at least this many tokens run the delta rule in chunks
     delta_chain = True        # False: the walk over a sequence's chunks as library products (what very tall states get)
 
+    delta_resident = 1024     # workgroups of the scan that run at one time (four per CU)
+
     def _delta_chunk_length(self, meta, H, d, vd):
         """Tokens per chunk of a long delta-rule scan: three passes of (rounds of resident workgroups) x (chunk tokens) token
-        steps in a row, plus the walk over a sequence's chunks (about two token steps per chunk)."""
+        steps in a row, plus the walk over a sequence's chunks (about four token steps per chunk)."""
         R = 1
-        while R * 32 < d:
+        while R * 16 < d:
             R *= 2
         best = None
         for length in (128, 96, 64, 48, 32):
             chunks = [-(-n // length) for _, _, n, _ in meta.seqs]
             cols = 64 // R                                   # columns of a wavefront; a workgroup is two or four of them
             blocks = -(-max(vd, d) // ((2 if max(vd, d) <= 2 * cols else 4) * cols))
-            cost = 3 * -(-(sum(chunks) * H * blocks) // self.scan_resident) * length + 2 * max(chunks)
+            cost = 3 * -(-(sum(chunks) * H * blocks) // self.delta_resident) * length + 4 * max(chunks)
             if best is None or cost < best[0]:
                 best = (cost, length)
         return best[1]
