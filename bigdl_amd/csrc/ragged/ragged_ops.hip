@@ -2,7 +2,7 @@
 // state + per-head norm + rotary + paged append, clamped gated activation, HGRN2 gates / scan / output norm, the stream
 // updates of the sandwich, parallel and sequential pre-norm blocks (the last over several copies of the stream) and of the
 // output-norm block (LayerNorm on a sublayer's result, causal convolution of the stream in front of the next mixer),
-// embedding rows, activations of dense feed-forwards, gates per channel.
+// embedding rows, activations of dense feed-forwards, gates per channel, the stream's update of parallel blocks with two norms.
 // gfx950, wave64.  Everything that the engine keeps in 32 bits (residual, norms, angles, gates, recurrent state) is
 // float here whatever the activation type T is.
 #include "ragged_common.h"

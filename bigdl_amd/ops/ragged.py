@@ -300,7 +300,8 @@ class BatchMeta:
 
 
 def _stream():
-    return torch.cuda.current_stream().cuda_stream
+    """PyTorch's current stream as a raw handle (without building the stream object: every launch asks)"""
+    return torch._C._cuda_getCurrentRawStream(torch._C._cuda_getDevice())
 
 
 def _ok(rc, what):
