@@ -800,7 +800,8 @@ class HipOps:
             raise ValueError("(gate, up) pairs expected")
         out = torch.empty(P.shape[0], P.shape[1] // 2, dtype=P.dtype, device=P.device)
         if out.numel():
-            _ok(lib().ragged_glu_pairs(P.data_ptr(), P.stride(0), None if row_gate is None else row_gate.data_ptr(), out.data_ptr(), P.shape[0], P.shape[1] // 2, _DT[P.dtype], _stream()),
+            _ok(lib().ragged_glu_pairs(P.data_ptr(), P.stride(0), None if row_gate is None else row_gate.data_ptr(), out.data_ptr(),
+                                       P.shape[0], P.shape[1] // 2, _DT[P.dtype], _stream()),
                 "glu_pairs")
         return out
 
@@ -1024,8 +1025,8 @@ class HipOps:
                  want_first=False, head_norms=False, q_temp=None):
         """Columns q [H d] | k [G d] | v [G vd] of P: q and k RMS-normed over the whole projection with a weight per channel, the
         first ``rot`` channels of every head turned (pairs i, i + rot / 2); ``head_norms``: every head normed by itself with a weight of
-        d channels that all heads share; ``q_temp`` = (coef, every): queries times 1 + coef ln(floor((pos + 1) / every) + 1); values RMS-normed per head (``v_norm``) and mixed with
-        ``first_in`` [T, G vd] as (1 - lam) v + lam first.  Keys and values go to their pages; returns (q float [T, H d], the
+        d channels that all heads share; ``q_temp`` = (coef, every): queries times 1 + coef ln(floor((pos + 1) / every) + 1);
+        values RMS-normed per head (``v_norm``) and mixed with ``first_in`` [T, G vd] as (1 - lam) v + lam first.  Keys and values go to their pages; returns (q float [T, H d], the
         values as float if ``want_first`` else None)."""
         _act(P, kpages, vpages)
         _f32(qw, kw, inv_freq, first_in)
@@ -1498,7 +1499,8 @@ class TorchOps:
         nq, nk = H * d, G * d
         rms = lambda v: v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)       # noqa: E731
         if head_norms:
-            qk = torch.cat([(rms(u[:, :nq].reshape(-1, H, d)) * qw).reshape(-1, nq), (rms(u[:, nq:nq + nk].reshape(-1, G, d)) * kw).reshape(-1, nk)], 1)
+            qk = torch.cat([(rms(u[:, :nq].reshape(-1, H, d)) * qw).reshape(-1, nq),
+                            (rms(u[:, nq:nq + nk].reshape(-1, G, d)) * kw).reshape(-1, nk)], 1)
         else:
             qk = torch.cat([rms(u[:, :nq]) * qw, rms(u[:, nq:nq + nk]) * kw], 1).contiguous()
         if q_temp:
